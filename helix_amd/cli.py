@@ -50,19 +50,26 @@ def runner(api_url: str = typer.Option("http://localhost:8080"),
            tunnel: bool = typer.Option(False, "--tunnel",
                                        help="reverse-dial (NAT-friendly): "
                                             "no inbound port needed"),
-           preload: str = typer.Option("", help="comma-separated models")):
+           preload: str = typer.Option("", help="comma-separated models or "
+                                                "checkpoint folders")):
     """Start a GPU runner: OpenAI-compatible server + heartbeat."""
     import threading
 
     import uvicorn
     from helix_amd.runner.heartbeat import heartbeat_loop
     from helix_amd.runner.http import create_runner_app
-    from helix_amd.runner.service import RunnerService
+    from helix_amd.models import registry
+    from helix_amd.runner.service import ModelSpec, RunnerService
     from helix_amd.server.config import load_config
     cfg = load_config()
     svc = RunnerService(device=device)
     for m in filter(None, preload.split(",")):
-        svc.ensure_loaded(m.strip())
+        m = m.strip()
+        if registry.is_folder(m):          # serve a checkpoint folder
+            name = os.path.basename(os.path.normpath(m))
+            svc.register_spec(ModelSpec(name, "llm", m))
+            m = name
+        svc.ensure_loaded(m)
     api = create_runner_app(svc, runner_id)
     if tunnel:
         addr = f"tunnel:{runner_id}"
@@ -472,6 +479,51 @@ def doctor():
         check("torch.distributed nccl (RCCL)",
               dist.is_nccl_available())
     raise typer.Exit(0 if ok else 1)
+
+
+@app.command()
+def generate(prompt: str = typer.Argument(..., help="text, or token ids "
+                                                    "with --ids"),
+             model: str = typer.Option("llama3-8b", "-m", "--model",
+                                       help="preset or checkpoint folder"),
+             max_tokens: int = typer.Option(64),
+             temperature: float = typer.Option(0.0),
+             top_p: float = typer.Option(1.0),
+             seed: int = typer.Option(0),
+             ids: bool = typer.Option(False, "--ids",
+                                      help="read and print token ids"),
+             dtype: str = typer.Option("bfloat16"),
+             device: str = typer.Option("cuda:0")):
+    """Generate once with a local engine (no server)."""
+    from helix_amd.engine.engine import EngineConfig, LLMEngine
+    from helix_amd.engine.sampling_params import SamplingParams
+    from helix_amd.utils.tokenizer import get_tokenizer
+    tok = None if ids else get_tokenizer()
+    tokens = [int(t) for t in prompt.replace(",", " ").split()] if ids \
+        else tok.encode(prompt, add_bos=True)
+    length = -(-(len(tokens) + max_tokens + 1) // 16) * 16
+    eng = LLMEngine(EngineConfig(
+        model=model, max_num_seqs=1, max_model_len=length, dtype=dtype,
+        kv_cache_blocks=length // 16 + 1, seed=seed,
+        eos_token_id=-1 if ids else tok.eos_token_id), device=device)
+    out = eng.generate([tokens], SamplingParams(
+        temperature=temperature, top_p=top_p, max_tokens=max_tokens,
+        seed=seed))[0]
+    typer.echo(" ".join(map(str, out)) if ids else tok.decode(out))
+
+
+@app.command("trace-run")
+def trace_run(model: str = typer.Option(..., help="checkpoint folder"),
+              out: str = typer.Option(..., help="folder for the logits"),
+              max_tokens: int = typer.Option(...),
+              dtype: str = typer.Option("bfloat16"),
+              device: str = typer.Option("cuda:0")):
+    """Replay token steps from standard input and write logits
+    (bin/trace_run is the same program)."""
+    from helix_amd.engine import replay
+    raise typer.Exit(replay.main(
+        ["--model", model, "--out", out, "--max-tokens", str(max_tokens),
+         "--dtype", dtype, "--device", device]))
 
 
 @app.command("export-gguf")

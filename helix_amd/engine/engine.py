@@ -20,8 +20,8 @@ import torch
 from helix_amd import ops
 from helix_amd.engine.kv_cache import KVCache, chain_hash
 from helix_amd.engine.sampling_params import SamplingParams
-from helix_amd.models.llama import (DecodeMeta, LlamaConfig, LlamaForCausalLM,
-                                    PrefillMeta, PRESETS)
+from helix_amd.models import registry
+from helix_amd.models.meta import DecodeMeta, MixedMeta, PrefillMeta
 
 _SEED_MIX = 0x9E3779B97F4A7C15
 
@@ -57,10 +57,25 @@ class Sequence:
     def total_len(self) -> int:
         return len(self.prompt_ids) + len(self.output_ids)
 
+    @property
+    def last_token(self) -> int:
+        return self.output_ids[-1] if self.output_ids \
+            else self.prompt_ids[-1]
+
+
+@dataclass
+class Span:
+    """Tokens [start, end) of a sequence, run in one step; ids are the
+    token ids themselves. The cache holds everything before start."""
+    seq: Sequence
+    start: int
+    end: int
+    ids: List[int]
+
 
 @dataclass
 class EngineConfig:
-    model: str = "llama3-8b"
+    model: str = "llama3-8b"                  # preset or checkpoint folder
     block_size: int = 16
     max_num_seqs: int = 64
     max_model_len: int = 8192
@@ -73,46 +88,56 @@ class EngineConfig:
     enable_prefix_caching: bool = True
     quantization: Optional[str] = None        # None | "fp8" (e4m3 W8A8)
     kv_cache_dtype: str = "bf16"              # "bf16" | "fp8" (e4m3 KV)
+    dtype: str = "bfloat16"                   # "bfloat16" | "float32"
+    mixed_steps: bool = False                 # decode beside prompt portions
 
 
 class LLMEngine:
     def __init__(self, cfg: EngineConfig, device: str = "cuda",
-                 model: Optional[LlamaForCausalLM] = None,
+                 model: Optional[torch.nn.Module] = None,
                  tp_size: int = 1, tp_rank: int = 0,
                  tp_group=None):
         self.cfg = cfg
         self.device = torch.device(device)
-        self.model_cfg: LlamaConfig = PRESETS[cfg.model]
+        self.model_cfg = model.cfg if model is not None \
+            else registry.get_config(cfg.model)
         self.tp_size = tp_size
         self.tp_rank = tp_rank
         self.tp_group = tp_group
+        self.dtype = {"bfloat16": torch.bfloat16,
+                      "float32": torch.float32}[cfg.dtype]
+        cls = registry.model_class(self.model_cfg)
+        if cls.paged_prefill:
+            if cfg.quantization or cfg.kv_cache_dtype != "bf16":
+                raise ValueError(f"{cfg.model}: quantized weights and KV "
+                                 "caches are not available for this model")
+            if cfg.block_size % 8:
+                raise ValueError("block_size must be a multiple of 8")
+        elif self.dtype != torch.bfloat16:
+            raise ValueError(f"{cfg.model} is served in bfloat16")
         if model is None:
-            dtype = torch.bfloat16
-            model = LlamaForCausalLM(self.model_cfg, tp_size, tp_rank)
-            model = model.to(dtype).to(self.device)
-            model.init_random(cfg.seed)
+            model = registry.build_model(cfg.model, self.dtype, self.device,
+                                         cfg.seed, tp_size, tp_rank,
+                                         cfg=self.model_cfg)
         if cfg.quantization == "fp8":
             from helix_amd.models.quant import quantize_model_fp8
             quantize_model_fp8(model)
         self.model = model
 
-        nkv = self.model_cfg.num_kv_heads // tp_size
+        kv_layers = self.model_cfg.kv_layers(tp_size)
+        kv_dtype = torch.uint8 if cfg.kv_cache_dtype == "fp8" else self.dtype
         num_blocks = cfg.kv_cache_blocks
         if num_blocks is None:
-            num_blocks = self._auto_kv_blocks(nkv)
-        kv_dtype = torch.uint8 if cfg.kv_cache_dtype == "fp8" \
-            else torch.bfloat16
-        self.kv = KVCache(self.model_cfg.num_layers, nkv,
-                          self.model_cfg.head_dim, cfg.block_size, num_blocks,
-                          self.device, dtype=kv_dtype)
+            num_blocks = self._auto_kv_blocks(kv_layers, kv_dtype)
+        self.kv = KVCache.for_layers(kv_layers, cfg.block_size, num_blocks,
+                                     self.device, dtype=kv_dtype)
         self.waiting: List[Sequence] = []
         self.running: List[Sequence] = []
         self.seqs: Dict[str, Sequence] = {}
         self.steps = 0
         if self.device.type == "cuda":
-            self.decode_ws = ops.decode_workspace(
-                cfg.max_num_seqs, self.model_cfg.num_heads // tp_size,
-                self.model_cfg.head_dim, cfg.max_model_len, self.device)
+            self.decode_ws = self.model.decode_workspace(
+                cfg.max_num_seqs, cfg.max_model_len, self.device)
         else:
             self.decode_ws = None
         # GPU penalty tables (lazy): [max_num_seqs, V] output counts +
@@ -158,16 +183,16 @@ class LLMEngine:
                 self.device)
 
     # ------------------------------------------------------------------
-    def _auto_kv_blocks(self, nkv: int) -> int:
+    def _auto_kv_blocks(self, kv_layers, kv_dtype) -> int:
         if self.device.type != "cuda":
             return 512
         free, total = torch.cuda.mem_get_info(self.device)
         budget = int(total * self.cfg.gpu_memory_utilization
                      - (total - free))
+        budget -= self.model_cfg.activation_bytes(self.cfg.max_prefill_tokens)
         budget = max(budget, 1 << 28)
-        n = KVCache.blocks_for_bytes(budget, self.model_cfg.num_layers, nkv,
-                                     self.model_cfg.head_dim,
-                                     self.cfg.block_size)
+        n = KVCache.blocks_for_bytes(budget, 0, 0, 0, self.cfg.block_size,
+                                     kv_dtype, kv_layers)
         # cap: max_num_seqs sequences of max_model_len
         cap = (self.cfg.max_num_seqs *
                (self.cfg.max_model_len // self.cfg.block_size + 1))
@@ -215,9 +240,12 @@ class LLMEngine:
     # ------------------------------------------------------------------
     def step(self) -> List[tuple]:
         """Run one engine iteration. Returns [(seq, token_id, finished)]."""
+        decode = []
+        if self.cfg.mixed_steps and self.running:
+            decode = self._schedule_decode()
         prefill_batch = self._schedule_prefill()
-        if prefill_batch:
-            out = self._run_prefill(prefill_batch)
+        if prefill_batch or decode:
+            out = self._run_prefill(prefill_batch, decode)
         elif self.running:
             out = self._run_decode()
         else:
@@ -317,39 +345,136 @@ class LLMEngine:
             seq.row = -1
         seq.pen_init = False
 
-    def _run_prefill(self, batch: List[Sequence]):
-        bs = self.cfg.block_size
-        input_ids, positions, slots, cu_q, cu_k = [], [], [], [0], [0]
-        gather_blk, gather_off = [], []
-        targets = getattr(self, "_chunk_target", {})
-        any_cached = any(s.cached_prefix for s in batch)
-        for seq in batch:
-            L = targets.get(seq.seq_id, len(seq.prompt_ids))
-            P = seq.cached_prefix
-            input_ids.extend(seq.prompt_ids[P:L])
-            positions.extend(range(P, L))
-            slots.extend(self._slot(seq, p) for p in range(P, L))
-            cu_q.append(cu_q[-1] + L - P)
-            cu_k.append(cu_k[-1] + L)
-            if any_cached:
-                for p in range(L):
-                    gather_blk.append(seq.block_table[p // bs])
-                    gather_off.append(p % bs)
+    def _prefill_meta(self, spans: List[Span]) -> PrefillMeta:
+        """Host-side batch of prompt portions."""
+        bs, dev = self.cfg.block_size, self.device
+        starts = np.array([s.start for s in spans], dtype=np.int64)
+        ends = np.array([s.end for s in spans], dtype=np.int64)
+        lens = ends - starts
+        rows = np.array([s.seq.row for s in spans], dtype=np.intp)
+        which = np.repeat(np.arange(len(spans)), lens)
+        cu_q = np.concatenate([[0], np.cumsum(lens)])
+        pos = np.arange(cu_q[-1]) - np.repeat(cu_q[:-1] - starts, lens)
+        slots = self._bt_np[rows[which], pos // bs].astype(np.int64) * bs \
+            + pos % bs
+
+        def dev_t(a, dtype):
+            return torch.from_numpy(
+                np.ascontiguousarray(a, dtype=dtype)).to(dev)
+
+        meta = PrefillMeta(cu_seqlens=dev_t(cu_q, np.int32),
+                           max_seqlen=int(lens.max()),
+                           slot_mapping=dev_t(slots, np.int64),
+                           positions=dev_t(pos, np.int64),
+                           max_len=int(ends.max()))
+        if self.model.paged_prefill:
+            nb = -(-meta.max_len // bs)
+            meta.block_tables = dev_t(self._bt_np[rows, :nb], np.int32)
+            meta.seq_lens = dev_t(ends, np.int32)
+            meta.row_seq = dev_t(which, np.int32)
+            meta.row_len = dev_t(pos + 1, np.int32)
+        elif starts.any():
+            # cached prefixes: gather the full context of every sequence
+            cu_k = np.concatenate([[0], np.cumsum(ends)])
+            kwhich = np.repeat(np.arange(len(spans)), ends)
+            kpos = np.arange(cu_k[-1]) - np.repeat(cu_k[:-1], ends)
+            meta.cu_seqlens_k = dev_t(cu_k, np.int32)
+            meta.gather_blk = dev_t(self._bt_np[rows[kwhich], kpos // bs],
+                                    np.int64)
+            meta.gather_off = dev_t(kpos % bs, np.int64)
+        return meta
+
+    def _fill_decode(self, spans: List[Span]) -> int:
+        """Stage single-token spans into the persistent host arrays."""
+        for i, s in enumerate(spans):
+            self._ids_np[i] = s.ids[0]
+            self._pos_np[i] = s.start
+            self._slots_np[i] = self._slot(s.seq, s.start)
+            self._lens_np[i] = s.start + 1
+            self._rows_np[i] = s.seq.row
+        return len(spans)
+
+    def _decode_tables(self, B: int):
+        max_len = int(self._lens_np[:B].max())
+        nb = (max_len - 1) // self.cfg.block_size + 1
+        # one C-speed gather of the persistent rows (no per-row tensors)
+        return self._bt_np[self._rows_np[:B], :nb], max_len
+
+    def _decode_meta(self, B: int) -> DecodeMeta:
+        bt_np, max_len = self._decode_tables(B)
         dev = self.device
-        meta = PrefillMeta(
-            cu_seqlens=torch.tensor(cu_q, dtype=torch.int32, device=dev),
-            max_seqlen=max(targets.get(s.seq_id, len(s.prompt_ids))
-                           - s.cached_prefix for s in batch),
-            slot_mapping=torch.tensor(slots, dtype=torch.int64, device=dev),
-            positions=torch.tensor(positions, dtype=torch.int64, device=dev),
-            cu_seqlens_k=(torch.tensor(cu_k, dtype=torch.int32, device=dev)
-                          if any_cached else None),
-            gather_blk=(torch.tensor(gather_blk, dtype=torch.int64,
-                                     device=dev) if any_cached else None),
-            gather_off=(torch.tensor(gather_off, dtype=torch.int64,
-                                     device=dev) if any_cached else None))
-        ids = torch.tensor(input_ids, dtype=torch.int64, device=dev)
+        return DecodeMeta(
+            block_tables=torch.from_numpy(bt_np).to(dev),
+            seq_lens=torch.from_numpy(self._lens_np[:B].copy()).to(dev),
+            slot_mapping=torch.from_numpy(self._slots_np[:B].copy()).to(dev),
+            positions=torch.from_numpy(self._pos_np[:B].copy()).to(dev),
+            max_len=max_len, workspace=self.decode_ws)
+
+    def _decode_logits(self, B: int) -> torch.Tensor:
+        """One decode step over the B staged rows -> logits [B, V]."""
+        if self.graph_runner is not None:
+            bt_np, max_len = self._decode_tables(B)
+            return self.graph_runner.run(
+                self._ids_np[:B], self._pos_np[:B], self._slots_np[:B],
+                bt_np, self._lens_np[:B], max_len)
+        meta = self._decode_meta(B)
+        ids = torch.from_numpy(self._ids_np[:B].copy()).to(self.device)
+        return self.model.compute_logits(
+            self.model(ids, self.kv.caches, meta))
+
+    def run_spans(self, spans: List[Span],
+                  want: List[List[int]]) -> Optional[torch.Tensor]:
+        """The model step: run all spans as one batch (prompt portions
+        beside single decoded tokens) over the paged cache. Pages must be
+        allocated. Returns the logits of the places want[i] of each span i,
+        in that order, or None when nothing is wanted."""
+        dev = self.device
+        single = [i for i, s in enumerate(spans) if s.end - s.start == 1]
+        several = [i for i, s in enumerate(spans) if s.end - s.start > 1]
+        order = single + several
+        first = {}
+        at = 0
+        for i in order:
+            first[i] = at
+            at += spans[i].end - spans[i].start
+        rows = [first[i] + w for i in range(len(spans)) for w in want[i]]
+        B = self._fill_decode([spans[i] for i in single])
+        if not several:
+            logits = self._decode_logits(B)
+            if not rows:
+                return None
+            if rows == list(range(B)):
+                return logits
+            return logits[torch.tensor(rows, dtype=torch.int64, device=dev)]
+        meta = self._prefill_meta([spans[i] for i in several])
+        if single:
+            dmeta = self._decode_meta(B)
+            meta = MixedMeta(
+                decode=dmeta, prefill=meta, num_decode=B,
+                slot_mapping=torch.cat([dmeta.slot_mapping,
+                                        meta.slot_mapping]),
+                positions=torch.cat([dmeta.positions, meta.positions]))
+        ids = torch.tensor([t for i in order for t in spans[i].ids],
+                           dtype=torch.int64, device=dev)
         hidden = self.model(ids, self.kv.caches, meta)
+        if not rows:
+            return None
+        return self.model.compute_logits(
+            hidden[torch.tensor(rows, dtype=torch.int64, device=dev)])
+
+    def _run_prefill(self, batch: List[Sequence],
+                     decode: List[Sequence] = ()):
+        """Prefill the scheduled portions, beside the decode rows of a mixed
+        step."""
+        bs = self.cfg.block_size
+        targets = getattr(self, "_chunk_target", {})
+        spans = [Span(s, s.total_len - 1, s.total_len, [s.last_token])
+                 for s in decode]
+        for s in batch:
+            end = targets.get(s.seq_id, len(s.prompt_ids))
+            spans.append(Span(s, s.cached_prefix, end,
+                              s.prompt_ids[s.cached_prefix:end]))
+        logits = self.run_spans(spans, [[len(s.ids) - 1] for s in spans])
         # register this batch's newly COMPLETED full blocks in the
         # prefix cache (partial chunks register only what they wrote)
         if self.cfg.enable_prefix_caching:
@@ -360,13 +485,10 @@ class LLMEngine:
                 for i in range(start, end):
                     self.kv.allocator.register_hash(seq.block_table[i],
                                                     seq.block_hashes[i])
-        last_rows = torch.tensor([c - 1 for c in cu_q[1:]], dtype=torch.int64,
-                                 device=dev)
-        logits = self.model.compute_logits(hidden[last_rows])
-        tokens = self._sample(batch, logits)
+        tokens = self._sample([s.seq for s in spans], logits)
         now = time.monotonic()
-        out = []
-        for seq, tok in zip(batch, tokens):
+        out = list(zip(decode, tokens))
+        for seq, tok in zip(batch, tokens[len(decode):]):
             T = targets.get(seq.seq_id, len(seq.prompt_ids))
             if T < len(seq.prompt_ids):
                 seq.cached_prefix = T      # partial chunk: KV written,
@@ -376,6 +498,55 @@ class LLMEngine:
             self.running.append(seq)
             out.append((seq, tok))
         return out
+
+    # ------------------------------------------------------------------
+    def extend(self, entries: List[tuple]) -> Optional[torch.Tensor]:
+        """Run given tokens instead of sampled ones: entries are (seq_id,
+        token ids, wanted places). A sequence is admitted at its first
+        entry and goes on where its last one ended; all entries are one
+        batch of the generation path (run_spans). Returns the wanted
+        logits. release() gives a sequence's pages and row back."""
+        bs = self.cfg.block_size
+        vocab = self.model_cfg.vocab_size
+        for sid, ids, want in entries:
+            if not ids or not all(0 <= t < vocab for t in ids):
+                raise ValueError(f"{sid}: no tokens, or outside the "
+                                 f"vocabulary of {vocab}")
+            if not all(0 <= w < len(ids) for w in want):
+                raise ValueError(f"{sid}: wanted place outside the entry")
+        if len({sid for sid, _, _ in entries}) != len(entries):
+            raise ValueError("one entry per sequence and step")
+        spans = []
+        for sid, ids, _ in entries:
+            seq = self.seqs.get(sid)
+            if seq is None:
+                if not self._free_rows:
+                    raise RuntimeError(
+                        f"more than {self.cfg.max_num_seqs} live sequences")
+                seq = Sequence(sid, [], SamplingParams(),
+                               status=SeqStatus.RUNNING)
+                self.seqs[sid] = seq
+            start, end = seq.total_len, seq.total_len + len(ids)
+            if end > self.cfg.max_model_len:
+                raise ValueError(f"{sid}: {end} tokens > max_model_len "
+                                 f"{self.cfg.max_model_len}")
+            need = (end + bs - 1) // bs - len(seq.block_table)
+            if need > 0:
+                seq.block_table.extend(self.kv.allocator.allocate(need))
+            self._assign_row(seq)
+            seq.prompt_ids.extend(ids)
+            spans.append(Span(seq, start, end, list(ids)))
+        logits = self.run_spans(spans, [list(w) for _, _, w in entries])
+        self.steps += 1
+        return logits
+
+    def release(self, seq_id: str):
+        """End a sequence that extend() admitted."""
+        seq = self.seqs.pop(seq_id)
+        self.kv.allocator.free(seq.block_table)
+        seq.block_table = []
+        self._release_row(seq)
+        seq.status = SeqStatus.FINISHED
 
     def _preempt_for_blocks(self):
         """Free KV by preempting the most recent running sequence back to
@@ -404,14 +575,12 @@ class LLMEngine:
         self.waiting.insert(0, victim)
         return victim
 
-    def _run_decode(self):
+    def _schedule_decode(self) -> List[Sequence]:
+        """Running sequences with a page for their next token; preempts
+        when the pool is exhausted."""
         bs = self.cfg.block_size
-        dev = self.device
         batch = []
         preempted = set()                     # ids preempted this step
-        nb_ = 0
-        ids_np, pos_np = self._ids_np, self._pos_np
-        slots_np, lens_np, rows_np = self._slots_np, self._lens_np, self._rows_np
         for seq in list(self.running):
             if seq.seq_id in preempted:
                 continue
@@ -430,38 +599,17 @@ class LLMEngine:
                 seq.block_table.extend(self.kv.allocator.allocate(1))
                 self._bt_np[seq.row, len(seq.block_table) - 1] = \
                     seq.block_table[-1]
-            if seq.seq_id in preempted:
-                continue
-            batch.append(seq)
-            ids_np[nb_] = (seq.output_ids[-1] if seq.output_ids
-                           else seq.prompt_ids[-1])
-            pos_np[nb_] = pos
-            slots_np[nb_] = self._slot(seq, pos)
-            lens_np[nb_] = pos + 1
-            rows_np[nb_] = seq.row
-            nb_ += 1
+            if seq.seq_id not in preempted:
+                batch.append(seq)
+        return [s for s in batch if s.seq_id not in preempted]
+
+    def _run_decode(self):
+        batch = self._schedule_decode()
         if not batch:
             return []
-        B = nb_
-        max_blocks = max(len(s.block_table) for s in batch)
-        # one C-speed gather of the persistent rows (no per-row tensors)
-        bt_np = self._bt_np[rows_np[:B], :max_blocks]
-        max_len = int(lens_np[:B].max())
-        if self.graph_runner is not None:
-            logits = self.graph_runner.run(ids_np[:B], pos_np[:B],
-                                           slots_np[:B], bt_np,
-                                           lens_np[:B], max_len)
-        else:
-            meta = DecodeMeta(
-                block_tables=torch.from_numpy(bt_np).to(dev),
-                seq_lens=torch.from_numpy(lens_np[:B].copy()).to(dev),
-                slot_mapping=torch.from_numpy(slots_np[:B].copy()).to(dev),
-                positions=torch.from_numpy(pos_np[:B].copy()).to(dev),
-                max_len=max_len,
-                workspace=self.decode_ws)
-            ids = torch.from_numpy(ids_np[:B].copy()).to(dev)
-            hidden = self.model(ids, self.kv.caches, meta)
-            logits = self.model.compute_logits(hidden)
+        spans = [Span(s, s.total_len - 1, s.total_len, [s.last_token])
+                 for s in batch]
+        logits = self._decode_logits(self._fill_decode(spans))
         tokens = self._sample(batch, logits)
         return list(zip(batch, tokens))
 

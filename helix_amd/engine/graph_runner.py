@@ -59,7 +59,7 @@ class CUDAGraphRunner:
         return min(b, self.max_model_len)
 
     def _capture(self, nb: int, lb: int) -> dict:
-        from helix_amd.models.llama import DecodeMeta
+        from helix_amd.models.meta import DecodeMeta
         meta = DecodeMeta(
             block_tables=self.in_bt[:nb],
             seq_lens=self.in_lens[:nb],

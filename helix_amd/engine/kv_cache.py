@@ -7,9 +7,11 @@ free-HBM at model load (see engine.scheduler for the multi-model packer).
 from __future__ import annotations
 
 import hashlib
-from typing import Dict, List, Optional, Tuple
+from typing import Dict, List, Optional, Sequence
 
 import torch
+
+from helix_amd.models.meta import KVLayer
 
 
 def chain_hash(prev: bytes, tokens: List[int]) -> bytes:
@@ -106,30 +108,45 @@ class BlockAllocator:
 
 
 class KVCache:
-    """Per-model paged KV storage: one (K, V) pair of
-    [num_blocks, Hkv, block_size, head_dim] bf16 tensors per layer."""
+    """Per-model paged KV storage: one (K, V) pair of page tensors per
+    layer. Uniform models have K and V as [num_blocks, Hkv, block_size,
+    head_dim]; `layers` gives each layer its own geometry (KVLayer)."""
 
     def __init__(self, num_layers: int, num_kv_heads: int, head_dim: int,
-                 block_size: int, num_blocks: int, device, dtype=torch.bfloat16):
+                 block_size: int, num_blocks: int, device,
+                 dtype=torch.bfloat16,
+                 layers: Optional[Sequence[KVLayer]] = None):
+        if layers is None:
+            layers = [KVLayer(num_kv_heads, head_dim, head_dim)] * num_layers
         self.block_size = block_size
         self.num_blocks = num_blocks
-        self.caches = []
-        for _ in range(num_layers):
-            k = torch.zeros(num_blocks, num_kv_heads, block_size, head_dim,
-                            dtype=dtype, device=device)
-            v = torch.zeros(num_blocks, num_kv_heads, block_size, head_dim,
-                            dtype=dtype, device=device)
-            self.caches.append((k, v))
+        self.layers = list(layers)
+        self.caches = [
+            tuple(torch.zeros(num_blocks, *shape, dtype=dtype, device=device)
+                  for shape in (l.k_shape(block_size), l.v_shape(block_size)))
+            for l in self.layers]
         self.allocator = BlockAllocator(num_blocks)
+
+    @classmethod
+    def for_layers(cls, layers: Sequence[KVLayer], block_size: int,
+                   num_blocks: int, device, dtype=torch.bfloat16):
+        return cls(len(layers), 0, 0, block_size, num_blocks, device, dtype,
+                   layers=layers)
 
     @staticmethod
     def block_bytes(num_layers: int, num_kv_heads: int, head_dim: int,
-                    block_size: int, dtype=torch.bfloat16) -> int:
+                    block_size: int, dtype=torch.bfloat16,
+                    layers: Optional[Sequence[KVLayer]] = None) -> int:
+        if layers is None:
+            layers = [KVLayer(num_kv_heads, head_dim, head_dim)] * num_layers
         el = torch.empty(0, dtype=dtype).element_size()
-        return 2 * num_layers * num_kv_heads * block_size * head_dim * el
+        return el * block_size * sum(l.num_kv_heads * (l.k_dim + l.v_dim)
+                                     for l in layers)
 
     @staticmethod
     def blocks_for_bytes(budget: int, num_layers: int, num_kv_heads: int,
-                         head_dim: int, block_size: int) -> int:
+                         head_dim: int, block_size: int,
+                         dtype=torch.bfloat16,
+                         layers: Optional[Sequence[KVLayer]] = None) -> int:
         return max(0, budget // KVCache.block_bytes(
-            num_layers, num_kv_heads, head_dim, block_size))
+            num_layers, num_kv_heads, head_dim, block_size, dtype, layers))

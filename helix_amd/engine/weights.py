@@ -102,6 +102,50 @@ def _map_hf_name(name: str):
     return name, None  # our native names pass through
 
 
+class _Stager:
+    """Copies host tensors to their destination views. On GPU they go
+    through double-buffered pinned memory and a side stream; a buffer's
+    event is waited for before the buffer is refilled."""
+
+    def __init__(self, device, use_async: bool = True):
+        self.device = device
+        self.side = torch.cuda.Stream(device) \
+            if (device.type == "cuda" and use_async) else None
+        self.pinned = [None, None]
+        self.events = [None, None]
+        self.cur = 0
+
+    def copy(self, dst_view: torch.Tensor, src: torch.Tensor):
+        src = src.to(dst_view.dtype)
+        if self.side is None:
+            dst_view.copy_(src)
+            return
+        cur = self.cur
+        n = src.numel() * src.element_size()
+        if self.pinned[cur] is None or self.pinned[cur].numel() < n:
+            self.pinned[cur] = torch.empty(max(n, 64 << 20),
+                                           dtype=torch.uint8, pin_memory=True)
+            self.events[cur] = torch.cuda.Event()
+        else:
+            self.events[cur].synchronize()
+        flat = self.pinned[cur][:n]
+        flat.copy_(src.contiguous().view(-1).view(torch.uint8))
+        with torch.cuda.stream(self.side):
+            if dst_view.is_contiguous():
+                dst_view.view(-1).view(torch.uint8).copy_(flat,
+                                                          non_blocking=True)
+            else:
+                dst_view.copy_(flat.view(src.dtype).view(src.shape),
+                               non_blocking=True)
+            self.events[cur].record(self.side)
+        self.cur ^= 1
+
+    def finish(self):
+        if self.side is not None:
+            torch.cuda.current_stream(self.device).wait_stream(self.side)
+            torch.cuda.synchronize(self.device)
+
+
 @torch.inference_mode()
 def load_llama_weights(model, ckpt_dir: str, use_async: bool = True):
     """Load a Llama checkpoint (HF layout or our native layout) into the
@@ -127,35 +171,8 @@ def load_llama_weights(model, ckpt_dir: str, use_async: bool = True):
     cfg = model.cfg
     q, kv = cfg.q_size, cfg.kv_size
     inter = cfg.intermediate_size
-    device = next(model.parameters()).device
-    on_gpu = device.type == "cuda"
-    side = torch.cuda.Stream(device) if (on_gpu and use_async) else None
-    # Double-buffered pinned staging: wait on a buffer's event before
-    # refilling it so the async copy out of it has completed.
-    pinned = [None, None]
-    events = [None, None]
-    cur = 0
-
-    def stage_copy(dst_view: torch.Tensor, src: torch.Tensor):
-        nonlocal cur
-        src = src.to(dst_view.dtype)
-        if side is None:
-            dst_view.copy_(src)
-            return
-        n = src.numel() * src.element_size()
-        if pinned[cur] is None or pinned[cur].numel() < n:
-            pinned[cur] = torch.empty(max(n, 64 << 20), dtype=torch.uint8,
-                                      pin_memory=True)
-            events[cur] = torch.cuda.Event()
-        else:
-            events[cur].synchronize()
-        flat = pinned[cur][:n]
-        flat.copy_(src.contiguous().view(-1).view(torch.uint8))
-        with torch.cuda.stream(side):
-            dst_view.view(-1).view(torch.uint8).copy_(flat,
-                                                      non_blocking=True)
-            events[cur].record(side)
-        cur ^= 1
+    stager = _Stager(next(model.parameters()).device, use_async)
+    stage_copy = stager.copy
 
     loaded = 0
     for name, tensor in iter_safetensors(ckpt_dir):
@@ -177,8 +194,40 @@ def load_llama_weights(model, ckpt_dir: str, use_async: bool = True):
         else:
             stage_copy(p.data, tensor)
         loaded += 1
-    if side is not None:
-        torch.cuda.current_stream(device).wait_stream(side)
-        torch.cuda.synchronize(device)
+    stager.finish()
     log.info("loaded %d tensors from %s", loaded, ckpt_dir)
     return loaded
+
+
+@torch.inference_mode()
+def load_mapped_weights(model, ckpt_dir: str, use_async: bool = True) -> int:
+    """Load a checkpoint through the model's own name map
+    (checkpoint_targets: tensor name -> destination view). Every target
+    has to be there, with its exact shape."""
+    targets = model.checkpoint_targets()
+    missing = set(targets) - set(model.optional_checkpoint_names())
+    stager = _Stager(next(model.parameters()).device, use_async)
+    loaded = 0
+    for name, tensor in iter_safetensors(ckpt_dir):
+        dst = targets.get(name)
+        if dst is None:
+            log.debug("skipping unknown weight %s", name)
+            continue
+        if tuple(tensor.shape) != tuple(dst.shape):
+            raise ValueError(f"{name}: checkpoint has {tuple(tensor.shape)}, "
+                             f"the configuration {tuple(dst.shape)}")
+        stager.copy(dst, tensor)
+        missing.discard(name)
+        loaded += 1
+    stager.finish()
+    if missing:
+        raise ValueError(f"{ckpt_dir} lacks {sorted(missing)}")
+    log.info("loaded %d tensors from %s", loaded, ckpt_dir)
+    return loaded
+
+
+def load_weights(model, ckpt_dir: str, use_async: bool = True) -> int:
+    """Load a checkpoint into any causal LM of the registry."""
+    if hasattr(model, "checkpoint_targets"):
+        return load_mapped_weights(model, ckpt_dir, use_async)
+    return load_llama_weights(model, ckpt_dir, use_async)

@@ -19,6 +19,8 @@ import torch.nn as nn
 import torch.nn.functional as F
 
 from helix_amd import ops
+from helix_amd.models.meta import (DecodeMeta, KVLayer,  # noqa: F401
+                                   MixedMeta, PrefillMeta)
 from helix_amd.ops import make_cos_sin_cache
 
 
@@ -47,6 +49,45 @@ class LlamaConfig:
     @property
     def kv_size(self) -> int:
         return self.num_kv_heads * self.head_dim
+
+    def kv_layers(self, tp_size: int = 1) -> list:
+        return [KVLayer(self.num_kv_heads // tp_size, self.head_dim,
+                        self.head_dim)] * self.num_layers
+
+    def num_weights(self) -> tuple:
+        """(embedding and head, per-layer total) parameter counts."""
+        emb = self.vocab_size * self.hidden_size * \
+            (1 if self.tie_embeddings else 2)
+        per_layer = (self.hidden_size * (self.q_size + 2 * self.kv_size)
+                     + self.q_size * self.hidden_size
+                     + 3 * self.hidden_size * self.intermediate_size)
+        return emb, self.num_layers * per_layer
+
+    def activation_bytes(self, tokens: int) -> int:
+        return 0            # covered by the memory-utilization margin
+
+    @classmethod
+    def from_json(cls, d: dict, name: str = "llama") -> "LlamaConfig":
+        """From a Hugging Face config.json (llama, mistral, qwen2)."""
+        heads = d["num_attention_heads"]
+        qwen = (d.get("architectures") or [""])[0].startswith("Qwen2")
+        window = d.get("sliding_window") or 0
+        if not d.get("use_sliding_window", not qwen):
+            window = 0
+        return cls(
+            name=name, vocab_size=d["vocab_size"],
+            hidden_size=d["hidden_size"],
+            intermediate_size=d["intermediate_size"],
+            num_layers=d["num_hidden_layers"], num_heads=heads,
+            num_kv_heads=d.get("num_key_value_heads") or heads,
+            head_dim=d.get("head_dim") or d["hidden_size"] // heads,
+            rms_norm_eps=d.get("rms_norm_eps", 1e-5),
+            rope_base=float(d.get("rope_theta", 10000.0)),
+            max_position=d.get("max_position_embeddings", 8192),
+            tie_embeddings=d.get("tie_word_embeddings", False),
+            sliding_window=window,
+            attention_bias=d.get("attention_bias", qwen),
+            rope_scaling=d.get("rope_scaling") or {})
 
 
 PRESETS = {
@@ -91,34 +132,6 @@ PRESETS = {
 }
 
 
-@dataclass
-class PrefillMeta:
-    """Varlen prefill: q/k/v are concatenated new tokens of all sequences.
-    With prefix caching, q covers only the uncached suffix; attention
-    gathers the full context K/V from the paged cache (gather_blk/off)
-    and cu_seqlens_k carries the full-context boundaries."""
-    cu_seqlens: torch.Tensor       # [B+1] int32 (new-token boundaries)
-    max_seqlen: int
-    slot_mapping: torch.Tensor     # [T] int64 cache slots for new tokens
-    positions: torch.Tensor        # [T] int64
-    cu_seqlens_k: Optional[torch.Tensor] = None   # [B+1] int32 full context
-    gather_blk: Optional[torch.Tensor] = None     # [Tk] int64
-    gather_off: Optional[torch.Tensor] = None     # [Tk] int64
-    is_prefill: bool = True
-
-
-@dataclass
-class DecodeMeta:
-    """One new token per running sequence."""
-    block_tables: torch.Tensor     # [B, max_blocks] int32
-    seq_lens: torch.Tensor         # [B] int32 (context incl. current token)
-    slot_mapping: torch.Tensor     # [B] int64
-    positions: torch.Tensor        # [B] int64
-    max_len: int = 0               # host-side max(seq_lens) (avoids sync)
-    workspace: Optional[tuple] = None
-    is_prefill: bool = False
-
-
 class HLinear(nn.Linear):
     """nn.Linear routed through ops.linear: decode-shaped (skinny-M)
     GEMMs run the owned split-K MFMA kernel, prefill-shaped ones stay on
@@ -150,42 +163,55 @@ class Attention(nn.Module):
         # fused strided split + rope + paged-cache write (one kernel, no
         # .contiguous() copies); compact K/V emitted only when the
         # fresh-prefill attention path consumes them directly
+        mixed = isinstance(meta, MixedMeta)
+        prefill = meta.prefill if mixed else meta
         want_kv = meta.is_prefill and \
-            getattr(meta, "cu_seqlens_k", None) is None
+            getattr(prefill, "cu_seqlens_k", None) is None
         q, k, v = ops.rope_qkv_cache(
             meta.positions, qkv, cos_sin, self.nh, self.nkv, self.hd,
             kv_cache=kv_cache, slot_mapping=meta.slot_mapping,
             want_kv=want_kv)
-        if meta.is_prefill:
-            if meta.cu_seqlens_k is not None:
-                # cached-prefix prefill: full-context K/V gathered from
-                # the paged cache (new tokens were just written above)
-                k_cache, v_cache = kv_cache
-                k_all = k_cache[meta.gather_blk, :, meta.gather_off]
-                v_all = v_cache[meta.gather_blk, :, meta.gather_off]
-                if k_all.dtype == torch.uint8:      # fp8 KV cache
-                    k_all = ops.kv_fp8_dequant(k_all, q.dtype)
-                    v_all = ops.kv_fp8_dequant(v_all, q.dtype)
-                o = ops.attn_prefill(q, k_all, v_all, meta.cu_seqlens,
-                                     meta.max_seqlen, self.scale,
-                                     window=self.window,
-                                     cu_seqlens_k=meta.cu_seqlens_k)
-            else:
-                o = ops.attn_prefill(q, k, v, meta.cu_seqlens,
-                                     meta.max_seqlen, self.scale,
-                                     window=self.window)
+        if mixed:
+            n = meta.num_decode
+            o = torch.cat([
+                self._attend_decode(q[:n], kv_cache, meta.decode),
+                self._attend_prefill(q[n:], k[n:] if want_kv else None,
+                                     v[n:] if want_kv else None, kv_cache,
+                                     prefill)])
+        elif meta.is_prefill:
+            o = self._attend_prefill(q, k, v, kv_cache, meta)
         else:
-            k_cache, v_cache = kv_cache
-            o = ops.paged_attn_decode(q, k_cache, v_cache, meta.block_tables,
-                                      meta.seq_lens, self.scale,
-                                      meta.workspace,
-                                      meta.max_len or None,
-                                      window=self.window)
+            o = self._attend_decode(q, kv_cache, meta)
         out = self.o_proj(o.view(T, -1))
         if self.tp_size > 1:
             from helix_amd import parallel
             out = parallel.tp_all_reduce(out)
         return out
+
+    def _attend_prefill(self, q, k, v, kv_cache, meta):
+        if meta.cu_seqlens_k is None:
+            return ops.attn_prefill(q, k, v, meta.cu_seqlens,
+                                    meta.max_seqlen, self.scale,
+                                    window=self.window)
+        # cached-prefix prefill: full-context K/V gathered from the paged
+        # cache (new tokens were just written)
+        k_cache, v_cache = kv_cache
+        k_all = k_cache[meta.gather_blk, :, meta.gather_off]
+        v_all = v_cache[meta.gather_blk, :, meta.gather_off]
+        if k_all.dtype == torch.uint8:      # fp8 KV cache
+            k_all = ops.kv_fp8_dequant(k_all, q.dtype)
+            v_all = ops.kv_fp8_dequant(v_all, q.dtype)
+        return ops.attn_prefill(q, k_all, v_all, meta.cu_seqlens,
+                                meta.max_seqlen, self.scale,
+                                window=self.window,
+                                cu_seqlens_k=meta.cu_seqlens_k)
+
+    def _attend_decode(self, q, kv_cache, meta):
+        k_cache, v_cache = kv_cache
+        return ops.paged_attn_decode(q, k_cache, v_cache, meta.block_tables,
+                                     meta.seq_lens, self.scale,
+                                     meta.workspace, meta.max_len or None,
+                                     window=self.window)
 
 
 class MLP(nn.Module):
@@ -229,6 +255,8 @@ class DecoderLayer(nn.Module):
 
 
 class LlamaForCausalLM(nn.Module):
+    paged_prefill = False        # cached prefixes are gathered
+
     def __init__(self, cfg: LlamaConfig, tp_size: int = 1, tp_rank: int = 0):
         super().__init__()
         self.cfg = cfg
@@ -270,6 +298,11 @@ class LlamaForCausalLM(nn.Module):
         if self.lm_head is not None:
             return self.lm_head(hidden)
         return F.linear(hidden, self.embed_tokens.weight)
+
+    def decode_workspace(self, max_batch: int, max_len: int, device):
+        return ops.decode_workspace(max_batch,
+                                    self.cfg.num_heads // self.tp_size,
+                                    self.cfg.head_dim, max_len, device)
 
     @torch.inference_mode()
     def init_random(self, seed: int = 0):

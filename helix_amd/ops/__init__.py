@@ -8,6 +8,7 @@ logic is testable without a GPU.
 from __future__ import annotations
 
 import os
+from dataclasses import dataclass
 
 import torch
 
@@ -23,6 +24,8 @@ try:
 except ImportError as e:  # pragma: no cover
     _C_ERR = str(e)
 
+_C_ext = None
+
 
 def _native():
     if _C is None:
@@ -33,8 +36,30 @@ def _native():
     return _C
 
 
-def have_native() -> bool:
-    return _C is not None
+def _native_ext():
+    """helix_amd._C_ext, imported at first use (a program may build it
+    after this module was imported)."""
+    global _C_ext
+    if _C_ext is None:
+        try:
+            from helix_amd import _C_ext as mod  # type: ignore
+        except ImportError as e:
+            raise RuntimeError(
+                "helix_amd._C_ext native extension is not built but a GPU "
+                "tensor was passed. Build it with `python setup.py build_ext "
+                "--inplace` (PYTORCH_ROCM_ARCH=gfx950). Import error: "
+                f"{e}") from e
+        _C_ext = mod
+    return _C_ext
+
+
+def have_native(name: str = "_C") -> bool:
+    if name == "_C":
+        return _C is not None
+    try:
+        return _native_ext() is not None
+    except RuntimeError:
+        return False
 
 
 def rms_norm(x: torch.Tensor, w: torch.Tensor, eps: float) -> torch.Tensor:
@@ -340,3 +365,167 @@ def mfma_probe(a: torch.Tensor, b: torch.Tensor) -> torch.Tensor:
     d = torch.empty(16, 16, dtype=torch.float32, device=a.device)
     _native().mfma_probe(d, a, b)
     return d
+
+
+# ---------------------------------------------------------------------------
+# Depth-averaged fp32 residual stream, PolyNorm, talking-head attention
+# ---------------------------------------------------------------------------
+
+@dataclass
+class TalkParams:
+    """Constants of one talking-head attention layer. softcap / window 0,
+    slopes / talk None switch the mechanism off."""
+    scale: float
+    softcap: float = 0.0
+    window: int = 0
+    slopes: torch.Tensor | None = None     # [H] fp32 distance bias per head
+    talk: torch.Tensor | None = None       # [H, H] fp32 mixing matrix
+
+    def max_keys(self, max_len: int) -> int:
+        return min(max_len, self.window) if self.window else max_len
+
+
+def embed_norm(ids: torch.Tensor, embed: torch.Tensor, w: torch.Tensor,
+               eps: float, x: torch.Tensor) -> torch.Tensor:
+    """x (fp32, written) <- embed[ids]; returns its RMS norm times w."""
+    if embed.is_cuda:
+        h = torch.empty(x.shape, dtype=embed.dtype, device=x.device)
+        _native_ext().embed_norm(h, x, ids, embed, w, eps)
+        return h
+    return ref.embed_norm(ids, embed, w, eps, x)
+
+
+def depth_norm(x: torch.Tensor, y: torch.Tensor, hist: torch.Tensor,
+               n_prev: int, coef: torch.Tensor, w: torch.Tensor, eps: float,
+               store_new: bool = True,
+               x_out: torch.Tensor | None = None) -> torch.Tensor:
+    """Layer result X = x + y, depth average over hist[:n_prev] and X, RMS
+    norm. Appends X to hist (store_new), writes the average to x_out (which
+    may be x), returns the normed rows in y's dtype."""
+    if y.is_cuda:
+        h = torch.empty(x.shape, dtype=y.dtype, device=y.device)
+        _native_ext().depth_norm(h, x_out, x, y, hist, n_prev, store_new,
+                                 coef, w, eps)
+        return h
+    return ref.depth_norm(x, y, hist, n_prev, coef, w, eps, store_new, x_out)
+
+
+def poly_norm(z: torch.Tensor, coef: torch.Tensor, eps: float,
+              out: torch.Tensor | None = None) -> torch.Tensor:
+    """a N(z) + b N(z^2) + c N(z^3) + e, N = division by the row's root
+    mean square; coef = (a, b, c, e) fp32. z and out may be column slices."""
+    if out is None:
+        out = torch.empty(z.shape, dtype=z.dtype, device=z.device)
+    if z.is_cuda:
+        _native_ext().poly_norm(out, z, coef, eps)
+    else:
+        out.copy_(ref.poly_norm(z, coef, eps))
+    return out
+
+
+def unit_qkv_cache(z: torch.Tensor, offsets, num_q: int, head_dim: int,
+                   kv_cache, slot_mapping: torch.Tensor, eps: float,
+                   v_first: torch.Tensor | None = None,
+                   lam: torch.Tensor | None = None, first: bool = False,
+                   ff=None) -> torch.Tensor:
+    """Epilogue of the fused input projection z: unit-RMS q and k heads (no
+    weight), value mixing, paged-cache write; returns q [T, H, Dp].
+
+    offsets = (q, k, v) column starts. lam switches value mixing on: the
+    first such layer writes its values to v_first, later ones blend
+    (1 - lam) v + lam v_first. ff = (z_cols, out_cols, coef) runs PolyNorm
+    in the same launch. Cache: K [nblk, G, bs, Dp], V [nblk, G, E, bs].
+    """
+    kc, vc = kv_cache
+    if z.is_cuda:
+        q = torch.empty(z.shape[0], num_q, kc.shape[3], dtype=z.dtype,
+                        device=z.device)
+        args = (z, *offsets, q, kc, vc, slot_mapping, v_first, lam, first,
+                head_dim, eps)
+        if ff is None:
+            _native_ext().unit_qkv_cache(*args)
+        else:
+            zf, out, coef = ff
+            _native_ext().layer_epilogue(*args, out, zf, coef)
+        return q
+    if ff is not None:
+        zf, out, coef = ff
+        out.copy_(ref.poly_norm(zf, coef, eps))
+    return ref.unit_qkv_cache(z, offsets, num_q, head_dim, kc, vc,
+                              slot_mapping, eps, v_first, lam, first)
+
+
+# Partition granularity of the row kernels (QUANT in talk_attn_rows.hip) and
+# their scratch bound when they process a whole prompt.
+TALK_PARTITION = 128
+TALK_SCRATCH_FLOATS = 64 << 20
+
+
+def _talk_parts(rows: int, num_kv: int, max_keys: int) -> int:
+    return min(-(-max_keys // TALK_PARTITION),
+               max(1, 1024 // max(1, rows * num_kv)))
+
+
+def talk_scratch_floats(rows: int, num_q: int, num_kv: int, v_dim: int,
+                        max_keys: int) -> int:
+    parts = _talk_parts(rows, num_kv, max_keys)
+    return rows * num_q * (max_keys + parts * (2 + v_dim))
+
+
+def talk_attn_rows(out: torch.Tensor, q: torch.Tensor, kv_cache,
+                   block_tables: torch.Tensor, row_len: torch.Tensor,
+                   max_len: int, p: TalkParams, gate=None, row_seq=None,
+                   workspace: torch.Tensor | None = None) -> None:
+    """out [R, H*E] <- attention of single query rows; row r reads the
+    first row_len[r] cached tokens of block-table row row_seq[r] (r if
+    None). gate: [R, H] logits, one sigmoid factor per head."""
+    kc, vc = kv_cache
+    if not q.is_cuda:
+        ref.talk_attn_rows(out, q, kc, vc, block_tables, row_len, p, gate,
+                           row_seq)
+        return
+    R, H = q.shape[:2]
+    G, E = vc.shape[1:3]
+    keys = p.max_keys(max_len)
+    need = talk_scratch_floats(R, H, G, E, keys)
+    if workspace is None or workspace.numel() < need:
+        workspace = torch.empty(need, dtype=torch.float32, device=q.device)
+    parts = _talk_parts(R, G, keys)
+    a, b = R * H * keys, R * H * parts * 2
+    _native_ext().talk_attn_rows(
+        out, q, kc, vc, block_tables, row_seq, row_len, keys, p.scale,
+        p.softcap, p.window, p.slopes, p.talk, gate,
+        workspace[:a].view(R, H, keys),
+        workspace[a:a + b].view(R, H, parts, 2),
+        workspace[a + b:need].view(R, H, parts, E))
+
+
+def talk_attn_prefill(out: torch.Tensor, q: torch.Tensor, kv_cache,
+                      block_tables: torch.Tensor, cu_seqlens: torch.Tensor,
+                      seq_lens: torch.Tensor, max_q: int, max_len: int,
+                      row_seq: torch.Tensor, row_len: torch.Tensor,
+                      p: TalkParams, gate=None) -> None:
+    """Prompt portions: sequence b's rows cu_seqlens[b]..[b+1] are the last
+    ones of its seq_lens[b] cached tokens. bf16 runs the MFMA kernel; fp32
+    and oversized heads run the row kernels in slices of bounded scratch
+    (row_seq / row_len map each row to its sequence and visible length)."""
+    kc, vc = kv_cache
+    if not q.is_cuda:
+        ref.talk_attn_rows(out, q, kc, vc, block_tables, row_len, p, gate,
+                           row_seq)
+        return
+    T, H, Dp = q.shape
+    G, E = vc.shape[1:3]
+    if q.dtype == torch.bfloat16 and \
+            _native_ext().talk_prefill_fits(H, Dp, E):
+        _native_ext().talk_attn_prefill(
+            out, q, kc, vc, block_tables, cu_seqlens, seq_lens, max_q,
+            p.scale, p.softcap, p.window, p.slopes, p.talk, gate)
+        return
+    keys = p.max_keys(max_len)
+    step = max(1, TALK_SCRATCH_FLOATS // (H * (keys + 2 + E)))
+    for r in range(0, T, step):
+        s = slice(r, min(T, r + step))
+        talk_attn_rows(out[s], q[s], kv_cache, block_tables, row_len[s],
+                       max_len, p, None if gate is None else gate[s],
+                       row_seq[s])

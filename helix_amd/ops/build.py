@@ -1,0 +1,29 @@
+"""In-tree build of the native extensions, on demand.
+
+A source checkout has no built libraries; a program that needs one calls
+ensure() before it imports helix_amd.ops. Only the named extension is
+compiled (gfx950, cross-compilation needs no GPU).
+"""
+from __future__ import annotations
+
+import glob
+import os
+import subprocess
+import sys
+
+ROOT = os.path.dirname(os.path.dirname(os.path.dirname(
+    os.path.abspath(__file__))))
+
+
+def is_built(name: str) -> bool:
+    return bool(glob.glob(os.path.join(ROOT, "helix_amd", f"{name}.*.so")))
+
+
+def ensure(name: str) -> None:
+    """Compile extension `name` unless its library is there. The compiler's
+    output goes to standard error."""
+    if is_built(name):
+        return
+    env = dict(os.environ, PYTORCH_ROCM_ARCH="gfx950", HELIX_BUILD_ONLY=name)
+    subprocess.run([sys.executable, "setup.py", "build_ext", "--inplace"],
+                   cwd=ROOT, env=env, check=True, stdout=sys.stderr)

@@ -208,3 +208,91 @@ def gemm_bf16(x: torch.Tensor, w: torch.Tensor, bias=None,
     if act == 1:
         out = torch.nn.functional.gelu(out, approximate="tanh")
     return out.to(x.dtype)
+
+
+def _rms_inv(x: torch.Tensor, eps: float) -> torch.Tensor:
+    return torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
+
+
+def embed_norm(ids, embed, w, eps, x):
+    x.copy_(embed[ids])
+    return (x * _rms_inv(x, eps) * w).to(embed.dtype)
+
+
+def depth_norm(x, y, hist, n_prev, coef, w, eps, store_new=True, x_out=None):
+    new = x + y.float()
+    avg = coef[n_prev] * new + torch.einsum("n,ntw->tw", coef[:n_prev],
+                                            hist[:n_prev])
+    if store_new:
+        hist[n_prev] = new
+    if x_out is not None:
+        x_out.copy_(avg)
+    return (avg * _rms_inv(avg, eps) * w).to(y.dtype)
+
+
+def poly_norm(z, coef, eps):
+    zf = z.float()
+    z2, z3 = zf * zf, zf * zf * zf
+    a, b, c, e = coef.unbind()
+    return (a * zf * _rms_inv(zf, eps) + b * z2 * _rms_inv(z2, eps)
+            + c * z3 * _rms_inv(z3, eps) + e).to(z.dtype)
+
+
+def unit_qkv_cache(z, offsets, num_q, head_dim, k_cache, v_cache,
+                   slot_mapping, eps, v_first=None, lam=None, first=False):
+    T = z.shape[0]
+    _, G, bs, Dp = k_cache.shape
+    E = v_cache.shape[2]
+    qo, ko, vo = offsets
+
+    def unit(cols, n):
+        u = cols.reshape(T, n, head_dim).float()
+        u = torch.nn.functional.pad(u * _rms_inv(u, eps), (0, Dp - head_dim))
+        return u.to(z.dtype)
+
+    q = unit(z[:, qo:qo + num_q * head_dim], num_q)
+    k = unit(z[:, ko:ko + G * head_dim], G)
+    v = z[:, vo:vo + G * E]
+    if lam is not None:
+        if first:
+            v_first.copy_(v)
+        else:
+            v = ((1 - lam) * v.float() + lam * v_first.float()).to(z.dtype)
+    live = slot_mapping >= 0
+    slots = slot_mapping[live]
+    blk, off = slots // bs, slots % bs
+    k_cache[blk, :, off] = k[live].to(k_cache.dtype)
+    v_cache[blk, :, :, off] = v.reshape(T, G, E)[live].to(v_cache.dtype)
+    return q
+
+
+def talk_attn_rows(out, q, k_cache, v_cache, block_tables, row_len, p,
+                   gate=None, row_seq=None):
+    R, H, _ = q.shape
+    _, G, bs, _ = k_cache.shape
+    E = v_cache.shape[2]
+    for r in range(R):
+        n = int(row_len[r])
+        lo = max(0, n - p.window) if p.window else 0
+        b0, b1 = lo // bs, (n + bs - 1) // bs
+        row = r if row_seq is None else int(row_seq[r])
+        blocks = block_tables[row, b0:b1].long()
+        k = k_cache[blocks].transpose(1, 2).flatten(0, 1)
+        v = v_cache[blocks].permute(0, 3, 1, 2).flatten(0, 1)
+        k = k[lo - b0 * bs:n - b0 * bs].float()
+        v = v[lo - b0 * bs:n - b0 * bs].float()
+        s = torch.einsum("gcd,ngd->gcn", q[r].float().view(G, H // G, -1),
+                         k).reshape(H, -1) * p.scale
+        if p.softcap:
+            s = p.softcap * torch.tanh(s / p.softcap)
+        if p.slopes is not None:
+            dist = (n - 1 - torch.arange(lo, n)).to(s.dtype)
+            s = s - p.slopes[:, None] * dist
+        w = torch.softmax(s, -1)
+        if p.talk is not None:
+            w = p.talk @ w
+        o = torch.einsum("gcn,nge->gce", w.view(G, H // G, -1),
+                         v).reshape(H, E)
+        if gate is not None:
+            o = o * torch.sigmoid(gate[r].float())[:, None]
+        out[r] = o.reshape(-1).to(out.dtype)

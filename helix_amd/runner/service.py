@@ -20,9 +20,10 @@ from typing import Dict, List, Optional
 import torch
 
 from helix_amd.engine.engine import EngineConfig, LLMEngine, Sequence
+from helix_amd.engine.kv_cache import KVCache
 from helix_amd.engine.sampling_params import SamplingParams
 from helix_amd.models.bert import BERT_PRESETS, BertEmbeddingModel
-from helix_amd.models.llama import PRESETS as LLAMA_PRESETS
+from helix_amd.models import registry
 from helix_amd.utils.tokenizer import get_tokenizer
 
 log = logging.getLogger("helix_amd.runner")
@@ -33,7 +34,7 @@ class ModelSpec:
     """Manifest entry (replaces compose-profile YAML model entries)."""
     name: str
     kind: str = "llm"                  # llm | embedding
-    preset: str = "llama3-8b"
+    preset: str = "llama3-8b"          # preset name or checkpoint folder
     max_model_len: int = 8192
     max_num_seqs: int = 64
     kv_cache_blocks: Optional[int] = None
@@ -50,6 +51,8 @@ DEFAULT_SPECS = {
     "mistral-7b": ModelSpec("mistral-7b", "llm", "mistral-7b"),
     "qwen2-7b": ModelSpec("qwen2-7b", "llm", "qwen2-7b",
                           max_model_len=32768),
+    "zederax-8b": ModelSpec("zederax-8b", "llm", "zederax-8b"),
+    "zederax-1b": ModelSpec("zederax-1b", "llm", "zederax-1b"),
     "bge-base": ModelSpec("bge-base", "embedding", "bge-base"),
     "siglip-base": ModelSpec("siglip-base", "vision", "siglip-base"),
     "tiny-vit": ModelSpec("tiny-vit", "vision", "tiny-vit"),
@@ -61,6 +64,8 @@ DEFAULT_SPECS = {
                       kv_cache_blocks=256),
     "tiny-gqa": ModelSpec("tiny-gqa", "llm", "tiny-gqa", max_model_len=512,
                           kv_cache_blocks=256),
+    "tiny-zederax": ModelSpec("tiny-zederax", "llm", "tiny-zederax",
+                              max_model_len=256, kv_cache_blocks=256),
     "tiny-bert": ModelSpec("tiny-bert", "embedding", "tiny-bert"),
 }
 
@@ -91,16 +96,13 @@ def estimate_model_bytes(spec: ModelSpec, block_size: int = 16) -> int:
         per_layer = 4 * cfg.hidden_size ** 2 + \
             2 * cfg.hidden_size * cfg.intermediate_size
         return 2 * (n + cfg.num_layers * per_layer) + (64 << 20)
-    cfg = LLAMA_PRESETS[spec.preset]
-    emb = cfg.vocab_size * cfg.hidden_size * (1 if cfg.tie_embeddings else 2)
-    per_layer = (cfg.hidden_size * (cfg.q_size + 2 * cfg.kv_size)  # qkv
-                 + cfg.q_size * cfg.hidden_size                     # o
-                 + 3 * cfg.hidden_size * cfg.intermediate_size)     # mlp
+    cfg = registry.get_config(spec.preset)
+    emb, layers = cfg.num_weights()
     wbytes = 1 if spec.quantization == "fp8" else 2
     # fp8 halves the projection weights (embeddings/lm_head stay bf16)
-    weights = 2 * emb + wbytes * cfg.num_layers * per_layer
-    kv_block = 2 * cfg.num_layers * cfg.num_kv_heads * block_size * \
-        cfg.head_dim * 2
+    weights = 2 * emb + wbytes * layers
+    kv_block = KVCache.block_bytes(0, 0, 0, block_size,
+                                   layers=cfg.kv_layers())
     if spec.kv_cache_blocks:
         kv = kv_block * spec.kv_cache_blocks
     else:
@@ -118,12 +120,11 @@ class LLMInstance:
         kv_blocks = spec.kv_cache_blocks
         if kv_blocks is None and torch.cuda.is_available():
             free, total = torch.cuda.mem_get_info(torch.device(device))
-            from helix_amd.engine.kv_cache import KVCache
-            cfg = LLAMA_PRESETS[spec.preset]
+            cfg = registry.get_config(spec.preset)
             budget = int(total * spec.kv_memory_fraction)
             kv_blocks = KVCache.blocks_for_bytes(
                 min(budget, max(free - (2 << 30), 1 << 28)),
-                cfg.num_layers, cfg.num_kv_heads, cfg.head_dim, 16)
+                0, 0, 0, 16, layers=cfg.kv_layers())
         self.engine = LLMEngine(
             EngineConfig(model=spec.preset, max_model_len=spec.max_model_len,
                          max_num_seqs=spec.max_num_seqs,

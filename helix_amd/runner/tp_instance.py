@@ -78,6 +78,8 @@ def _tp_worker(rank: int, world: int, preset: str, engine_kwargs: dict,
         else:
             device = "cpu"
         parallel.init_tp(world, backend=backend)
+        if preset not in PRESETS:
+            raise ValueError(f"{preset} has no tensor-parallel form")
         cfg = PRESETS[preset]
         # One-shot xGMI allreduce sized for the decode messages
         # (B x hidden bf16); prefill messages exceed it and fall back to

@@ -1,6 +1,9 @@
-"""Build the helix_amd native extension in-tree for MI355X (gfx950).
+"""Build the helix_amd native extensions in-tree for MI355X (gfx950).
 
 Usage: PYTORCH_ROCM_ARCH=gfx950 python setup.py build_ext --inplace
+
+HELIX_BUILD_ONLY (comma-separated module names, e.g. "_C_ext") limits the
+build to the extensions one model needs.
 """
 import os
 import glob
@@ -17,22 +20,28 @@ HIP_DIR = os.path.join(ROOT, "helix_amd", "ops", "hip")
 # them from ordinary float code and some have given wrong results here.
 NO_PACKED_FP32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
-sources = sorted(
-    f for f in glob.glob(os.path.join(HIP_DIR, "*.hip"))
-    if not f.endswith("_hip.hip")       # torch-hipify build artifacts
-) + [os.path.join(HIP_DIR, "bindings.cpp")]
+
+def extension(name, folder):
+    sources = sorted(
+        f for f in glob.glob(os.path.join(folder, "*.hip"))
+        if not f.endswith("_hip.hip")       # torch-hipify build artifacts
+    ) + [os.path.join(folder, "bindings.cpp")]
+    return CUDAExtension(
+        name=f"helix_amd.{name}",
+        sources=sources,
+        extra_compile_args={
+            "cxx": ["-O3", "-std=c++17"],
+            "nvcc": ["-O3", "-std=c++17"] + NO_PACKED_FP32,
+        },
+    )
+
+
+EXTENSIONS = {"_C": HIP_DIR, "_C_ext": os.path.join(HIP_DIR, "ext")}
+only = [n for n in os.environ.get("HELIX_BUILD_ONLY", "").split(",") if n]
 
 setup(
     name="helix_amd_C",
-    ext_modules=[
-        CUDAExtension(
-            name="helix_amd._C",
-            sources=sources,
-            extra_compile_args={
-                "cxx": ["-O3", "-std=c++17"],
-                "nvcc": ["-O3", "-std=c++17"] + NO_PACKED_FP32,
-            },
-        )
-    ],
+    ext_modules=[extension(n, d) for n, d in EXTENSIONS.items()
+                 if not only or n in only],
     cmdclass={"build_ext": BuildExtension},
 )
