@@ -38,7 +38,9 @@ class CUDAGraphRunner:
         self.in_bt = torch.zeros(B, self.max_blocks, dtype=torch.int32,
                                  device=device)
         self.in_lens = torch.ones(B, dtype=torch.int32, device=device)
-        # pinned host staging (one DMA per field per step)
+        # pinned host staging (one DMA per field per step); the event says
+        # when the last step's copies are through and it may be refilled
+        self.staged = torch.cuda.Event()
         self.h_ids = torch.zeros(B, dtype=torch.int64, pin_memory=True)
         self.h_pos = torch.zeros(B, dtype=torch.int64, pin_memory=True)
         self.h_slots = torch.zeros(B, dtype=torch.int64, pin_memory=True)
@@ -98,6 +100,7 @@ class CUDAGraphRunner:
         # Stage inputs into pinned host buffers then one async DMA per
         # field (pad rows are inert: slot -1 => no KV write; seq_len 1 =>
         # one garbage token read).
+        self.staged.synchronize()
         self.h_ids[:nb] = 0
         self.h_pos[:nb] = 0
         self.h_slots[:nb] = -1
@@ -115,6 +118,7 @@ class CUDAGraphRunner:
         self.in_slots[:nb].copy_(self.h_slots[:nb], non_blocking=True)
         self.in_lens[:nb].copy_(self.h_lens[:nb], non_blocking=True)
         self.in_bt[:nb].copy_(self.h_bt[:nb], non_blocking=True)
+        self.staged.record()
 
         if key not in self.graphs:
             self.graphs[key] = self._capture(nb, lb)
