@@ -136,6 +136,24 @@ def run_coresident(args) -> None:
     }))
 
 
+def run_design(args) -> None:
+    """Prefill / decode throughput of the Zederax presets and of equally
+    large Llama models, and kernel by kernel distance from the roofline."""
+    from helix_amd.engine import design_bench
+    names = args.design.split(",")
+    res = design_bench.run(names, "cuda:0", min(args.steps, 32),
+                           args.design_part)
+    first = res[names[0]].get("zederax")
+    print(json.dumps({
+        "metric": "tokens/sec (design)",
+        "value": first[-1]["decode_tok_s"] if first else None,
+        "unit": "tokens/s", "n_gpus": 1, "steps": min(args.steps, 32),
+        "warmup": 4, "higher_is_better": True, "scaling": "weak",
+        "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+        "config": {"model": args.design, "parallelism": "dp1"},
+        "design": res}))
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -158,8 +176,16 @@ def main():
                     help="fp8: e4m3 KV cache (opt-in)")
     ap.add_argument("--temperature", type=float, default=0.0)
     ap.add_argument("--top-p", type=float, default=1.0)
+    ap.add_argument("--design", type=str, default="",
+                    help="instead of the headline: comma-separated Zederax "
+                         "presets, each beside a Llama of equal size")
+    ap.add_argument("--design-part", type=str, default="all",
+                    choices=["all", "throughput", "kernels"])
     args = ap.parse_args()
 
+    if args.design:
+        run_design(args)
+        return
     if args.coresident:
         run_coresident(args)
         return

@@ -274,6 +274,8 @@ class LLMEngine:
         self._chunk_target: Dict[str, int] = {}
         while self.waiting and len(self.running) + len(batch) < self.cfg.max_num_seqs:
             seq = self.waiting[0]
+            if seq.row < 0 and not self._free_rows:
+                break                # rows are held by extend() sequences
             L = len(seq.prompt_ids)
             first = not seq.block_table
             matched: List[int] = []

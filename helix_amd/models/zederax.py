@@ -131,7 +131,7 @@ PRESETS = {
         AttentionSpec(heads=32, kv_heads=8, dim=128, vdim=128, window=4096,
                       scale=128 ** -0.5, softcap=50.0, v_mix=True), 8192),
     "zederax-1b": _uniform(
-        "zederax-1b", 32000, 2048, 16, 8192,
+        "zederax-1b", 32000, 2048, 16, 8448,
         AttentionSpec(heads=16, kv_heads=4, dim=128, vdim=128, window=2048,
                       scale=128 ** -0.5, softcap=50.0, v_mix=True), 8192),
     # mixed layers for CPU tests and smoke runs
