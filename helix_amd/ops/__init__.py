@@ -518,9 +518,12 @@ def talk_attn_prefill(out: torch.Tensor, q: torch.Tensor, kv_cache,
     G, E = vc.shape[1:3]
     if q.dtype == torch.bfloat16 and \
             _native_ext().talk_prefill_fits(H, Dp, E):
+        talk = p.talk if p.talk is not None else torch.eye(
+            H, device=q.device)
+        lse = torch.empty(T, H, dtype=torch.float32, device=q.device)
         _native_ext().talk_attn_prefill(
             out, q, kc, vc, block_tables, cu_seqlens, seq_lens, max_q,
-            p.scale, p.softcap, p.window, p.slopes, p.talk, gate)
+            p.scale, p.softcap, p.window, p.slopes, talk, gate, lse)
         return
     keys = p.max_keys(max_len)
     step = max(1, TALK_SCRATCH_FLOATS // (H * (keys + 2 + E)))

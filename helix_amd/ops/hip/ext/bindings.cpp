@@ -33,7 +33,8 @@ void talk_attn_prefill(torch::Tensor out, torch::Tensor q, torch::Tensor kc,
                        torch::Tensor vc, torch::Tensor block_tables,
                        torch::Tensor cu_seqlens, torch::Tensor seq_lens,
                        int64_t max_q, double scale, double cap,
-                       int64_t window, OptT slopes, OptT talk, OptT gate);
+                       int64_t window, OptT slopes, torch::Tensor talk,
+                       OptT gate, torch::Tensor lse);
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("embed_norm", &embed_norm,

@@ -69,7 +69,7 @@ __device__ __forceinline__ float exp_s<float>(float x) { return expf(x); }
 
 template <typename S>
 __device__ __forceinline__ float tanh_s(float x) {
-  return 1.f - 2.f / (1.f + __expf(2.f * x));
+  return 1.f - 2.f * __builtin_amdgcn_rcpf(1.f + __expf(2.f * x));
 }
 template <>
 __device__ __forceinline__ float tanh_s<float>(float x) { return tanhf(x); }
