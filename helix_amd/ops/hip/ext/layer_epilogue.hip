@@ -2,12 +2,14 @@
 //
 //  - unit_qkv_cache: per-head unit-RMS q and k (no weight), value mixing
 //    with the values an earlier layer had for the same token, and the
-//    paged-cache write, one workgroup per token, one wave per head.
+//    paged-cache write. q/k: one workgroup per token. v: one workgroup per
+//    16 tokens, transposed through LDS so that 16 lanes write the 16
+//    neighbouring slots of one value dim.
 //  - poly_norm: a N(z) + b N(z^2) + c N(z^3) + e over a token's feed-forward
 //    vector, N = division by the root mean square.
-//  - layer_epilogue: both in one launch (grid.y selects the role), since
-//    both consume the same projection output and neither fills the chip
-//    alone when few tokens decode.
+//  - layer_epilogue: both in one launch, since both consume the same
+//    projection output and neither fills the chip alone when few tokens
+//    decode. grid.y selects the role.
 //
 // Cache layout: K [nblk, G, bs, Dp] with rows padded to Dp (zeros), so a
 // row is a run of 16-byte loads; V TRANSPOSED inside a block,
@@ -39,12 +41,14 @@ struct QkvArgs {
   int first;
   float eps;
   int H, G, D, Dp, E, bs;
+  int64_t T;
+  int lph;                 // lanes per head of the vector path, 0: scalar
+  int v_split;             // workgroups that share one token group's columns
 };
 
 template <typename S>
-__device__ __forceinline__ void unit_head(const S* src, S* dst, S* dst2,
-                                          int D, int Dp, float eps,
-                                          int lane) {
+__device__ __forceinline__ void unit_head(const S* src, S* dst, int D,
+                                          int Dp, float eps, int lane) {
   float ss = 0.f;
   for (int d = lane; d < D; d += WAVE) {
     const float v = ld1(src + d);
@@ -53,44 +57,95 @@ __device__ __forceinline__ void unit_head(const S* src, S* dst, S* dst2,
   ss = wave_reduce_sum(ss);
   const float inv = 1.f / sqrtf(ss / D + eps);
   for (int d = lane; d < Dp; d += WAVE) {
-    const float v = d < D ? ld1(src + d) * inv : 0.f;
-    if (dst != nullptr) st1(dst + d, v);
-    if (dst2 != nullptr) st1(dst2 + d, v);
+    st1(dst + d, d < D ? ld1(src + d) * inv : 0.f);
   }
 }
 
+// q and k heads of one token. vec: heads are runs of aligned 8-element
+// vectors; lph lanes (a power of two) hold one head, 64 / lph heads a wave.
 template <typename S>
-__device__ __forceinline__ void qkv_role(const QkvArgs<S>& p) {
+__device__ __forceinline__ void qk_role(const QkvArgs<S>& p) {
   const int64_t t = blockIdx.x;
+  if (t >= p.T) return;
   const int wid = threadIdx.x / WAVE, lane = threadIdx.x & (WAVE - 1);
   const S* src = p.z + t * p.z_stride;
   const int64_t slot = p.slots[t];
   const int64_t blk = slot >= 0 ? slot / p.bs : 0;
   const int off = slot >= 0 ? (int)(slot % p.bs) : 0;
+  if (p.lph > 0) {
+    const int per = WAVE / p.lph, sub = lane / p.lph;
+    const int d = (lane % p.lph) * 8;
+    for (int h0 = wid * per; h0 < p.H + p.G; h0 += NW * per) {
+      const int h = h0 + sub;
+      const bool live = h < p.H + p.G && d < p.D;
+      float v[8];
+      float ss = 0.f;
+      if (live) {
+        ldv<8>(src + (h < p.H ? p.q_off + h * p.D
+                              : p.k_off + (h - p.H) * p.D) + d, v);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) ss += v[i] * v[i];
+      }
+      for (int o = p.lph / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, WAVE);
+      if (!live) continue;
+      const float inv = 1.f / sqrtf(ss / p.D + p.eps);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[i] *= inv;
+      if (h < p.H)
+        stv<8>(p.q_out + (t * p.H + h) * p.Dp + d, v);
+      else if (slot >= 0)
+        stv<8>(p.k_cache +
+                   ((blk * p.G + h - p.H) * p.bs + off) * p.Dp + d, v);
+    }
+    return;
+  }
   for (int h = wid; h < p.H + p.G; h += NW) {
     if (h < p.H) {
       unit_head<S>(src + p.q_off + h * p.D,
-                   p.q_out + (t * p.H + h) * p.Dp, nullptr, p.D, p.Dp,
-                   p.eps, lane);
+                   p.q_out + (t * p.H + h) * p.Dp, p.D, p.Dp, p.eps, lane);
     } else if (slot >= 0) {
       const int g = h - p.H;
       unit_head<S>(src + p.k_off + g * p.D,
-                   p.k_cache + ((blk * p.G + g) * p.bs + off) * p.Dp,
-                   nullptr, p.D, p.Dp, p.eps, lane);
+                   p.k_cache + ((blk * p.G + g) * p.bs + off) * p.Dp, p.D,
+                   p.Dp, p.eps, lane);
     }
   }
+}
+
+// Values of VTOK tokens, VCOL columns at a time. (g, e) = (i / E, i % E)
+// makes a column of [blk, G, E, bs] one index i.
+constexpr int VTOK = 16, VCOL = 128, VPITCH = VCOL + 1;
+
+template <typename S>
+__device__ __forceinline__ void v_role(const QkvArgs<S>& p, float* tile) {
   const int n = p.G * p.E;
+  const int64_t t0 = (int64_t)(blockIdx.x / p.v_split) * VTOK;
+  if (t0 >= p.T) return;
+  const int nt = (int)min((int64_t)VTOK, p.T - t0);
   const float lam = (p.lam != nullptr && !p.first) ? *p.lam : 0.f;
-  for (int i = threadIdx.x; i < n; i += NT) {
-    float v = ld1(src + p.v_off + i);
-    if (p.lam != nullptr) {
-      if (p.first) st1(p.v_first + t * n + i, v);
-      else v = (1.f - lam) * v + lam * ld1(p.v_first + t * n + i);
+  const int my = threadIdx.x % VTOK;          // token this lane writes
+  const int64_t slot = my < nt ? p.slots[t0 + my] : -1;
+  const int64_t dst = slot >= 0 ? slot / p.bs * n * p.bs + slot % p.bs : 0;
+  for (int c0 = (blockIdx.x % p.v_split) * VCOL; c0 < n;
+       c0 += p.v_split * VCOL) {
+    const int nc = min(VCOL, n - c0);
+    for (int i = threadIdx.x; i < nt * VCOL; i += NT) {
+      const int tk = i / VCOL, c = i % VCOL;
+      if (c >= nc) continue;
+      float v = ld1(p.z + (t0 + tk) * p.z_stride + p.v_off + c0 + c);
+      if (p.lam != nullptr) {
+        S* carry = p.v_first + (t0 + tk) * n + c0 + c;
+        if (p.first) st1(carry, v);
+        else v = (1.f - lam) * v + lam * ld1(carry);
+      }
+      tile[tk * VPITCH + c] = v;
     }
-    if (slot >= 0) {
-      // (g, e) = (i / E, i % E): [blk, G, E, bs] makes it one index
-      st1(p.v_cache + (blk * n + i) * p.bs + off, v);
-    }
+    __syncthreads();
+    if (slot >= 0)
+      for (int c = threadIdx.x / VTOK; c < nc; c += NT / VTOK)
+        st1(p.v_cache + dst + (int64_t)(c0 + c) * p.bs,
+            tile[my * VPITCH + c]);
+    __syncthreads();
   }
 }
 
@@ -159,7 +214,9 @@ __device__ __forceinline__ void poly_role(const PolyArgs<S>& p, float* red) {
 
 template <typename S>
 __global__ __launch_bounds__(NT) void unit_qkv_kernel(QkvArgs<S> p) {
-  qkv_role<S>(p);
+  __shared__ float tile[VTOK * VPITCH];
+  if (blockIdx.y == 0) qk_role<S>(p);
+  else v_role<S>(p, tile);
 }
 
 template <typename S, int VN>
@@ -171,9 +228,14 @@ __global__ __launch_bounds__(NT) void poly_norm_kernel(PolyArgs<S> p) {
 template <typename S, int VN>
 __global__ __launch_bounds__(NT) void layer_epilogue_kernel(QkvArgs<S> a,
                                                             PolyArgs<S> b) {
-  __shared__ float red[3 * NW];
-  if (blockIdx.y == 0) qkv_role<S>(a);
-  else poly_role<S, VN>(b, red);
+  __shared__ float sh[VTOK * VPITCH];
+  if (blockIdx.y == 0) {
+    if (blockIdx.x < a.T) poly_role<S, VN>(b, sh);
+  } else if (blockIdx.y == 1) {
+    qk_role<S>(a);
+  } else {
+    v_role<S>(a, sh);
+  }
 }
 
 template <typename S>
@@ -226,7 +288,22 @@ QkvArgs<S> qkv_args(torch::Tensor z, int64_t q_off, int64_t k_off,
   a.v_cache = (S*)v_cache.data_ptr();
   a.slots = slots.data_ptr<int64_t>();
   a.eps = (float)eps;
+  a.T = T;
+  const uint64_t m = 8 * sizeof(S) - 1;
+  const bool vec = D % 8 == 0 && D <= 8 * WAVE && q_off % 8 == 0 &&
+                   k_off % 8 == 0 && a.z_stride % 8 == 0 &&
+                   ((uint64_t)a.z & m) == 0;
+  a.lph = 0;
+  if (vec)
+    for (a.lph = 1; a.lph * 8 < D;) a.lph *= 2;
+  a.v_split = std::min(16, cdiv(a.G * a.E, VCOL));
   return a;
+}
+
+// workgroups along x: one per token, or per (token group, column share)
+template <typename S>
+int grid_x(const QkvArgs<S>& a) {
+  return std::max((int)a.T, cdiv((int)a.T, VTOK) * a.v_split);
 }
 
 template <typename S>
@@ -279,7 +356,7 @@ void unit_qkv_cache(torch::Tensor z, int64_t q_off, int64_t k_off,
   HELIX_BY_TYPE(z, "unit_qkv_cache", {
     auto a = qkv_args<S>(z, q_off, k_off, v_off, q_out, k_cache, v_cache,
                          slots, v_first, lam, first, head_dim, eps);
-    hipLaunchKernelGGL((unit_qkv_kernel<S>), dim3(z.size(0)), dim3(NT), 0,
+    hipLaunchKernelGGL((unit_qkv_kernel<S>), dim3(grid_x(a), 2), dim3(NT), 0,
                        stream, a);
   })
 }
@@ -315,10 +392,10 @@ void layer_epilogue(torch::Tensor z, int64_t q_off, int64_t k_off,
                          slots, v_first, lam, first, head_dim, eps);
     auto b = poly_args<S>(ff_z, ff_out, coef, eps);
     if (poly_aligned(b))
-      hipLaunchKernelGGL((layer_epilogue_kernel<S, 8>), dim3(z.size(0), 2),
+      hipLaunchKernelGGL((layer_epilogue_kernel<S, 8>), dim3(grid_x(a), 3),
                          dim3(NT), 0, stream, a, b);
     else
-      hipLaunchKernelGGL((layer_epilogue_kernel<S, 1>), dim3(z.size(0), 2),
+      hipLaunchKernelGGL((layer_epilogue_kernel<S, 1>), dim3(grid_x(a), 3),
                          dim3(NT), 0, stream, a, b);
   })
 }

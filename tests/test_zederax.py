@@ -106,13 +106,14 @@ def _pages(n_tokens, bs, extra, g):
 
 @pytest.mark.parametrize("dev", DEVICES)
 @pytest.mark.parametrize("dtype", [F32, BF16])
-@pytest.mark.parametrize("H,G,D,E", [(6, 2, 40, 24), (3, 3, 20, 17),
-                                     (8, 1, 64, 80), (1, 1, 130, 8)])
-def test_unit_qkv_and_value_mixing(dev, dtype, H, G, D, E):
+@pytest.mark.parametrize("H,G,D,E,T", [
+    (6, 2, 40, 24, 21), (3, 3, 20, 17, 21), (8, 1, 64, 80, 7),
+    (1, 1, 130, 8, 33), (9, 3, 128, 128, 40), (2, 2, 256, 72, 17)])
+def test_unit_qkv_and_value_mixing(dev, dtype, H, G, D, E, T):
     """Unit heads, padding, both roles of value mixing, skipped slots, and
     the fused launch with PolyNorm."""
     g = torch.Generator().manual_seed(H * D)
-    T, bs, F = 21, 8, 56
+    bs, F = 8, 56
     Dp = -(-D // 8) * 8
     off, at = [], 8
     for n in (H * D, G * D, G * E, F):
@@ -167,6 +168,9 @@ ATTN = [
     (12, 4, 72, 48, 50, 7.0, False, True),
     (16, 2, 128, 128, 64, 10.0, True, True),
     (32, 8, 128, 96, 40, 50.0, True, True),
+    (32, 8, 128, 128, 45, 12.0, True, True),
+    (8, 2, 64, 64, 31, 9.0, True, True),
+    (32, 4, 64, 64, 0, 9.0, True, True),
     (24, 24, 24, 40, 1, 30.0, True, True),
     (40, 8, 32, 32, 37, 8.0, True, True),      # beyond the MFMA kernel
     (3, 1, 144, 136, 45, 50.0, True, True),     # beyond the MFMA kernel
