@@ -248,7 +248,7 @@ __global__ __launch_bounds__(256) void talk_stats_kernel(PrefillArgs a) {
 // (lse, the mixing matrix) waits in LDS.
 template <int HPW, int DT, int ET, bool FAST>
 __global__ __launch_bounds__(512) void talk_values_kernel(PrefillArgs a) {
-  extern __shared__ uint16_t lds[];
+  extern __shared__ __attribute__((aligned(16))) uint16_t lds[];
   const int lane = threadIdx.x & (WAVE - 1);
   const int wid = __builtin_amdgcn_readfirstlane(threadIdx.x / WAVE);
   const int nwaves = blockDim.x / WAVE;

@@ -17,6 +17,16 @@
 // sized by the host so small batches still fill the 256 CUs. Compiled for
 // bf16 and fp32 storage; all math is fp32.
 //
+// bf16 runs both streams on MFMA, which is idle otherwise and keeps the VALU
+// out of the way of the loads:
+//
+//   scores  4 tiles of 16 keys accumulate into ONE 16x16 result: tile u's
+//           A operand holds the 4 queries in rows 4u..4u+3 and zeros
+//           elsewhere, so lane (hi, lo) ends up with the 4 heads of key
+//           16 hi + lo: a lane per key, no lane idle.
+//   values  the mixed weights are the A operand, split into two bf16 terms
+//           (17 significant bits), V pages are B operands as they lie.
+//
 // Cache layout: K [nblk, G, bs, Dp]; V [nblk, G, E, bs] (8 tokens of one
 // value dim are one 16-byte load).
 #include "elem.h"
@@ -41,16 +51,45 @@ struct RowGeom {
   int window, H, G, bs, span, part, max_parts, hchunks;
 };
 
-// DP > 0: compile-time padded key size (multiple of 8); 0: runtime dp.
-template <typename S, int DP, int HC>
+// Per-thread (max, sum) of HC heads -> one pair per partition.
+template <typename S, int HC>
+__device__ __forceinline__ void store_stats(const float (&mx)[HC],
+                                            const float (&sm)[HC],
+                                            float (&red)[2][HC][NWV], int nh,
+                                            float* ml, int64_t head0,
+                                            int max_parts, int part) {
+  const int wid = threadIdx.x / WAVE, lane = threadIdx.x & (WAVE - 1);
+#pragma unroll
+  for (int i = 0; i < HC; ++i) {
+    const float wm = wave_reduce_max(mx[i]);
+    const float ws = wave_reduce_sum(sm[i] * exp_s<S>(mx[i] - wm));
+    if (lane == 0) {
+      red[0][i][wid] = wm;
+      red[1][i][wid] = ws;
+    }
+  }
+  __syncthreads();
+  if ((int)threadIdx.x < nh) {
+    const int i = threadIdx.x;
+    float M = NEG, L = 0.f;
+    for (int w = 0; w < NWV; ++w) M = fmaxf(M, red[0][i][w]);
+    for (int w = 0; w < NWV; ++w)
+      L += red[1][i][w] * exp_s<S>(red[0][i][w] - M);
+    float* o = ml + ((head0 + i) * max_parts + part) * 2;
+    o[0] = M;
+    o[1] = L;
+  }
+}
+
+// Score pass, a thread per key.
+template <typename S, int HC>
 __global__ __launch_bounds__(NT) void row_scores_kernel(
     float* __restrict__ scores, float* __restrict__ ml,
     const S* __restrict__ q, const S* __restrict__ kc,
-    const float* __restrict__ slopes, float scale, float cap, int dp_rt,
+    const float* __restrict__ slopes, float scale, float cap, int Dp,
     RowGeom m) {
   extern __shared__ float q_lds[];            // [HC][Dp]
   __shared__ float red[2][HC][NWV];
-  const int Dp = DP > 0 ? DP : dp_rt;
   const int row = blockIdx.x, part = blockIdx.z;
   const int g = blockIdx.y / m.hchunks, hc = blockIdx.y % m.hchunks;
   const int HG = m.H / m.G;
@@ -82,31 +121,13 @@ __global__ __launch_bounds__(NT) void row_scores_kernel(
     float acc[HC];
 #pragma unroll
     for (int i = 0; i < HC; ++i) acc[i] = 0.f;
-    if constexpr (DP > 0 && sizeof(S) == 2) {
-      u16x8 raw[DP / 8];
+    for (int j = 0; j < Dp; j += 8) {
+      float k[8];
+      ldv<8>(krow + j, k);
 #pragma unroll
-      for (int j = 0; j < DP / 8; ++j)
-        raw[j] = *reinterpret_cast<const u16x8*>(krow + j * 8);
+      for (int i = 0; i < HC; ++i)
 #pragma unroll
-      for (int j = 0; j < DP / 8; ++j) {
-        float k[8];
-#pragma unroll
-        for (int e = 0; e < 8; ++e) k[e] = bf16_to_f32(raw[j][e]);
-#pragma unroll
-        for (int i = 0; i < HC; ++i)
-#pragma unroll
-          for (int e = 0; e < 8; ++e)
-            acc[i] += q_lds[i * DP + j * 8 + e] * k[e];
-      }
-    } else {
-      for (int j = 0; j < Dp; j += 8) {
-        float k[8];
-        ldv<8>(krow + j, k);
-#pragma unroll
-        for (int i = 0; i < HC; ++i)
-#pragma unroll
-          for (int e = 0; e < 8; ++e) acc[i] += q_lds[i * Dp + j + e] * k[e];
-      }
+        for (int e = 0; e < 8; ++e) acc[i] += q_lds[i * Dp + j + e] * k[e];
     }
 #pragma unroll
     for (int i = 0; i < HC; ++i) {
@@ -120,55 +141,108 @@ __global__ __launch_bounds__(NT) void row_scores_kernel(
       }
     }
   }
-  const int wid = threadIdx.x / WAVE, lane = threadIdx.x & (WAVE - 1);
-#pragma unroll
-  for (int i = 0; i < HC; ++i) {
-    const float wm = wave_reduce_max(mx[i]);
-    const float ws = wave_reduce_sum(sm[i] * exp_s<S>(mx[i] - wm));
-    if (lane == 0) {
-      red[0][i][wid] = wm;
-      red[1][i][wid] = ws;
-    }
-  }
-  __syncthreads();
-  if ((int)threadIdx.x < nh) {
-    const int i = threadIdx.x;
-    float M = NEG, L = 0.f;
-    for (int w = 0; w < NWV; ++w) M = fmaxf(M, red[0][i][w]);
-    for (int w = 0; w < NWV; ++w)
-      L += red[1][i][w] * exp_s<S>(red[0][i][w] - M);
-    float* o = ml + (((int64_t)row * m.H + h0 + i) * m.max_parts + part) * 2;
-    o[0] = M;
-    o[1] = L;
-  }
+  store_stats<S, HC>(mx, sm, red, nh, ml, (int64_t)row * m.H + h0,
+                     m.max_parts, part);
 }
 
-// Value pass. w_lds holds the mixed weights of this workgroup's heads for
-// one chunk; positions outside [p0, p1) weigh 0, so V is read in aligned
-// groups of 8 tokens. Threads own value dims (one dim each, strided).
-template <typename S, int HC>
-__global__ __launch_bounds__(NT) void row_values_kernel(
-    S* __restrict__ out, int64_t out_stride, float* __restrict__ tmp,
-    const float* __restrict__ scores, const float* __restrict__ ml,
-    const S* __restrict__ vc, const float* __restrict__ talk,
-    const S* __restrict__ gate, int64_t gate_stride, int E, int nparts,
+// Score pass on MFMA. DT k-steps of 32 (Dp <= 32*DT); HC a multiple of 4.
+template <int DT, int HC>
+__global__ __launch_bounds__(NT) void row_scores_mfma_kernel(
+    float* __restrict__ scores, float* __restrict__ ml,
+    const uint16_t* __restrict__ q, const uint16_t* __restrict__ kc,
+    const float* __restrict__ slopes, float scale, float cap, int Dp,
     RowGeom m) {
-  extern __shared__ float sh[];
-  float* w_lds = sh;                          // [HC][CHUNK + 8]
-  float* M_lds = w_lds + HC * (CHUNK + 8);    // [H]
-  float* I_lds = M_lds + m.H;                 // [H] 1 / denominator
-  float* T_lds = I_lds + m.H;                 // [H][HC] mixing columns
+  __shared__ float red[2][HC][NWV];
   const int row = blockIdx.x, part = blockIdx.z;
   const int g = blockIdx.y / m.hchunks, hc = blockIdx.y % m.hchunks;
   const int HG = m.H / m.G;
   const int h0 = g * HG + hc * HC;
   const int nh = min(HC, HG - hc * HC);
   const int len = m.row_len[row];
-  const int lo = m.window > 0 ? max(0, len - m.window) : 0;
-  const int p0 = lo + part * m.part;
+  const int lo_key = m.window > 0 ? max(0, len - m.window) : 0;
+  const int p0 = lo_key + part * m.part;
   const int p1 = min(len, p0 + m.part);
   if (p0 >= len) return;
-  const int np = cdiv(len - lo, m.part);
+  const int wid = threadIdx.x / WAVE, lane = threadIdx.x & (WAVE - 1);
+  const int lo = lane & 15, hi = lane >> 4;
+
+  // lane lo feeds head lo & 3 of every group of 4
+  u16x8 qf[HC / 4][DT];
+#pragma unroll
+  for (int j = 0; j < HC / 4; ++j)
+#pragma unroll
+    for (int kt = 0; kt < DT; ++kt) {
+      const int h = j * 4 + (lo & 3), d = kt * 32 + hi * 8;
+      qf[j][kt] = h < nh && d < Dp
+                      ? *reinterpret_cast<const u16x8*>(
+                            q + ((int64_t)row * m.H + h0 + h) * Dp + d)
+                      : u16x8{0, 0, 0, 0, 0, 0, 0, 0};
+    }
+  const int* bt =
+      m.bt + (int64_t)(m.row_seq ? m.row_seq[row] : row) * m.bt_stride;
+  const float inv_cap = cap > 0.f ? 1.f / cap : 0.f;
+  float slope[HC], mx[HC], sm[HC];
+#pragma unroll
+  for (int i = 0; i < HC; ++i) {
+    slope[i] = (slopes != nullptr && i < nh) ? slopes[h0 + i] : 0.f;
+    mx[i] = NEG;
+    sm[i] = 0.f;
+  }
+  for (int base = p0 + wid * WAVE; base < p1; base += NWV * WAVE) {
+    u16x8 kf[4][DT];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int tok = min(base + u * 16 + lo, p1 - 1);
+      const uint16_t* kr =
+          kc + (((int64_t)bt[tok / m.bs] * m.G + g) * m.bs + tok % m.bs) * Dp +
+          hi * 8;
+#pragma unroll
+      for (int kt = 0; kt < DT; ++kt)
+        kf[u][kt] = kt * 32 + hi * 8 < Dp
+                        ? *reinterpret_cast<const u16x8*>(kr + kt * 32)
+                        : u16x8{0, 0, 0, 0, 0, 0, 0, 0};
+    }
+    const int tok = base + lane;
+#pragma unroll
+    for (int j = 0; j < HC / 4; ++j) {
+      floatx4 c = floatx4{0, 0, 0, 0};
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+#pragma unroll
+        for (int kt = 0; kt < DT; ++kt) {
+          u16x8 a = (lo >> 2) == u ? qf[j][kt]
+                                   : u16x8{0, 0, 0, 0, 0, 0, 0, 0};
+          c = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+              *reinterpret_cast<bf16x8*>(&a),
+              *reinterpret_cast<bf16x8*>(&kf[u][kt]), c, 0, 0, 0);
+        }
+      if (tok < p1) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int i = j * 4 + r;
+          if (i < nh) {
+            const float s = cap_and_bias<uint16_t>(
+                c[r], scale, cap, inv_cap, slope[i], len - 1 - tok);
+            scores[((int64_t)row * m.H + h0 + i) * m.span + tok - lo_key] = s;
+            const float mn = fmaxf(mx[i], s);
+            sm[i] = sm[i] * __expf(mx[i] - mn) + __expf(s - mn);
+            mx[i] = mn;
+          }
+        }
+      }
+    }
+  }
+  store_stats<uint16_t, HC>(mx, sm, red, nh, ml, (int64_t)row * m.H + h0,
+                            m.max_parts, part);
+}
+
+// Denominators of all heads and this workgroup's rows of the mixing matrix.
+template <typename S, int HC>
+__device__ __forceinline__ void load_mixing(float* M_lds, float* I_lds,
+                                            float* T_lds, const float* ml,
+                                            const float* talk, int row,
+                                            int h0, int nh, int np,
+                                            const RowGeom& m) {
   for (int h = threadIdx.x; h < m.H; h += NT) {
     const float* s = ml + ((int64_t)row * m.H + h) * m.max_parts * 2;
     float M = NEG, L = 0.f;
@@ -186,7 +260,51 @@ __global__ __launch_bounds__(NT) void row_values_kernel(
     T_lds[i] = t;
   }
   __syncthreads();
+}
 
+// w[i] += sum over all heads of talk * softmax weight, for one key whose
+// scores start at s.
+template <typename S, int HC>
+__device__ __forceinline__ void mixed_weights(float (&w)[HC], const float* s,
+                                              const float* M_lds,
+                                              const float* I_lds,
+                                              const float* T_lds,
+                                              const RowGeom& m) {
+#pragma unroll 8
+  for (int h = 0; h < m.H; ++h) {
+    const float p = exp_s<S>(s[(int64_t)h * m.span] - M_lds[h]) * I_lds[h];
+#pragma unroll
+    for (int i = 0; i < HC; ++i) w[i] += T_lds[h * HC + i] * p;
+  }
+}
+
+// Value pass. w_lds holds the mixed weights of this workgroup's heads for
+// one chunk; positions outside [p0, p1) weigh 0, so V is read in aligned
+// groups of 8 tokens. Threads own value dims (one dim each, strided).
+template <typename S, int HC>
+__global__ __launch_bounds__(NT) void row_values_kernel(
+    S* __restrict__ out, int64_t out_stride, float* __restrict__ tmp,
+    const float* __restrict__ scores, const float* __restrict__ ml,
+    const S* __restrict__ vc, const float* __restrict__ talk,
+    const S* __restrict__ gate, int64_t gate_stride, int E, int nparts,
+    RowGeom m) {
+  extern __shared__ __attribute__((aligned(16))) float sh[];
+  float* w_lds = sh;                          // [HC][CHUNK + 8]
+  float* M_lds = w_lds + HC * (CHUNK + 8);    // [H]
+  float* I_lds = M_lds + m.H;                 // [H] 1 / denominator
+  float* T_lds = I_lds + m.H;                 // [H][HC] mixing columns
+  const int row = blockIdx.x, part = blockIdx.z;
+  const int g = blockIdx.y / m.hchunks, hc = blockIdx.y % m.hchunks;
+  const int HG = m.H / m.G;
+  const int h0 = g * HG + hc * HC;
+  const int nh = min(HC, HG - hc * HC);
+  const int len = m.row_len[row];
+  const int lo = m.window > 0 ? max(0, len - m.window) : 0;
+  const int p0 = lo + part * m.part;
+  const int p1 = min(len, p0 + m.part);
+  if (p0 >= len) return;
+  load_mixing<S, HC>(M_lds, I_lds, T_lds, ml, talk, row, h0, nh,
+                     cdiv(len - lo, m.part), m);
   const int* bt =
       m.bt + (int64_t)(m.row_seq ? m.row_seq[row] : row) * m.bt_stride;
   constexpr int ND = 4;                       // dims per thread: E <= 512
@@ -203,16 +321,10 @@ __global__ __launch_bounds__(NT) void row_values_kernel(
       float w[HC];
 #pragma unroll
       for (int i = 0; i < HC; ++i) w[i] = 0.f;
-      if (tok >= p0 && tok < p1) {
-        const float* s = scores + (int64_t)row * m.H * m.span + tok - lo;
-#pragma unroll 4
-        for (int h = 0; h < m.H; ++h) {
-          const float p =
-              exp_s<S>(s[(int64_t)h * m.span] - M_lds[h]) * I_lds[h];
-#pragma unroll
-          for (int i = 0; i < HC; ++i) w[i] += T_lds[h * HC + i] * p;
-        }
-      }
+      if (tok >= p0 && tok < p1)
+        mixed_weights<S, HC>(
+            w, scores + (int64_t)row * m.H * m.span + tok - lo, M_lds, I_lds,
+            T_lds, m);
 #pragma unroll
       for (int i = 0; i < HC; ++i) w_lds[i * (CHUNK + 8) + threadIdx.x] = w[i];
     }
@@ -262,6 +374,122 @@ __global__ __launch_bounds__(NT) void row_values_kernel(
   }
 }
 
+// Value pass on MFMA (bf16). Waves own value tiles of 16 dims, ET of them at
+// most (E <= 32 * ET for the 2 waves).
+template <int ET, int HC>
+__global__ __launch_bounds__(NT) void row_values_mfma_kernel(
+    uint16_t* __restrict__ out, int64_t out_stride, float* __restrict__ tmp,
+    const float* __restrict__ scores, const float* __restrict__ ml,
+    const uint16_t* __restrict__ vc, const float* __restrict__ talk,
+    const uint16_t* __restrict__ gate, int64_t gate_stride, int E, int nparts,
+    RowGeom m) {
+  extern __shared__ __attribute__((aligned(16))) float sh[];
+  constexpr int WPITCH = CHUNK + 8;
+  float* M_lds = sh;                          // [H]
+  float* I_lds = M_lds + m.H;                 // [H] 1 / denominator
+  float* T_lds = I_lds + m.H;                 // [H][HC] mixing columns
+  __shared__ __attribute__((aligned(16))) uint16_t w_hi[HC * WPITCH];
+  __shared__ __attribute__((aligned(16))) uint16_t w_lo[HC * WPITCH];
+  const int row = blockIdx.x, part = blockIdx.z;
+  const int g = blockIdx.y / m.hchunks, hc = blockIdx.y % m.hchunks;
+  const int HG = m.H / m.G;
+  const int h0 = g * HG + hc * HC;
+  const int nh = min(HC, HG - hc * HC);
+  const int len = m.row_len[row];
+  const int lo_key = m.window > 0 ? max(0, len - m.window) : 0;
+  const int p0 = lo_key + part * m.part;
+  const int p1 = min(len, p0 + m.part);
+  if (p0 >= len) return;
+  load_mixing<uint16_t, HC>(M_lds, I_lds, T_lds, ml, talk, row, h0, nh,
+                            cdiv(len - lo_key, m.part), m);
+  const int* bt =
+      m.bt + (int64_t)(m.row_seq ? m.row_seq[row] : row) * m.bt_stride;
+  const int wid = threadIdx.x / WAVE, lane = threadIdx.x & (WAVE - 1);
+  const int lo = lane & 15, hi = lane >> 4;
+  floatx4 acc[ET];
+#pragma unroll
+  for (int c = 0; c < ET; ++c) acc[c] = floatx4{0, 0, 0, 0};
+
+  for (int base = p0 & ~7; base < p1; base += CHUNK) {
+    const int n32 = (min(CHUNK, p1 - base) + 31) / 32;
+    {
+      const int tok = base + threadIdx.x;
+      float w[HC];
+#pragma unroll
+      for (int i = 0; i < HC; ++i) w[i] = 0.f;
+      if (tok >= p0 && tok < p1)
+        mixed_weights<uint16_t, HC>(
+            w, scores + (int64_t)row * m.H * m.span + tok - lo_key, M_lds,
+            I_lds, T_lds, m);
+#pragma unroll
+      for (int i = 0; i < HC; ++i) {
+        const uint16_t h = f32_to_bf16(w[i]);
+        w_hi[i * WPITCH + threadIdx.x] = h;
+        w_lo[i * WPITCH + threadIdx.x] = f32_to_bf16(w[i] - bf16_to_f32(h));
+      }
+    }
+    __syncthreads();
+#pragma unroll 2
+    for (int j = 0; j < n32; ++j) {
+      const int t8 = base + j * 32 + hi * 8;
+      const int tv = min(t8, (p1 - 1) & ~7);
+      const uint16_t* vp =
+          vc + (((int64_t)bt[tv / m.bs] * m.G + g) * E + lo) * m.bs +
+          tv % m.bs;
+      u16x8 vf[ET];
+#pragma unroll
+      for (int c = 0; c < ET; ++c) {
+        const int dim0 = (c * NWV + wid) * 16;
+        vf[c] = dim0 + lo < E ? *reinterpret_cast<const u16x8*>(
+                                    vp + (int64_t)dim0 * m.bs)
+                              : u16x8{0, 0, 0, 0, 0, 0, 0, 0};
+      }
+      u16x8 ah = u16x8{0, 0, 0, 0, 0, 0, 0, 0}, al = ah;
+      if (lo < HC) {
+        ah = *reinterpret_cast<const u16x8*>(w_hi + lo * WPITCH + j * 32 +
+                                             hi * 8);
+        al = *reinterpret_cast<const u16x8*>(w_lo + lo * WPITCH + j * 32 +
+                                             hi * 8);
+      }
+      const bool tail = base + j * 32 + 32 > p1;
+#pragma unroll
+      for (int c = 0; c < ET; ++c) {
+        if (tail) {                           // stale slots: not even 0 * x
+#pragma unroll
+          for (int e = 0; e < 8; ++e)
+            if (t8 + e >= p1) vf[c][e] = 0;
+        }
+        const bf16x8 b = *reinterpret_cast<bf16x8*>(&vf[c]);
+        acc[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+            *reinterpret_cast<bf16x8*>(&al), b, acc[c], 0, 0, 0);
+        acc[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+            *reinterpret_cast<bf16x8*>(&ah), b, acc[c], 0, 0, 0);
+      }
+    }
+    __syncthreads();
+  }
+#pragma unroll
+  for (int c = 0; c < ET; ++c) {
+    const int dim = (c * NWV + wid) * 16 + lo;
+    if (dim >= E) continue;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int i = hi * 4 + r;
+      if (i >= nh) continue;
+      const int h = h0 + i;
+      if (nparts == 1) {
+        float o = acc[c][r];
+        if (gate != nullptr)
+          o /= 1.f + __expf(-bf16_to_f32(gate[row * gate_stride + h]));
+        out[row * out_stride + (int64_t)h * E + dim] = f32_to_bf16(o);
+      } else {
+        tmp[(((int64_t)row * m.H + h) * m.max_parts + part) * E + dim] =
+            acc[c][r];
+      }
+    }
+  }
+}
+
 template <typename S>
 __global__ __launch_bounds__(NT) void row_reduce_kernel(
     S* __restrict__ out, int64_t out_stride, const float* __restrict__ tmp,
@@ -300,14 +528,9 @@ void launch_rows(RowCall<S>& c) {
   c.m.hchunks = cdiv(c.m.H / c.m.G, HC);
   const dim3 grid(c.R, c.m.G * c.m.hchunks, c.nparts);
   const size_t q_bytes = (size_t)HC * c.D * sizeof(float);
-#define HELIX_SCORES(DP)                                                     \
-  hipLaunchKernelGGL((row_scores_kernel<S, DP, HC>), grid, dim3(NT),         \
-                     q_bytes, c.stream, c.scores, c.ml, c.q, c.kc, c.slopes, \
-                     c.scale, c.cap, c.D, c.m)
-  if (c.D == 128 && sizeof(S) == 2) HELIX_SCORES(128);
-  else if (c.D == 64 && sizeof(S) == 2) HELIX_SCORES(64);
-  else HELIX_SCORES(0);
-#undef HELIX_SCORES
+  hipLaunchKernelGGL((row_scores_kernel<S, HC>), grid, dim3(NT), q_bytes,
+                     c.stream, c.scores, c.ml, c.q, c.kc, c.slopes, c.scale,
+                     c.cap, c.D, c.m);
   const size_t v_bytes =
       (HC * (CHUNK + 8) + (2 + HC) * c.m.H) * sizeof(float);
   hipLaunchKernelGGL((row_values_kernel<S, HC>), grid, dim3(NT), v_bytes,
@@ -319,9 +542,43 @@ void launch_rows(RowCall<S>& c) {
                        c.gate_stride, c.E, c.m);
 }
 
+template <int HC>
+void launch_rows_mfma(RowCall<uint16_t>& c) {
+  c.m.hchunks = cdiv(c.m.H / c.m.G, HC);
+  const dim3 grid(c.R, c.m.G * c.m.hchunks, c.nparts);
+#define HELIX_SCORES(DT)                                                     \
+  hipLaunchKernelGGL((row_scores_mfma_kernel<DT, HC>), grid, dim3(NT), 0,    \
+                     c.stream, c.scores, c.ml, c.q, c.kc, c.slopes, c.scale, \
+                     c.cap, c.D, c.m)
+  if (c.D <= 64) HELIX_SCORES(2);
+  else HELIX_SCORES(4);
+#undef HELIX_SCORES
+  const size_t bytes = (2 + HC) * c.m.H * sizeof(float);
+#define HELIX_VALUES(ET)                                                     \
+  hipLaunchKernelGGL((row_values_mfma_kernel<ET, HC>), grid, dim3(NT),       \
+                     bytes, c.stream, c.out, c.out_stride, c.tmp, c.scores,  \
+                     c.ml, c.vc, c.talk, c.gate, c.gate_stride, c.E,         \
+                     c.nparts, c.m)
+  if (c.E <= 64) HELIX_VALUES(2);
+  else if (c.E <= 128) HELIX_VALUES(4);
+  else HELIX_VALUES(8);
+#undef HELIX_VALUES
+  if (c.nparts > 1)
+    hipLaunchKernelGGL((row_reduce_kernel<uint16_t>), dim3(c.R, c.m.H),
+                       dim3(NT), 0, c.stream, c.out, c.out_stride, c.tmp,
+                       c.gate, c.gate_stride, c.E, c.m);
+}
+
 template <typename S>
 void dispatch_rows(RowCall<S>& c) {
   const int HG = c.m.H / c.m.G;
+  if constexpr (sizeof(S) == 2) {
+    if (c.D <= 128 && c.E <= 256) {
+      if (HG <= 4) launch_rows_mfma<4>(c);
+      else launch_rows_mfma<8>(c);
+      return;
+    }
+  }
   if (HG == 1) launch_rows<S, 1>(c);
   else if (HG == 2) launch_rows<S, 2>(c);
   else if (HG <= 4) launch_rows<S, 4>(c);
@@ -390,7 +647,7 @@ void talk_attn_rows(torch::Tensor out, torch::Tensor q, torch::Tensor kc,
 
   // partitions: enough workgroups for the chip, in whole QUANTs
   const int HG = H / G;
-  const int hc = HG == 1 ? 1 : HG == 2 ? 2 : HG <= 4 ? 4 : 8;
+  const int hc = HG <= 4 ? 4 : 8;
   const int wg = R * G * cdiv(HG, hc);
   int nparts = std::max(1, 1024 / std::max(1, wg));
   nparts = std::min<int>({nparts, cdiv(max_keys, QUANT), (int)max_parts});
