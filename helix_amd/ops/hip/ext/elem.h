@@ -59,6 +59,14 @@ __device__ __forceinline__ void stv(float* p, const float* in) {
   }
 }
 
+// Two floats -> two bf16 (round to nearest even), a in the low half; one
+// v_cvt_pk_bf16_f32 on gfx950.
+__device__ __forceinline__ uint32_t pack_bf16(float a, float b) {
+  typedef __attribute__((ext_vector_type(2))) __bf16 bf16x2;
+  const bf16x2 v = __builtin_convertvector(f32x2{a, b}, bf16x2);
+  return __builtin_bit_cast(uint32_t, v);
+}
+
 // exp / tanh per storage type: the fp32 build takes the library functions,
 // the bf16 build the native exponential (absolute error of the capped
 // score below 1e-5 for caps up to a few hundred).

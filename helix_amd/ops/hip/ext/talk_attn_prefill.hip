@@ -197,6 +197,8 @@ __global__ __launch_bounds__(256) void talk_stats_kernel(PrefillArgs a) {
     w.load_k(k0, row0, w.kvh[0]);
     w.load_k(k1, row1, w.kvh[0]);
     const int64_t cur0 = row0, cur1 = row1;
+    const int idist0 = w.dist(0, kb + w.lo);
+    const float dist0 = (float)idist0;
     row0 = w.key_row(kb + KT + w.lo);         // next tile's page lookup
     row1 = w.key_row(kb + KT + 16 + w.lo);
 #pragma unroll
@@ -208,12 +210,11 @@ __global__ __launch_bounds__(256) void talk_stats_kernel(PrefillArgs a) {
       const floatx4 d0 = w.dot(i, k0), d1 = w.dot(i, k1);
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        const int dd = w.dist(r, kb + w.lo);
-        float s0 = score(d0[r], w.slope2[i], (float)dd);
-        float s1 = score(d1[r], w.slope2[i], (float)(dd - 16));
+        float s0 = score(d0[r], w.slope2[i], dist0 + (float)r);
+        float s1 = score(d1[r], w.slope2[i], dist0 + (float)(r - 16));
         if (!full) {
-          if (w.masked(dd)) s0 = NEG;
-          if (w.masked(dd - 16)) s1 = NEG;
+          if (w.masked(idist0 + r)) s0 = NEG;
+          if (w.masked(idist0 + r - 16)) s1 = NEG;
         }
         const float mn = fmaxf(mx[i][r], fmaxf(s0, s1));
         sm[i][r] = sm[i][r] * __builtin_amdgcn_exp2f(mx[i][r] - mn) +
@@ -308,11 +309,13 @@ __global__ __launch_bounds__(512) void talk_values_kernel(PrefillArgs a) {
 #pragma unroll 1
     for (int sub = 0; sub < 2; ++sub) {
       const int64_t row = w.key_row(kb + sub * 16 + lo);
+      const int idist0 = w.dist(0, kb + sub * 16 + lo);
+      const float dist0 = (float)idist0;
       u16x8 kf[DT];
       constexpr int HP = HPW < 2 ? 1 : 2;     // heads stored together
 #pragma unroll
       for (int i0 = 0; i0 < HPW; i0 += HP) {
-        uint32_t ph[4], pl[4];
+        float p[HP][4];
 #pragma unroll
         for (int j = 0; j < HP; ++j) {
           const int i = i0 + j;
@@ -322,14 +325,9 @@ __global__ __launch_bounds__(512) void talk_values_kernel(PrefillArgs a) {
               lse_lds + min(hbase + i, H - 1) * QT + hi * 4);
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
-            const int dd = w.dist(r, kb + sub * 16 + lo);
-            const float s = score(d[r], w.slope2[i], (float)dd);
-            float p = __builtin_amdgcn_exp2f(s - lse[r]);
-            if (!full && w.masked(dd)) p = 0.f;
-            const uint32_t vh = f32_to_bf16(p);
-            const uint32_t vl = f32_to_bf16(p - bf16_to_f32(vh));
-            ph[r] = j == 0 ? vh : ph[r] | vh << 16;
-            pl[r] = j == 0 ? vl : pl[r] | vl << 16;
+            p[j][r] = __builtin_amdgcn_exp2f(
+                score(d[r], w.slope2[i], dist0 + (float)r) - lse[r]);
+            if (!full && w.masked(idist0 + r)) p[j][r] = 0.f;
           }
         }
         // (row, key) pair -> its heads, two bf16 terms
@@ -337,12 +335,17 @@ __global__ __launch_bounds__(512) void talk_values_kernel(PrefillArgs a) {
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int pos = ((hi * 4 + r) * KT + sub * 16 + lo) * PP + h;
+          const float p0 = p[0][r], p1 = HP == 2 ? p[HP - 1][r] : 0.f;
+          const uint32_t ph = pack_bf16(p0, p1);
+          const uint32_t pl =
+              pack_bf16(p0 - __builtin_bit_cast(float, ph << 16),
+                        p1 - __builtin_bit_cast(float, ph & 0xffff0000u));
           if (HP == 2 && (FAST || h + 1 < H)) {
-            *reinterpret_cast<uint32_t*>(p_hi + pos) = ph[r];
-            *reinterpret_cast<uint32_t*>(p_lo + pos) = pl[r];
+            *reinterpret_cast<uint32_t*>(p_hi + pos) = ph;
+            *reinterpret_cast<uint32_t*>(p_lo + pos) = pl;
           } else if (FAST || h < H) {
-            p_hi[pos] = (uint16_t)ph[r];
-            p_lo[pos] = (uint16_t)pl[r];
+            p_hi[pos] = (uint16_t)ph;
+            p_lo[pos] = (uint16_t)pl;
           }
         }
       }
@@ -372,13 +375,15 @@ __global__ __launch_bounds__(512) void talk_values_kernel(PrefillArgs a) {
               *reinterpret_cast<const bf16x8*>(
                   t_lds + ((2 + m) * WAVE + lane) * 8), ph, c, 0, 0, 0);
         c = __builtin_amdgcn_mfma_f32_16x16x32_bf16(th, ph, c, 0, 0, 0);
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int h = m * 16 + hi * 4 + r;
-          if (h < H)
-            w_lds[(h * QT + grp / 2) * WP + (grp & 1) * 16 + lo] =
-                f32_to_bf16(c[r]);
-        }
+        const uint32_t c01 = pack_bf16(c[0], c[1]);
+        const uint32_t c23 = pack_bf16(c[2], c[3]);
+        uint16_t* wp = w_lds + ((m * 16 + hi * 4) * QT + grp / 2) * WP +
+                       (grp & 1) * 16 + lo;
+        const int left = H - (m * 16 + hi * 4);
+        if (left > 0) wp[0] = (uint16_t)c01;
+        if (left > 1) wp[QT * WP] = (uint16_t)(c01 >> 16);
+        if (left > 2) wp[2 * QT * WP] = (uint16_t)c23;
+        if (left > 3) wp[3 * QT * WP] = (uint16_t)(c23 >> 16);
       }
     }
     __syncthreads();

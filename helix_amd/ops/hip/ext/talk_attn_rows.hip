@@ -423,9 +423,10 @@ __global__ __launch_bounds__(NT) void row_values_mfma_kernel(
             I_lds, T_lds, m);
 #pragma unroll
       for (int i = 0; i < HC; ++i) {
-        const uint16_t h = f32_to_bf16(w[i]);
-        w_hi[i * WPITCH + threadIdx.x] = h;
-        w_lo[i * WPITCH + threadIdx.x] = f32_to_bf16(w[i] - bf16_to_f32(h));
+        const uint32_t h = pack_bf16(w[i], 0.f);
+        w_hi[i * WPITCH + threadIdx.x] = (uint16_t)h;
+        w_lo[i * WPITCH + threadIdx.x] = (uint16_t)pack_bf16(
+            w[i] - __builtin_bit_cast(float, h << 16), 0.f);
       }
     }
     __syncthreads();
