@@ -578,8 +578,9 @@ class LLMEngine:
         return victim
 
     def _schedule_decode(self) -> List[Sequence]:
-        """Running sequences with a page for their next token; preempts
-        when the pool is exhausted."""
+        """Running sequences with a page for their next token, staged in
+        the persistent host arrays; preempts (newest first, so never a row
+        that is already staged) when the pool is exhausted."""
         bs = self.cfg.block_size
         batch = []
         preempted = set()                     # ids preempted this step
@@ -601,17 +602,23 @@ class LLMEngine:
                 seq.block_table.extend(self.kv.allocator.allocate(1))
                 self._bt_np[seq.row, len(seq.block_table) - 1] = \
                     seq.block_table[-1]
-            if seq.seq_id not in preempted:
-                batch.append(seq)
-        return [s for s in batch if s.seq_id not in preempted]
+            if seq.seq_id in preempted:
+                continue
+            # stage the row right here: one pass over the batch a step
+            i = len(batch)
+            self._ids_np[i] = seq.last_token
+            self._pos_np[i] = pos
+            self._slots_np[i] = seq.block_table[nblk - 1] * bs + pos % bs
+            self._lens_np[i] = pos + 1
+            self._rows_np[i] = seq.row
+            batch.append(seq)
+        return batch
 
     def _run_decode(self):
         batch = self._schedule_decode()
         if not batch:
             return []
-        spans = [Span(s, s.total_len - 1, s.total_len, [s.last_token])
-                 for s in batch]
-        logits = self._decode_logits(self._fill_decode(spans))
+        logits = self._decode_logits(len(batch))
         tokens = self._sample(batch, logits)
         return list(zip(batch, tokens))
 
