@@ -115,6 +115,8 @@ class LLMEngine:
                 raise ValueError("block_size must be a multiple of 8")
         elif self.dtype != torch.bfloat16:
             raise ValueError(f"{cfg.model} is served in bfloat16")
+        if self.dtype == torch.float32:
+            torch.set_float32_matmul_precision("highest")   # no TF32 modes
         if model is None:
             model = registry.build_model(cfg.model, self.dtype, self.device,
                                          cfg.seed, tp_size, tp_rank,

@@ -598,13 +598,18 @@ def test_greedy_generation(folders, dev, mixed):
 
 
 @pytest.mark.parametrize("dev", DEVICES)
-def test_long_decode(folders, dev):
+@pytest.mark.parametrize("name,dtype,n,cuts", [
+    ("varied", "float32", 300, [5] + [1] * 295),
+    ("varied", "bfloat16", 300, [5] + [1] * 295),
+    ("wide", "bfloat16", 560, [2, 300, 198] + [1] * 60),
+    ("wide", "float32", 560, [500] + [1] * 60)])
+def test_long_decode(folders, dev, name, dtype, n, cuts):
     """Far past every window, page by page."""
-    folder, cfg, w = folders["varied"]
-    ids = prompt(cfg, 300, 8)
-    eng = engine_for(folder, dev, "float32")
-    got = run_cut(eng, "a", ids, [5] + [1] * 295)
-    check_rows(got, want_logits("varied", cfg, w, ids), "float32")
+    folder, cfg, w = folders[name]
+    ids = prompt(cfg, n, 8)
+    eng = engine_for(folder, dev, dtype)
+    got = run_cut(eng, "a", ids, cuts)
+    check_rows(got, want_logits(name, cfg, w, ids), dtype)
 
 
 def test_model_tests_notice_mistakes(folders):
