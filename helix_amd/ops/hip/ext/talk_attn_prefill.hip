@@ -556,7 +556,9 @@ void talk_attn_prefill(torch::Tensor out, torch::Tensor q, torch::Tensor kc,
   a.E = E;
   a.bs = bs;
   auto stream = at::hip::getCurrentHIPStream();
-  if (H <= 8) by_size<1>(a, max_q, B, stream);
-  else if (H <= 16) by_size<2>(a, max_q, B, stream);
-  else by_size<4>(a, max_q, B, stream);
+  // heads of a wave should share their K and V rows; 8 waves at most
+  const int HG = H / G;
+  if (HG % 4 == 0 || H > 16) by_size<4>(a, max_q, B, stream);
+  else if (HG % 2 == 0 || H > 8) by_size<2>(a, max_q, B, stream);
+  else by_size<1>(a, max_q, B, stream);
 }

@@ -171,6 +171,8 @@ ATTN = [
     (32, 8, 128, 128, 45, 12.0, True, True),
     (8, 2, 64, 64, 31, 9.0, True, True),
     (32, 4, 64, 64, 0, 9.0, True, True),
+    (12, 6, 64, 64, 31, 9.0, True, True),
+    (6, 6, 128, 128, 0, 9.0, True, True),
     (24, 24, 24, 40, 1, 30.0, True, True),
     (40, 8, 32, 32, 37, 8.0, True, True),      # beyond the MFMA kernel
     (3, 1, 144, 136, 45, 50.0, True, True),     # beyond the MFMA kernel
