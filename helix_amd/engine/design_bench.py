@@ -129,7 +129,7 @@ def kernels(z: ZederaxConfig, device, decode_batch: int = 256,
                         torch.rand(H, device=device),
                         torch.randn(H, H, device=device) * 0.2)
 
-    # --- decode attention: K and V of every row once
+    # --- decode attention: the visible K and V of every row once
     for B, L in ((decode_batch, decode_len), (64, 4096), (1, 4096)):
         nb = L // bs
         bt = torch.randperm(B * nb, device=device).int().view(B, nb)
@@ -140,12 +140,12 @@ def kernels(z: ZederaxConfig, device, decode_batch: int = 256,
                          device=device)
         t = _time(lambda: ops.talk_attn_rows(o, q, (kc, vc), bt, lens, L, tp,
                                              gate, workspace=ws))
-        nbytes = 2.0 * B * L * G * (D + E)
+        nbytes = 2.0 * B * tp.max_keys(L) * G * (D + E)
         new = _row(t, nbytes)
         vl = vc.view(B * nb, G, bs, E)
         lws = ops.decode_workspace(B, H, D, L, device)
         t = _time(lambda: ops.paged_attn_decode(q, kc, vl, bt, lens, m.scale,
-                                                lws, L))
+                                                lws, L, window=m.window))
         pair(f"decode_attention_b{B}_l{L}", new, _row(t, nbytes))
         del kc, vc, vl
 

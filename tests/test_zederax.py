@@ -709,6 +709,24 @@ def test_registry(tmp_path, folders):
         assert torch.equal(dst, w[n].float()), n
 
 
+def test_registry_loads_llama_folders(tmp_path):
+    from helix_amd.engine.weights import save_sharded
+    from helix_amd.models.llama import PRESETS as LLAMA, LlamaForCausalLM
+    c = LLAMA["tiny-qwen"]
+    (tmp_path / "config.json").write_text(json.dumps({
+        "architectures": ["Qwen2ForCausalLM"], "vocab_size": c.vocab_size,
+        "hidden_size": c.hidden_size, "num_hidden_layers": c.num_layers,
+        "intermediate_size": c.intermediate_size, "num_attention_heads": 4,
+        "num_key_value_heads": 2, "rope_theta": 10000.0, "rms_norm_eps": 1e-5,
+        "max_position_embeddings": 512}))
+    src = LlamaForCausalLM(c).init_random(5)
+    save_sharded(src, str(tmp_path))
+    m = registry.build_model(str(tmp_path), F32, torch.device("cpu"))
+    assert m.cfg.attention_bias and m.cfg.sliding_window == 0
+    for (n, a), (_, b) in zip(src.named_parameters(), m.named_parameters()):
+        assert torch.equal(a, b), n
+
+
 def test_checkpoint_errors(tmp_path, folders):
     from safetensors.torch import save_file
     folder, cfg, w = folders["varied"]
