@@ -21,7 +21,8 @@ from helix_amd import ops
 from helix_amd.engine.kv_cache import KVCache, chain_hash
 from helix_amd.engine.sampling_params import SamplingParams
 from helix_amd.models import registry
-from helix_amd.models.meta import DecodeMeta, MixedMeta, PrefillMeta
+from helix_amd.models.meta import (DecodeMeta, MixedMeta, PrefillMeta,
+                                   StateLayer)
 
 _SEED_MIX = 0x9E3779B97F4A7C15
 
@@ -41,7 +42,8 @@ class Sequence:
     output_ids: List[int] = field(default_factory=list)
     status: SeqStatus = SeqStatus.WAITING
     block_table: List[int] = field(default_factory=list)
-    row: int = -1                          # persistent block-table row slot
+    row: int = -1                          # persistent slot: block-table
+                                           # row and recurrent state
     cached_prefix: int = 0                 # tokens served from prefix cache
     block_hashes: List[bytes] = field(default_factory=list)
     arrival_time: float = field(default_factory=time.monotonic)
@@ -127,12 +129,17 @@ class LLMEngine:
         self.model = model
 
         kv_layers = self.model_cfg.kv_layers(tp_size)
+        # A cached page says nothing about the recurrent state at its end,
+        # so models that have one compute every prompt from its start.
+        self.prefix_caching = cfg.enable_prefix_caching and not any(
+            isinstance(l, StateLayer) for l in kv_layers)
         kv_dtype = torch.uint8 if cfg.kv_cache_dtype == "fp8" else self.dtype
         num_blocks = cfg.kv_cache_blocks
         if num_blocks is None:
             num_blocks = self._auto_kv_blocks(kv_layers, kv_dtype)
         self.kv = KVCache.for_layers(kv_layers, cfg.block_size, num_blocks,
-                                     self.device, dtype=kv_dtype)
+                                     self.device, dtype=kv_dtype,
+                                     state_slots=cfg.max_num_seqs)
         self.waiting: List[Sequence] = []
         self.running: List[Sequence] = []
         self.seqs: Dict[str, Sequence] = {}
@@ -192,6 +199,8 @@ class LLMEngine:
         budget = int(total * self.cfg.gpu_memory_utilization
                      - (total - free))
         budget -= self.model_cfg.activation_bytes(self.cfg.max_prefill_tokens)
+        budget -= KVCache.state_bytes(kv_layers, self.cfg.max_num_seqs,
+                                      kv_dtype)
         budget = max(budget, 1 << 28)
         n = KVCache.blocks_for_bytes(budget, 0, 0, 0, self.cfg.block_size,
                                      kv_dtype, kv_layers)
@@ -283,7 +292,7 @@ class LLMEngine:
             matched: List[int] = []
             if first:
                 # prefix-cache match (chain hashes over full blocks)
-                if self.cfg.enable_prefix_caching:
+                if self.prefix_caching:
                     if not seq.block_hashes:
                         h = b""
                         for i in range(L // bs):
@@ -370,10 +379,13 @@ class LLMEngine:
                            max_seqlen=int(lens.max()),
                            slot_mapping=dev_t(slots, np.int64),
                            positions=dev_t(pos, np.int64),
-                           max_len=int(ends.max()))
+                           max_len=int(ends.max()),
+                           state_slots=dev_t(rows, np.int32),
+                           starts=starts, ends=ends, block_size=bs)
         if self.model.paged_prefill:
             nb = -(-meta.max_len // bs)
-            meta.block_tables = dev_t(self._bt_np[rows, :nb], np.int32)
+            meta.host_tables = self._bt_np[rows, :nb]
+            meta.block_tables = dev_t(meta.host_tables, np.int32)
             meta.seq_lens = dev_t(ends, np.int32)
             meta.row_seq = dev_t(which, np.int32)
             meta.row_len = dev_t(pos + 1, np.int32)
@@ -412,7 +424,9 @@ class LLMEngine:
             seq_lens=torch.from_numpy(self._lens_np[:B].copy()).to(dev),
             slot_mapping=torch.from_numpy(self._slots_np[:B].copy()).to(dev),
             positions=torch.from_numpy(self._pos_np[:B].copy()).to(dev),
-            max_len=max_len, workspace=self.decode_ws)
+            max_len=max_len, workspace=self.decode_ws,
+            state_slots=torch.from_numpy(
+                self._rows_np[:B].astype(np.int32)).to(dev))
 
     def _decode_logits(self, B: int) -> torch.Tensor:
         """One decode step over the B staged rows -> logits [B, V]."""
@@ -420,7 +434,7 @@ class LLMEngine:
             bt_np, max_len = self._decode_tables(B)
             return self.graph_runner.run(
                 self._ids_np[:B], self._pos_np[:B], self._slots_np[:B],
-                bt_np, self._lens_np[:B], max_len)
+                bt_np, self._lens_np[:B], max_len, self._rows_np[:B])
         meta = self._decode_meta(B)
         ids = torch.from_numpy(self._ids_np[:B].copy()).to(self.device)
         return self.model.compute_logits(
@@ -481,7 +495,7 @@ class LLMEngine:
         logits = self.run_spans(spans, [[len(s.ids) - 1] for s in spans])
         # register this batch's newly COMPLETED full blocks in the
         # prefix cache (partial chunks register only what they wrote)
-        if self.cfg.enable_prefix_caching:
+        if self.prefix_caching:
             for seq in batch:
                 T = targets.get(seq.seq_id, len(seq.prompt_ids))
                 start = seq.cached_prefix // bs

@@ -38,6 +38,9 @@ class CUDAGraphRunner:
         self.in_bt = torch.zeros(B, self.max_blocks, dtype=torch.int32,
                                  device=device)
         self.in_lens = torch.ones(B, dtype=torch.int32, device=device)
+        # recurrent-state slots; -1 (pad rows, capture) leaves states alone
+        self.in_state = torch.full((B,), -1, dtype=torch.int32,
+                                   device=device)
         # pinned host staging (one DMA per field per step); the event says
         # when the last step's copies are through and it may be refilled
         self.staged = torch.cuda.Event()
@@ -45,6 +48,8 @@ class CUDAGraphRunner:
         self.h_pos = torch.zeros(B, dtype=torch.int64, pin_memory=True)
         self.h_slots = torch.zeros(B, dtype=torch.int64, pin_memory=True)
         self.h_lens = torch.ones(B, dtype=torch.int32, pin_memory=True)
+        self.h_state = torch.full((B,), -1, dtype=torch.int32,
+                                  pin_memory=True)
         self.h_bt = torch.zeros(B, self.max_blocks, dtype=torch.int32,
                                 pin_memory=True)
 
@@ -68,8 +73,11 @@ class CUDAGraphRunner:
             slot_mapping=self.in_slots[:nb],
             positions=self.in_pos[:nb],
             max_len=lb,
-            workspace=self.workspace)
+            workspace=self.workspace,
+            state_slots=self.in_state[:nb])
         ids = self.in_ids[:nb]
+        # the warm-up runs repeat a step: harmless for pages, not for states
+        self.in_state.fill_(-1)
         # Warm up on a side stream (allocator state, lazy inits).
         s = torch.cuda.Stream()
         s.wait_stream(torch.cuda.current_stream())
@@ -91,7 +99,7 @@ class CUDAGraphRunner:
         return {"graph": g, "logits": logits}
 
     def run(self, input_ids, positions, slots, block_tables, seq_lens,
-            max_len: int) -> torch.Tensor:
+            max_len: int, state_slots=None) -> torch.Tensor:
         """All args numpy arrays (or lists); returns logits[:B]."""
         B = len(input_ids)
         nb = self.batch_bucket(B)
@@ -106,6 +114,10 @@ class CUDAGraphRunner:
         self.h_slots[:nb] = -1
         self.h_lens[:nb] = 1
         self.h_bt[:nb].zero_()
+        self.h_state[:nb] = -1
+        if state_slots is not None:
+            self.h_state[:B] = torch.as_tensor(state_slots,
+                                               dtype=torch.int32)
         self.h_ids[:B] = torch.as_tensor(input_ids, dtype=torch.int64)
         self.h_pos[:B] = torch.as_tensor(positions, dtype=torch.int64)
         self.h_slots[:B] = torch.as_tensor(slots, dtype=torch.int64)
@@ -118,10 +130,11 @@ class CUDAGraphRunner:
         self.in_slots[:nb].copy_(self.h_slots[:nb], non_blocking=True)
         self.in_lens[:nb].copy_(self.h_lens[:nb], non_blocking=True)
         self.in_bt[:nb].copy_(self.h_bt[:nb], non_blocking=True)
-        self.staged.record()
 
         if key not in self.graphs:
             self.graphs[key] = self._capture(nb, lb)
+        self.in_state[:nb].copy_(self.h_state[:nb], non_blocking=True)
+        self.staged.record()
         entry = self.graphs[key]
         entry["graph"].replay()
         return entry["logits"][:B]

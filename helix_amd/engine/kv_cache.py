@@ -11,7 +11,7 @@ from typing import Dict, List, Optional, Sequence
 
 import torch
 
-from helix_amd.models.meta import KVLayer
+from helix_amd.models.meta import KVLayer, StateLayer
 
 
 def chain_hash(prev: bytes, tokens: List[int]) -> bytes:
@@ -110,18 +110,24 @@ class BlockAllocator:
 class KVCache:
     """Per-model paged KV storage: one (K, V) pair of page tensors per
     layer. Uniform models have K and V as [num_blocks, Hkv, block_size,
-    head_dim]; `layers` gives each layer its own geometry (KVLayer)."""
+    head_dim]; `layers` gives each layer its own geometry (KVLayer).
+    Recurrent layers (StateLayer) have no pages: their tensors hold one
+    entry per sequence slot."""
 
     def __init__(self, num_layers: int, num_kv_heads: int, head_dim: int,
                  block_size: int, num_blocks: int, device,
                  dtype=torch.bfloat16,
-                 layers: Optional[Sequence[KVLayer]] = None):
+                 layers: Optional[Sequence] = None,
+                 state_slots: int = 0):
         if layers is None:
             layers = [KVLayer(num_kv_heads, head_dim, head_dim)] * num_layers
         self.block_size = block_size
         self.num_blocks = num_blocks
         self.layers = list(layers)
         self.caches = [
+            tuple(torch.zeros(state_slots, *shape, dtype=dt or dtype,
+                              device=device) for shape, dt in l.tensors)
+            if isinstance(l, StateLayer) else
             tuple(torch.zeros(num_blocks, *shape, dtype=dtype, device=device)
                   for shape in (l.k_shape(block_size), l.v_shape(block_size)))
             for l in self.layers]
@@ -129,9 +135,17 @@ class KVCache:
 
     @classmethod
     def for_layers(cls, layers: Sequence[KVLayer], block_size: int,
-                   num_blocks: int, device, dtype=torch.bfloat16):
+                   num_blocks: int, device, dtype=torch.bfloat16,
+                   state_slots: int = 0):
         return cls(len(layers), 0, 0, block_size, num_blocks, device, dtype,
-                   layers=layers)
+                   layers=layers, state_slots=state_slots)
+
+    @staticmethod
+    def state_bytes(layers: Sequence, slots: int,
+                    dtype=torch.bfloat16) -> int:
+        """Memory of the recurrent state of `slots` sequences."""
+        return slots * sum(l.bytes_per_slot(dtype) for l in layers
+                           if isinstance(l, StateLayer))
 
     @staticmethod
     def block_bytes(num_layers: int, num_kv_heads: int, head_dim: int,
@@ -141,12 +155,15 @@ class KVCache:
             layers = [KVLayer(num_kv_heads, head_dim, head_dim)] * num_layers
         el = torch.empty(0, dtype=dtype).element_size()
         return el * block_size * sum(l.num_kv_heads * (l.k_dim + l.v_dim)
-                                     for l in layers)
+                                     for l in layers
+                                     if isinstance(l, KVLayer))
 
     @staticmethod
     def blocks_for_bytes(budget: int, num_layers: int, num_kv_heads: int,
                          head_dim: int, block_size: int,
                          dtype=torch.bfloat16,
                          layers: Optional[Sequence[KVLayer]] = None) -> int:
-        return max(0, budget // KVCache.block_bytes(
-            num_layers, num_kv_heads, head_dim, block_size, dtype, layers))
+        per_block = KVCache.block_bytes(num_layers, num_kv_heads, head_dim,
+                                        block_size, dtype, layers)
+        # layers without pages: blocks only count tokens
+        return max(0, budget // max(per_block, block_size))

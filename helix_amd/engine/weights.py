@@ -9,7 +9,8 @@ import glob
 import json
 import logging
 import os
-from typing import Dict, Iterator, Tuple
+from dataclasses import dataclass
+from typing import Callable, Dict, Iterator, List, Tuple
 
 import torch
 
@@ -199,11 +200,28 @@ def load_llama_weights(model, ckpt_dir: str, use_async: bool = True):
     return loaded
 
 
+@dataclass
+class Placement:
+    """Where a checkpoint tensor goes when that is not one view of its own
+    shape: into padded rows, or into several layouts. parts: (destination,
+    function of the stored tensor)."""
+    shape: Tuple[int, ...]
+    parts: List[Tuple[torch.Tensor, Callable]]
+
+    @property
+    def device(self):
+        return self.parts[0][0].device
+
+    def copy_(self, src: torch.Tensor, copy: Callable = torch.Tensor.copy_):
+        for dst, fn in self.parts:
+            copy(dst, fn(src))
+
+
 @torch.inference_mode()
 def load_mapped_weights(model, ckpt_dir: str, use_async: bool = True) -> int:
     """Load a checkpoint through the model's own name map
-    (checkpoint_targets: tensor name -> destination view). Every target
-    has to be there, with its exact shape."""
+    (checkpoint_targets: tensor name -> destination view or Placement).
+    Every target has to be there, with its exact shape."""
     targets = model.checkpoint_targets()
     missing = set(targets) - set(model.optional_checkpoint_names())
     stager = _Stager(next(model.parameters()).device, use_async)
@@ -216,7 +234,10 @@ def load_mapped_weights(model, ckpt_dir: str, use_async: bool = True) -> int:
         if tuple(tensor.shape) != tuple(dst.shape):
             raise ValueError(f"{name}: checkpoint has {tuple(tensor.shape)}, "
                              f"the configuration {tuple(dst.shape)}")
-        stager.copy(dst, tensor)
+        if isinstance(dst, Placement):
+            dst.copy_(tensor, stager.copy)
+        else:
+            stager.copy(dst, tensor)
         missing.discard(name)
         loaded += 1
     stager.finish()

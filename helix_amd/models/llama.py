@@ -256,6 +256,7 @@ class DecoderLayer(nn.Module):
 
 class LlamaForCausalLM(nn.Module):
     paged_prefill = False        # cached prefixes are gathered
+    extension = "_C"             # native library of its kernels
 
     def __init__(self, cfg: LlamaConfig, tp_size: int = 1, tp_rank: int = 0):
         super().__init__()

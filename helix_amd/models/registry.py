@@ -10,15 +10,18 @@ import json
 import os
 from typing import Callable, Dict, Optional
 
-from helix_amd.models import llama, zederax
+from helix_amd.models import llama, nibezen, zederax
 from helix_amd.models.llama import LlamaConfig, LlamaForCausalLM
+from helix_amd.models.nibezen import NibezenConfig, NibezenForCausalLM
 from helix_amd.models.zederax import ZederaxConfig, ZederaxForCausalLM
 
 MODEL_CLASSES = {LlamaConfig: LlamaForCausalLM,
+                 NibezenConfig: NibezenForCausalLM,
                  ZederaxConfig: ZederaxForCausalLM}
 
 # config.json architecture -> reader(dict, name) of the configuration
 CONFIG_READERS: Dict[str, Callable] = {
+    "Nibezen": NibezenConfig.from_json,
     "Zederax": ZederaxConfig.from_json,
     "LlamaForCausalLM": LlamaConfig.from_json,
     "MistralForCausalLM": LlamaConfig.from_json,
@@ -32,11 +35,12 @@ def is_folder(model: str) -> bool:
 
 def get_config(model: str):
     """Configuration of a preset or of a checkpoint folder."""
-    for presets in (llama.PRESETS, zederax.PRESETS):
+    families = (llama.PRESETS, nibezen.PRESETS, zederax.PRESETS)
+    for presets in families:
         if model in presets:
             return presets[model]
     if not is_folder(model):
-        known = sorted([*llama.PRESETS, *zederax.PRESETS])
+        known = sorted(name for presets in families for name in presets)
         raise KeyError(f"unknown model {model!r}: neither a folder with "
                        f"config.json nor one of {known}")
     with open(os.path.join(model, "config.json")) as f:

@@ -27,12 +27,9 @@ import torch
 import torch.nn as nn
 
 from helix_amd import ops
+from helix_amd.models.base import Float32Kept, round_up
 from helix_amd.models.llama import HLinear
 from helix_amd.models.meta import KVLayer, MixedMeta
-
-
-def _up(n: int, m: int) -> int:
-    return -(-n // m) * m
 
 
 @dataclass(frozen=True)
@@ -72,7 +69,7 @@ class ZederaxConfig:
         return len(self.layers)
 
     def kv_layers(self, tp_size: int = 1) -> List[KVLayer]:
-        return [KVLayer(l.mixer.kv_heads, _up(l.mixer.dim, 8), l.mixer.vdim,
+        return [KVLayer(l.mixer.kv_heads, round_up(l.mixer.dim, 8), l.mixer.vdim,
                         v_transposed=True) for l in self.layers]
 
     def num_weights(self) -> Tuple[int, int]:
@@ -144,22 +141,7 @@ PRESETS = {
 }
 
 
-class _Float32Kept(nn.Module):
-    """Small tensors that stay fp32 through .to(bfloat16): the kernels use
-    them in 32-bit (norm weights, mixing and averaging coefficients)."""
-    kept: Tuple[str, ...] = ()
-
-    def _apply(self, fn, recurse=True):
-        held = {n: getattr(self, n).data for n in self.kept
-                if getattr(self, n) is not None}
-        super()._apply(fn, recurse)
-        for n, t in held.items():
-            cur = getattr(self, n)
-            cur.data = t.to(cur.device)
-        return self
-
-
-class ZederaxLayer(_Float32Kept):
+class ZederaxLayer(Float32Kept):
     kept = ("norm_w", "talk", "vmix", "act", "dwa", "slopes")
 
     def __init__(self, cfg: ZederaxConfig, index: int):
@@ -173,11 +155,11 @@ class ZederaxLayer(_Float32Kept):
         for name, n in (("q", H * m.dim), ("k", G * m.dim),
                         ("v", G * m.vdim), ("up", spec.ff), ("g", H)):
             self.cols[name] = (at, n)
-            at = _up(at + n, 8)
-        self.in_proj = HLinear(W, _up(at, 64), bias=True)
+            at = round_up(at + n, 8)
+        self.in_proj = HLinear(W, round_up(at, 64), bias=True)
         # [o | down] share the accumulator
-        self.down_at = _up(H * m.vdim, 8)
-        self.out_width = _up(self.down_at + spec.ff, 8)
+        self.down_at = round_up(H * m.vdim, 8)
+        self.out_width = round_up(self.down_at + spec.ff, 8)
         self.out_proj = HLinear(self.out_width, W, bias=False)
         for p in (self.in_proj.weight, self.in_proj.bias,
                   self.out_proj.weight):
@@ -249,9 +231,10 @@ class ZederaxLayer(_Float32Kept):
                               meta.row_len, p, gate)
 
 
-class ZederaxForCausalLM(_Float32Kept):
+class ZederaxForCausalLM(Float32Kept):
     kept = ("final_norm_w",)
     paged_prefill = True         # prompts attend through the paged cache
+    extension = "_C_ext"         # native library of its kernels
 
     def __init__(self, cfg: ZederaxConfig, tp_size: int = 1,
                  tp_rank: int = 0):

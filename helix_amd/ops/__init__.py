@@ -13,7 +13,7 @@ from dataclasses import dataclass
 import torch
 
 from . import reference as ref
-from .reference import make_cos_sin_cache  # re-export
+from .reference import make_cos_sin_cache, yarn_frequencies  # re-export
 
 _C = None
 _C_ERR: str | None = None

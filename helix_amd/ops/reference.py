@@ -87,6 +87,31 @@ def make_cos_sin_cache(head_dim: int, max_pos: int, base: float = 10000.0,
     return torch.cat([freqs.cos(), freqs.sin()], dim=-1)
 
 
+def yarn_frequencies(dims: int, base: float,
+                     scaling: dict | None = None) -> tuple:
+    """(float64 frequency of each of the dims/2 pairs, amplitude of cos and
+    sin). With scaling (factor, original, fast, slow), pairs that turn less
+    than `slow` times over the original context are slowed down by factor,
+    those that turn more than `fast` times are left alone, with a linear ramp
+    over the pair number between."""
+    import math
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    freq = float(base) ** (-2.0 * i / dims)
+    if not scaling:
+        return freq, 1.0
+    factor, original = float(scaling["factor"]), float(scaling["original"])
+
+    def turning(n):
+        return dims * math.log(original / (2 * math.pi * n)) / \
+            (2 * math.log(base))
+
+    lo = max(math.floor(turning(float(scaling["fast"]))), 0)
+    hi = min(math.ceil(turning(float(scaling["slow"]))), dims - 1)
+    ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+    return (freq / factor * ramp + freq * (1 - ramp),
+            0.1 * math.log(factor) + 1.0)
+
+
 def silu_and_mul(x: torch.Tensor) -> torch.Tensor:
     i = x.shape[-1] // 2
     g, u = x[..., :i].float(), x[..., i:].float()
