@@ -62,8 +62,10 @@ def main(argv=None) -> int:
     args = ap.parse_args(argv)
 
     if args.device.startswith("cuda"):
+        from helix_amd.models import registry
         from helix_amd.ops import build
-        build.ensure("_C_ext")
+        build.ensure(registry.model_class(
+            registry.get_config(args.model)).extension)
     os.makedirs(args.out, exist_ok=True)
     engine = make_engine(args.model, args.dtype, args.max_tokens,
                          args.device)

@@ -12,6 +12,7 @@ from dataclasses import dataclass
 
 import torch
 
+from . import build
 from . import reference as ref
 from .reference import make_cos_sin_cache, yarn_frequencies  # re-export
 
@@ -24,9 +25,6 @@ try:
 except ImportError as e:  # pragma: no cover
     _C_ERR = str(e)
 
-_C_ext = None
-
-
 def _native():
     if _C is None:
         raise RuntimeError(
@@ -37,27 +35,14 @@ def _native():
 
 
 def _native_ext():
-    """helix_amd._C_ext, imported at first use (a program may build it
-    after this module was imported)."""
-    global _C_ext
-    if _C_ext is None:
-        try:
-            from helix_amd import _C_ext as mod  # type: ignore
-        except ImportError as e:
-            raise RuntimeError(
-                "helix_amd._C_ext native extension is not built but a GPU "
-                "tensor was passed. Build it with `python setup.py build_ext "
-                "--inplace` (PYTORCH_ROCM_ARCH=gfx950). Import error: "
-                f"{e}") from e
-        _C_ext = mod
-    return _C_ext
+    return build.load("_C_ext")
 
 
 def have_native(name: str = "_C") -> bool:
     if name == "_C":
         return _C is not None
     try:
-        return _native_ext() is not None
+        return build.load(name) is not None
     except RuntimeError:
         return False
 

@@ -7,6 +7,7 @@ compiled (gfx950, cross-compilation needs no GPU).
 from __future__ import annotations
 
 import glob
+import importlib
 import os
 import subprocess
 import sys
@@ -27,3 +28,21 @@ def ensure(name: str) -> None:
     env = dict(os.environ, PYTORCH_ROCM_ARCH="gfx950", HELIX_BUILD_ONLY=name)
     subprocess.run([sys.executable, "setup.py", "build_ext", "--inplace"],
                    cwd=ROOT, env=env, check=True, stdout=sys.stderr)
+
+
+_loaded: dict = {}
+
+
+def load(name: str):
+    """Extension `name`, imported at first use (a program may build it after
+    helix_amd.ops was imported)."""
+    if name not in _loaded:
+        try:
+            _loaded[name] = importlib.import_module(f"helix_amd.{name}")
+        except ImportError as e:
+            raise RuntimeError(
+                f"helix_amd.{name} native extension is not built but a GPU "
+                "tensor was passed. Build it with `python setup.py build_ext "
+                "--inplace` (PYTORCH_ROCM_ARCH=gfx950). Import error: "
+                f"{e}") from e
+    return _loaded[name]

@@ -1,7 +1,7 @@
 // Element access shared by the kernels that come in a bf16 and an fp32
 // build: storage type S is uint16_t (bf16 bits) or float, math is fp32.
 #pragma once
-#include "../common.h"
+#include "common.h"
 
 namespace helix {
 

@@ -8,7 +8,7 @@
 // One workgroup per token. Everything is read once: the averaged row stays
 // in registers between the sum and the norm. The history is [depth, T, W]
 // fp32, so each X_j row is one contiguous streak.
-#include "elem.h"
+#include "../elem.h"
 #include <torch/extension.h>
 #include <ATen/hip/HIPContext.h>
 

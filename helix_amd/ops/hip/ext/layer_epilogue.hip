@@ -16,7 +16,7 @@
 // [nblk, G, E, bs], so 8 consecutive tokens of one value dim are one
 // 16-byte load. That is the B operand of the weights-times-values MFMA, and
 // it lets the attention kernels read V straight into registers.
-#include "elem.h"
+#include "../elem.h"
 #include <torch/extension.h>
 #include <ATen/hip/HIPContext.h>
 

@@ -27,7 +27,7 @@
 //   A: lane l holds A[row = lo][k = hi*8 + i]
 //   B: lane l holds B[k = hi*8 + i][col = lo]
 //   C: lane l holds C[row = hi*4 + r][col = lo]
-#include "elem.h"
+#include "../elem.h"
 #include <torch/extension.h>
 #include <ATen/hip/HIPContext.h>
 

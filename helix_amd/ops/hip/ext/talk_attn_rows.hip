@@ -29,7 +29,7 @@
 //
 // Cache layout: K [nblk, G, bs, Dp]; V [nblk, G, E, bs] (8 tokens of one
 // value dim are one 16-byte load).
-#include "elem.h"
+#include "../elem.h"
 #include <torch/extension.h>
 #include <ATen/hip/HIPContext.h>
 

@@ -9,26 +9,11 @@ from typing import Optional
 
 import torch
 
+from . import build
 from . import hybrid_reference as ref
 
-_C = None
-
-
 def _native():
-    """helix_amd._C_hybrid, imported at first use (a program may build it
-    after this module was imported)."""
-    global _C
-    if _C is None:
-        try:
-            from helix_amd import _C_hybrid as mod  # type: ignore
-        except ImportError as e:
-            raise RuntimeError(
-                "helix_amd._C_hybrid native extension is not built but a GPU "
-                "tensor was passed. Build it with `python setup.py build_ext "
-                "--inplace` (PYTORCH_ROCM_ARCH=gfx950). Import error: "
-                f"{e}") from e
-        _C = mod
-    return _C
+    return build.load("_C_hybrid")
 
 
 # ----------------------------------------------------------- residual stream
@@ -136,15 +121,15 @@ def latent_epilogue(z: torch.Tensor, p: LatentParams,
     ref.latent_epilogue(z, p, positions, norm_w, eps, cache, slots)
 
 
-# Keys of one tile of the row kernel; enough workgroups to fill the chip.
-LATENT_TILE = 32
+# Cached rows of a partition at least; enough workgroups to fill the chip.
+LATENT_PART = 128
 LATENT_TARGET_WGS = 512
 
 
 def latent_parts(rows: int, heads: int, keys: int) -> int:
     """Key partitions per row of the MFMA row kernel."""
-    groups = -(-heads // 64)
-    return max(1, min(-(-keys // (4 * LATENT_TILE)),
+    groups = -(-heads // 32)
+    return max(1, min(-(-keys // LATENT_PART),
                       LATENT_TARGET_WGS // max(1, rows * groups)))
 
 
@@ -300,11 +285,12 @@ def ssm_prompt(y: torch.Tensor, z: torch.Tensor, p: SSMParams, w: SSMWeights,
                          int(meta.positions[cu[b]]), w)
         return
     C = _native()
-    if not C.ssm_chunks_fit(z, p.vdim, p.state):
+    if not C.ssm_chunks_fit(z, p.vdim, p.state, p.conv):
         xbc = torch.empty(z.shape[0], p.channels, dtype=z.dtype,
                           device=z.device)
         C.conv_span(xbc, z, p.xbc_at, w.conv, w.conv_b, ring,
-                    meta.state_slots, meta.positions, meta.cu_seqlens)
+                    meta.state_slots, meta.positions, meta.cu_seqlens,
+                    meta.max_seqlen)
         C.ssm_step(y, z, xbc, p.z_at, p.xbc_at, p.dt_at, w.conv, w.conv_b,
                    w.dt_bias, w.A_log, w.D, ring, state, meta.state_slots,
                    meta.positions, meta.cu_seqlens)
