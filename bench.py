@@ -137,13 +137,15 @@ def run_coresident(args) -> None:
 
 
 def run_design(args) -> None:
-    """Prefill / decode throughput of the Zederax presets and of equally
-    large Llama models, and kernel by kernel distance from the roofline."""
+    """Prefill / decode throughput of Zederax or Nibezen presets and of
+    equally large Llama models, and kernel by kernel distance from the
+    roofline."""
     from helix_amd.engine import design_bench
     names = args.design.split(",")
     res = design_bench.run(names, "cuda:0", min(args.steps, 32),
                            args.design_part)
-    first = res[names[0]].get("zederax")
+    first = next((v for k, v in res[names[0]].items()
+                  if k in ("zederax", "nibezen")), None)
     print(json.dumps({
         "metric": "tokens/sec (design)",
         "value": first[-1]["decode_tok_s"] if first else None,
@@ -178,7 +180,7 @@ def main():
     ap.add_argument("--top-p", type=float, default=1.0)
     ap.add_argument("--design", type=str, default="",
                     help="instead of the headline: comma-separated Zederax "
-                         "presets, each beside a Llama of equal size")
+                         "or Nibezen presets, each beside a Llama of equal size")
     ap.add_argument("--design-part", type=str, default="all",
                     choices=["all", "throughput", "kernels"])
     args = ap.parse_args()

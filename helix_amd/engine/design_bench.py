@@ -1,13 +1,12 @@
-"""Throughput of a Zederax model beside a Llama of equal size, and each of
+"""Throughput of a design's model beside a Llama of equal size, and each of
 its kernels beside the like kernel of the Llama path (bench.py --design).
 
-Equal size: same width, depth, heads, vocabulary and window; the Llama
-feed-forward has three matrices, so two thirds of the ff. A kernel's
-distance is its time over the time its roofline allows (8 TB/s HBM, 2.5
-PFLOP/s dense bf16).
+A kernel's distance is its time over the time its roofline allows (8 TB/s
+HBM, 2.5 PFLOP/s dense bf16).
 """
 from __future__ import annotations
 
+import sys
 import time
 from typing import Callable, Dict, List
 
@@ -23,7 +22,9 @@ from helix_amd.models.zederax import ZederaxConfig
 HBM, FLOPS = 8.0e12, 2.5e15
 
 
-def llama_twin(z: ZederaxConfig) -> LlamaConfig:
+def zederax_twin(z: ZederaxConfig) -> LlamaConfig:
+    """Same width, depth, heads, vocabulary and window; the Llama
+    feed-forward has three matrices, so two thirds of the ff."""
     m = z.layers[0].mixer
     return LlamaConfig(
         name=f"llama-as-{z.name}", vocab_size=z.vocab_size,
@@ -81,6 +82,7 @@ def throughput(cfg, device, shapes, steps: int) -> List[dict]:
                    "decode_tok_s": round(b * steps / (t3 - t2)),
                    "decode_ms": round((t3 - t2) / steps * 1e3, 3)}
         out.append(res)
+        print(f"{cfg.name}: {res}", file=sys.stderr, flush=True)
     del eng
     torch.cuda.empty_cache()
     return out
@@ -106,7 +108,7 @@ def _row(t: float, nbytes: float, flops: float = 0.0) -> dict:
             "distance": round(t / floor, 2)}
 
 
-def kernels(z: ZederaxConfig, device, decode_batch: int = 256,
+def zederax_kernels(z: ZederaxConfig, device, decode_batch: int = 256,
             decode_len: int = 1024, prompts: int = 8,
             prompt_len: int = 2048) -> Dict[str, dict]:
     """Each kernel of the new path and the like one, at one layer's size."""
@@ -221,19 +223,27 @@ def kernels(z: ZederaxConfig, device, decode_batch: int = 256,
     return out
 
 
+def _families():
+    from helix_amd.engine import design_bench_hybrid as hybrid
+    from helix_amd.models.nibezen import NibezenConfig
+    return {ZederaxConfig: ("zederax", zederax_twin, zederax_kernels),
+            NibezenConfig: ("nibezen", hybrid.twin, hybrid.kernels)}
+
+
 def run(names: List[str], device: str, steps: int, what: str) -> dict:
     result = {}
     for name in names:
         z = registry.get_config(name)
+        family, twin, kernels = _families()[type(z)]
         r = result[name] = {}
         if what in ("all", "throughput"):
             shapes = [(8, 2048), (64, 2048), (256, 1024)]
-            r["zederax"] = throughput(z, device, shapes, steps)
-            r["llama"] = throughput(llama_twin(z), device, shapes, steps)
+            r[family] = throughput(z, device, shapes, steps)
+            r["llama"] = throughput(twin(z), device, shapes, steps)
             for a in ("prefill_tok_s", "decode_tok_s"):
                 r[f"ratio_{a}"] = [
                     round(x[a] / y[a], 3)
-                    for x, y in zip(r["zederax"], r["llama"])]
+                    for x, y in zip(r[family], r["llama"])]
         if what in ("all", "kernels"):
             r["kernels"] = kernels(z, device)
     return result

@@ -39,17 +39,101 @@ struct Epilogue {
   float amp, eps;
 };
 
+// The pair (u, v) at columns j, j + 1 of a head turns by its angle.
+__device__ __forceinline__ void turn(float& u, float& v, const float* trig) {
+  const float a = u * trig[0] - v * trig[1];
+  v = v * trig[0] + u * trig[1];
+  u = a;
+}
+
 // Rotates q in place, writes the cache row. One workgroup per token; the
-// angles of the pairs are the same for all heads.
-template <typename S>
+// angles of the pairs are the same for all heads. N: elements of a thread's
+// accesses; rank, dims and columns are multiples of it.
+template <typename S, int N>
 __global__ __launch_bounds__(NT) void latent_epilogue_kernel(
     S* __restrict__ z, S* __restrict__ cache, Epilogue e) {
-  extern __shared__ float trig[];             // [pairs][2]
+  extern __shared__ __attribute__((aligned(16))) float trig[];  // [pairs][2]
+  __shared__ float red[16];
+  const int64_t t = blockIdx.x;
+  const int tid = threadIdx.x;
+  S* zr = z + t * e.z_stride;
+  const S* kv = zr + e.kv_at;
+  // the first query vector and the latent are under way during the angles
+  const int per = 2 * e.pairs / N, nq = e.heads * per;
+  auto q_at = [&](int i) {
+    const int h = i / per;
+    return zr + e.q_at + h * e.head_cols + e.dim_pad + (i - h * per) * N;
+  };
+  float q0[N], c0[N];
+  if (tid < nq) ldv<N>(q_at(tid), q0);
+  if (tid * N < e.rank) ldv<N>(kv + tid * N, c0);
+  for (int i = tid; i < e.pairs; i += NT) {
+    // whole turns off in double, the rest is a 32-bit angle
+    const double turns =
+        (double)e.pos[t] * e.freqs[i] * 0.15915494309189533577;
+    const float a = (float)((turns - floor(turns)) * 6.28318530717958647693);
+    float s, c;
+    sincosf(a, &s, &c);
+    trig[2 * i] = e.amp * c;
+    trig[2 * i + 1] = e.amp * s;
+  }
+  float ss = 0.f;
+  if (tid * N < e.rank) {
+#pragma unroll
+    for (int i = 0; i < N; ++i) ss += c0[i] * c0[i];
+  }
+  for (int d = (tid + NT) * N; d < e.rank; d += NT * N) {
+    float v[N];
+    ldv<N>(kv + d, v);
+#pragma unroll
+    for (int i = 0; i < N; ++i) ss += v[i] * v[i];
+  }
+  const float inv = 1.f / sqrtf(group_sum(ss, red) / e.rank + e.eps);
+
+  for (int i = tid; i < nq; i += NT) {
+    S* q = q_at(i);
+    if (i != tid) ldv<N>(q, q0);
+    const float* tr = trig + i % per * N;
+#pragma unroll
+    for (int j = 0; j < N; j += 2) turn(q0[j], q0[j + 1], tr + j);
+    stv<N>(q, q0);
+  }
+  const int64_t slot = e.slots[t];
+  if (slot < 0) return;
+  S* out = cache + slot * e.row;
+  for (int d = tid * N; d < e.row; d += NT * N) {
+    float v[N];
+    if (d < e.rank) {
+      float w[N];
+      ldv<N>(kv + d, v);
+      ldv<N>(e.norm_w + d, w);
+#pragma unroll
+      for (int i = 0; i < N; ++i) v[i] *= inv * w[i];
+    } else if (d >= e.rank_pad && d < e.rank_pad + e.rot_dim) {
+      ldv<N>(kv + d, v);
+      const int j0 = d - e.rank_pad;
+      if (j0 < 2 * e.pairs) {
+#pragma unroll
+        for (int j = 0; j < N; j += 2)
+          turn(v[j], v[j + 1], trig + j0 + j);
+      }
+    } else {
+#pragma unroll
+      for (int i = 0; i < N; ++i) v[i] = 0.f;
+    }
+    stv<N>(out + d, v);
+  }
+}
+
+// Any sizes.
+template <typename S>
+__global__ __launch_bounds__(NT) void latent_epilogue_any_kernel(
+    S* __restrict__ z, S* __restrict__ cache, Epilogue e) {
+  extern __shared__ float trig[];
   __shared__ float red[16];
   const int64_t t = blockIdx.x;
   S* zr = z + t * e.z_stride;
   for (int i = threadIdx.x; i < e.pairs; i += NT) {
-    // whole turns off in double, the rest is a 32-bit angle
     const double turns =
         (double)e.pos[t] * e.freqs[i] * 0.15915494309189533577;
     const float a = (float)((turns - floor(turns)) * 6.28318530717958647693);
@@ -65,7 +149,6 @@ __global__ __launch_bounds__(NT) void latent_epilogue_kernel(
     ss += v * v;
   }
   const float inv = 1.f / sqrtf(group_sum(ss, red) / e.rank + e.eps);
-
   const int64_t slot = e.slots[t];
   if (slot >= 0) {
     S* out = cache + slot * e.row;
@@ -77,22 +160,22 @@ __global__ __launch_bounds__(NT) void latent_epilogue_kernel(
         const int j = d - e.rank_pad;
         v = ld1(kv + d);
         if (j < 2 * e.pairs) {
-          const float c = trig[j & ~1], s = trig[j | 1];
-          const float other = ld1(kv + e.rank_pad + (j ^ 1));
-          v = (j & 1) ? v * c + other * s : v * c - other * s;
+          float u = ld1(kv + e.rank_pad + (j & ~1));
+          float w = ld1(kv + e.rank_pad + (j | 1));
+          turn(u, w, trig + (j & ~1));
+          v = (j & 1) ? w : u;
         }
       }
       st1(out + d, v);
     }
   }
-  if (e.pairs == 0) return;
   for (int i = threadIdx.x; i < e.heads * e.pairs; i += NT) {
     const int h = i / e.pairs, p = i - h * e.pairs;
     S* q = zr + e.q_at + h * e.head_cols + e.dim_pad + 2 * p;
-    const float u = ld1(q), v = ld1(q + 1);
-    const float c = trig[2 * p], s = trig[2 * p + 1];
-    st1(q, u * c - v * s);
-    st1(q + 1, v * c + u * s);
+    float u = ld1(q), v = ld1(q + 1);
+    turn(u, v, trig + 2 * p);
+    st1(q, u);
+    st1(q + 1, v);
   }
 }
 
@@ -209,6 +292,7 @@ __global__ __launch_bounds__(NT, 2) void latent_rows_kernel(
   __shared__ uint16_t kv[KEYS * PITCH];
   __shared__ uint16_t pw[HT * 16 * PP];
   __shared__ float stat[4][16];
+  __shared__ int slots[2][KEYS];              // cache rows of two tiles
 
   const int r = blockIdx.x, part = blockIdx.y, h0 = blockIdx.z * HT * 16;
   const int tid = threadIdx.x, wid = tid / WAVE, lane = tid & (WAVE - 1);
@@ -236,14 +320,19 @@ __global__ __launch_bounds__(NT, 2) void latent_rows_kernel(
   }
   const int* bt = m.bt + (int64_t)(m.row_seq ? m.row_seq[r] : r) * m.bt_stride;
   u16x8 reg[NL];
-  auto load = [&](int base) {
+  auto load = [&](int buf) {
 #pragma unroll
     for (int c = 0; c < NL; ++c) {
       const int e = c * NT + tid, key = e / (NK * 4), d = e % (NK * 4) * 8;
-      const int tok = min(base + key, p1 - 1);
-      const int64_t slot = (int64_t)bt[tok / m.bs] * m.bs + tok % m.bs;
-      reg[c] = d < m.row ? ld_u16x8(cache + slot * m.row + d) : zero;
+      reg[c] = d < m.row
+                   ? ld_u16x8(cache + (int64_t)slots[buf][key] * m.row + d)
+                   : zero;
     }
+  };
+  // page lookups run two tiles ahead of the rows, so no load waits for one
+  auto slot_of = [&](int base) {
+    const int tok = min(base + tid, p1 - 1);
+    return bt[tok / m.bs] * m.bs + tok % m.bs;
   };
   floatx4 acc[HT][DT];
   float m_run[HT], l = 0.f;
@@ -254,8 +343,14 @@ __global__ __launch_bounds__(NT, 2) void latent_rows_kernel(
     for (int d = 0; d < DT; ++d) acc[t][d] = floatx4{0, 0, 0, 0};
   }
 
-  load(p0);
-  for (int base = p0; base < p1; base += KEYS) {
+  if (tid < KEYS) {
+    slots[0][tid] = slot_of(p0);
+    slots[1][tid] = slot_of(p0 + KEYS);
+  }
+  __syncthreads();
+  load(0);
+  int buf = 0;
+  for (int base = p0; base < p1; base += KEYS, buf ^= 1) {
     __syncthreads();                          // the last tile is read
 #pragma unroll
     for (int c = 0; c < NL; ++c) {
@@ -264,7 +359,9 @@ __global__ __launch_bounds__(NT, 2) void latent_rows_kernel(
                                 e % (NK * 4) * 8) = reg[c];
     }
     __syncthreads();
-    if (base + KEYS < p1) load(base + KEYS);
+    int ahead = 0;
+    if (base + KEYS < p1) load(buf ^ 1);
+    if (tid < KEYS) ahead = slot_of(base + 2 * KEYS);
 
     // scores of 16 rows x 16 heads: lane has rows 4 hi + i, head lo
     floatx4 s = floatx4{0, 0, 0, 0};
@@ -330,6 +427,7 @@ __global__ __launch_bounds__(NT, 2) void latent_rows_kernel(
         }
       }
     }
+    if (tid < KEYS) slots[buf][tid] = ahead;  // this tile's are used
   }
 
   l += __shfl_xor(l, 16, WAVE);
@@ -639,14 +737,22 @@ void latent_epilogue(torch::Tensor z, int64_t q_at, int64_t heads,
   if (T == 0) return;
   auto stream = at::hip::getCurrentHIPStream();
   const int lds = std::max(1, e.pairs) * 2 * sizeof(float);
-  if (is_bf16(z))
-    hipLaunchKernelGGL((latent_epilogue_kernel<uint16_t>), dim3(T), dim3(NT),
-                       lds, stream, (uint16_t*)z.data_ptr(),
-                       (uint16_t*)cache.data_ptr(), e);
-  else
-    hipLaunchKernelGGL((latent_epilogue_kernel<float>), dim3(T), dim3(NT),
-                       lds, stream, (float*)z.data_ptr(),
-                       (float*)cache.data_ptr(), e);
+  const bool vec = rank % 8 == 0 && rot_dim % 8 == 0 && e.pairs % 4 == 0 &&
+                   rank_pad % 8 == 0 && row % 8 == 0 && dim_pad % 8 == 0 &&
+                   head_cols % 8 == 0 && q_at % 8 == 0 && kv_at % 8 == 0 &&
+                   e.z_stride % 8 == 0 && (uintptr_t)z.data_ptr() % 32 == 0;
+#define HELIX_EPI(K, S)                                                      \
+  hipLaunchKernelGGL((K), dim3(T), dim3(NT), lds, stream, (S*)z.data_ptr(),  \
+                     (S*)cache.data_ptr(), e)
+  if (is_bf16(z)) {
+    if (vec && e.pairs > 0)
+      HELIX_EPI((latent_epilogue_kernel<uint16_t, 8>), uint16_t);
+    else
+      HELIX_EPI((latent_epilogue_any_kernel<uint16_t>), uint16_t);
+  } else {
+    HELIX_EPI((latent_epilogue_any_kernel<float>), float);
+  }
+#undef HELIX_EPI
 }
 
 void latent_absorb(torch::Tensor q, torch::Tensor z, int64_t q_at,

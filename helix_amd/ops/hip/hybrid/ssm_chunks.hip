@@ -37,7 +37,7 @@ struct Conv {
   const int* row;
   const int* count;
   int64_t z_stride;
-  int xbc_at, dt_at, H, P, Pp, N, Np, G, taps, C;
+  int xbc_at, dt_at, H, P, Pp, N, Np, G, taps, C, vec;
 };
 
 // grid (chunks, channel blocks of 64 + blocks of 4 heads for da)
@@ -46,7 +46,7 @@ __global__ __launch_bounds__(NT) void conv_chunks_kernel(
     uint16_t* __restrict__ bt, uint16_t* __restrict__ c,
     float* __restrict__ da, const uint16_t* __restrict__ z, uint16_t* ring,
     Conv m) {
-  extern __shared__ __attribute__((aligned(16))) float sh[];
+  extern __shared__ __attribute__((aligned(16))) uint16_t sh[];
   const int n = blockIdx.x, tid = threadIdx.x;
   const int row = m.row[n], count = m.count[n], sq = m.seq[n];
   const int pb = cdiv(m.P, 64), nb = cdiv(m.Np, 64);
@@ -88,23 +88,38 @@ __global__ __launch_bounds__(NT) void conv_chunks_kernel(
     c0 = m.H * m.P + ((kind - 1) * m.G + unit) * m.N + part;
     nc = min(64, m.N - part);                 // may be none: padding
   }
+  // Inputs in LDS, a row per token: the chunk's own and those before it.
   const int before = m.taps - 1, rows = L + before;
-  constexpr int IP = 65;
-  float* in = sh;                             // [rows][IP]
-  uint16_t* ol = (uint16_t*)(sh + ((rows * IP + 3) & ~3));   // [L][LP]
+  uint16_t* in = sh;                          // [rows][LP]
+  uint16_t* tl = in + rows * LP;              // [64 channels][LP] result
+  uint16_t* rl = tl + 64 * LP;                // [64 tokens][LP] result
   const int seq0 = m.cu[sq], slot = m.slots[sq];
   const int64_t p0 = m.pos[row];
+  const uint16_t* zc = z + m.xbc_at + c0;
   uint16_t* rs = ring + (int64_t)max(slot, 0) * m.taps * m.C + c0;
-  for (int i = tid; i < rows * 64; i += NT) {
-    const int r = i / 64, ch = i % 64, t = r - before;
-    float v = 0.f;
-    if (ch < nc && t < count) {
-      if (row + t >= seq0)
-        v = bf16_to_f32(z[(row + t) * m.z_stride + m.xbc_at + c0 + ch]);
-      else if (slot >= 0 && p0 + t >= 0)
-        v = bf16_to_f32(rs[(p0 + t) % m.taps * m.C + ch]);
+  if (m.vec) {
+    for (int i = tid; i < rows * 8; i += NT) {
+      const int r = i / 8, ch = i % 8 * 8, t = r - before;
+      u16x8 v = {0, 0, 0, 0, 0, 0, 0, 0};
+      if (ch < nc && t < count) {
+        if (row + t >= seq0)
+          v = ld_u16x8(zc + (row + t) * m.z_stride + ch);
+        else if (slot >= 0 && p0 + t >= 0)
+          v = ld_u16x8(rs + (p0 + t) % m.taps * m.C + ch);
+      }
+      *reinterpret_cast<u16x8*>(in + r * LP + ch) = v;
     }
-    in[r * IP + ch] = v;
+  } else {
+    for (int i = tid; i < rows * 64; i += NT) {
+      const int r = i / 64, ch = i % 64, t = r - before;
+      uint16_t v = 0;
+      if (ch < nc && t < count) {
+        if (row + t >= seq0) v = zc[(row + t) * m.z_stride + ch];
+        else if (slot >= 0 && p0 + t >= 0)
+          v = rs[(p0 + t) % m.taps * m.C + ch];
+      }
+      in[r * LP + ch] = v;
+    }
   }
   __syncthreads();
   // The first chunk is the only reader of the ring; it also refills it with
@@ -115,48 +130,83 @@ __global__ __launch_bounds__(NT) void conv_chunks_kernel(
       const int t = len - k + i / 64, ch = i % 64;
       if (ch < nc)
         rs[(p0 + t) % m.taps * m.C + ch] =
-            z[(int64_t)(seq0 + t) * m.z_stride + m.xbc_at + c0 + ch];
+            zc[(int64_t)(seq0 + t) * m.z_stride + ch];
     }
   }
-  const int ch = tid >> 2, t0 = (tid & 3) * 16;
-  float acc[16];
-  const bool live = ch < nc;
-  const float bias = live ? m.conv_b[c0 + ch] : 0.f;
+  // A thread has two neighbouring channels of 8 tokens.
+  const int ch = tid % 32 * 2, t0 = tid / 32 * 8;
+  const int ca = c0 + min(ch, max(nc, 1) - 1);
+  const int cb = c0 + min(ch + 1, max(nc, 1) - 1);
+  float u[8], v[8];
+  if (nc > 0) {
+    const float b0 = m.conv_b[ca], b1 = m.conv_b[cb];
 #pragma unroll
-  for (int i = 0; i < 16; ++i) acc[i] = bias;
-  for (int k = 0; k < m.taps; ++k) {
-    const float w = live ? m.conv[(int64_t)(c0 + ch) * m.taps + k] : 0.f;
+    for (int i = 0; i < 8; ++i) {
+      u[i] = b0;
+      v[i] = b1;
+    }
+    const uint16_t* src = in + t0 * LP + ch;
+    auto tap = [&](int k, const uint32_t* x) {
+      const float w0 = m.conv[(int64_t)ca * m.taps + k];
+      const float w1 = m.conv[(int64_t)cb * m.taps + k];
 #pragma unroll
-    for (int i = 0; i < 16; ++i) acc[i] += w * in[(t0 + i + k) * IP + ch];
+      for (int i = 0; i < 8; ++i) {
+        u[i] += w0 * bf16_to_f32((uint16_t)x[i]);
+        v[i] += w1 * bf16_to_f32((uint16_t)(x[i] >> 16));
+      }
+    };
+    if (m.taps == 4) {
+      uint32_t x[11];
+#pragma unroll
+      for (int i = 0; i < 11; ++i)
+        x[i] = *reinterpret_cast<const uint32_t*>(src + i * LP);
+#pragma unroll
+      for (int k = 0; k < 4; ++k) tap(k, x + k);
+    } else {
+      for (int k = 0; k < m.taps; ++k) {
+        uint32_t x[8];
+#pragma unroll
+        for (int i = 0; i < 8; ++i)
+          x[i] = *reinterpret_cast<const uint32_t*>(src + (i + k) * LP);
+        tap(k, x);
+      }
+    }
   }
-#pragma unroll
-  for (int i = 0; i < 16; ++i)
-    acc[i] = live && t0 + i < count ? silu_s<uint16_t>(acc[i]) : 0.f;
-
-  const u16x8 lo = pack8(acc), hi = pack8(acc + 8);
-  uint16_t* t_out = nullptr;
-  if (kind == 0 && part + ch < m.Pp)
-    t_out = xt + (((int64_t)n * m.H + unit) * m.Pp + part + ch) * L;
-  else if (kind == 1 && part + ch < m.Np)
-    t_out = bt + (((int64_t)n * m.G + unit) * m.Np + part + ch) * L;
-  if (t_out != nullptr) {
-    *reinterpret_cast<u16x8*>(t_out + t0) = lo;
-    *reinterpret_cast<u16x8*>(t_out + t0 + 8) = hi;
-  }
-  if (kind == 0) return;
 #pragma unroll
   for (int i = 0; i < 8; ++i) {
-    ol[(t0 + i) * LP + ch] = lo[i];
-    ol[(t0 + 8 + i) * LP + ch] = hi[i];
+    u[i] = ch < nc && t0 + i < count ? silu_s<uint16_t>(u[i]) : 0.f;
+    v[i] = ch + 1 < nc && t0 + i < count ? silu_s<uint16_t>(v[i]) : 0.f;
+  }
+  if (kind != 2) {
+    *reinterpret_cast<u16x8*>(tl + ch * LP + t0) = pack8(u);
+    *reinterpret_cast<u16x8*>(tl + (ch + 1) * LP + t0) = pack8(v);
+  }
+  if (kind != 0) {
+#pragma unroll
+    for (int i = 0; i < 8; ++i)
+      *reinterpret_cast<uint32_t*>(rl + (t0 + i) * LP + ch) =
+          pack_bf16(u[i], v[i]);
   }
   __syncthreads();
-  uint16_t* o = kind == 1 ? b : c;
-  for (int i = tid; i < L * 8; i += NT) {
-    const int t = i / 8, d = i % 8 * 8;
-    if (part + d < m.Np)
-      *reinterpret_cast<u16x8*>(
-          o + (((int64_t)n * L + t) * m.G + unit) * m.Np + part + d) =
-          *reinterpret_cast<u16x8*>(ol + t * LP + d);
+  if (kind != 2) {
+    const int width = kind == 0 ? m.Pp : m.Np;
+    uint16_t* o = kind == 0
+                      ? xt + (((int64_t)n * m.H + unit) * m.Pp + part) * L
+                      : bt + (((int64_t)n * m.G + unit) * m.Np + part) * L;
+    for (int i = tid; i < 64 * 8; i += NT)
+      if (part + i / 8 < width)
+        *reinterpret_cast<u16x8*>(o + i * 8) =
+            ld_u16x8(tl + i / 8 * LP + i % 8 * 8);
+  }
+  if (kind != 0) {
+    uint16_t* o = kind == 1 ? b : c;
+    for (int i = tid; i < L * 8; i += NT) {
+      const int t = i / 8, d = i % 8 * 8;
+      if (part + d < m.Np)
+        *reinterpret_cast<u16x8*>(
+            o + (((int64_t)n * L + t) * m.G + unit) * m.Np + part + d) =
+            ld_u16x8(rl + t * LP + d);
+    }
   }
 }
 
@@ -172,49 +222,53 @@ struct Chunks {
   int z_at, H, P, Pp, N, Np, G, vec;
 };
 
-// NK: 32-wide steps of the state size. Wave w: tokens 16 w .. of the output,
-// values 16 w .. of the state.
-template <int NK>
+// NK: 32-wide steps of the state size; PW: 16-value tiles of a workgroup.
+// Wave w has tokens 16 w .. of the output, and of the state the value tile
+// w % PW in its share of the rows.
+template <int NK, int PW>
 __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void ssm_chunks_kernel(
     uint16_t* __restrict__ y, const uint16_t* __restrict__ z,
     const uint16_t* __restrict__ xt, const uint16_t* __restrict__ b,
     const uint16_t* __restrict__ bt, const uint16_t* __restrict__ c,
     Chunks m) {
   extern __shared__ __attribute__((aligned(16))) uint16_t lds[];
+  constexpr int PB = PW * 16, ST = NK * PW / 2, XL = PW / 2;
   const int NP = m.Np + 8;
   uint16_t* bl = lds;                         // [64 tokens][NP]
   uint16_t* btl = bl + L * NP;                // [Np][LP]
-  uint16_t* xl = btl + m.Np * LP;             // [64 values][LP]
-  uint16_t* sh = xl + 64 * LP;                // [64 values][NP]
-  uint16_t* sl = sh + 64 * NP;
-  float* al = (float*)(sl + 64 * NP);         // [64] sums, [64] steps
+  uint16_t* xl = btl + m.Np * LP;             // [PB values][LP]
+  uint16_t* sh = xl + PB * LP;                // [PB values][NP]
+  uint16_t* sl = sh + PB * NP;
+  float* al = (float*)(sl + PB * NP);         // [64] sums, [64] steps
   float* dl = al + L;
 
-  const int seq = blockIdx.y, h = blockIdx.x, p0 = blockIdx.z * 64;
+  const int seq = blockIdx.y, h = blockIdx.x, p0 = blockIdx.z * PB;
   const int g = h / (m.H / m.G);
   const int tid = threadIdx.x, wid = tid / WAVE, lane = tid & (WAVE - 1);
   const int lo = lane & 15, hi = lane >> 4;
-  const int np = min(64, m.P - p0), rowsp = min(64, m.Pp - p0);
+  const int np = min(PB, m.P - p0), rowsp = min(PB, m.Pp - p0);
   const int row0 = m.cu[seq], row1 = m.cu[seq + 1];
   const int slot = m.slots[seq];
   const int n0 = m.first[seq], n1 = m.first[seq + 1];
-  const int ks = m.Np / 32, ns = m.Np / 16, per = m.Np / 8;
+  const int ks = m.Np / 32, per = m.Np / 8;
   const u16x8 zero = {0, 0, 0, 0, 0, 0, 0, 0};
 
   // this wave's 16 columns of the state: lane has column lo, rows 4 hi + r
-  const int pcol = p0 + wid * 16 + lo;
-  floatx4 S[NK * 2];
+  // of the nts row tiles from nt0 on
+  const int pt = wid % PW, pcol = p0 + pt * 16 + lo;
+  const int nts = m.Np * PW / 64, nt0 = wid / PW * nts;
+  floatx4 S[ST];
   float* st = m.state + ((int64_t)max(slot, 0) * m.H + h) * m.N * m.P + pcol;
   const bool carried = slot >= 0 && m.pos[row0] > 0 && pcol < m.P;
 #pragma unroll
-  for (int t = 0; t < NK * 2; ++t)
+  for (int t = 0; t < ST; ++t)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int n = t * 16 + hi * 4 + r;
-      S[t][r] = carried && n < m.N ? st[(int64_t)n * m.P] : 0.f;
+      const int n = (nt0 + t) * 16 + hi * 4 + r;
+      S[t][r] = carried && t < nts && n < m.N ? st[(int64_t)n * m.P] : 0.f;
     }
 
-  u16x8 breg[NK], btreg[NK], xreg[2], creg[NK];
+  u16x8 breg[NK], btreg[NK], xreg[XL], creg[NK];
   float areg = 0.f;
   auto load = [&](int n) {
 #pragma unroll
@@ -233,7 +287,7 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void ssm_chunks_kernel(
                        : zero;
     }
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
+    for (int i = 0; i < XL; ++i) {
       const int e = i * NT + tid;
       xreg[i] = e < rowsp * 8
                     ? ld_u16x8(xt + (((int64_t)n * m.H + h) * m.Pp + p0) * L +
@@ -243,6 +297,7 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void ssm_chunks_kernel(
     if (tid < 2 * L) areg = m.da[((int64_t)n * m.H + h) * 2 * L + tid];
   };
 
+  const float Dh = m.D[h];
   load(n0);
   for (int n = n0; n < n1; ++n) {
     __syncthreads();                          // the last chunk is done
@@ -255,30 +310,47 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void ssm_chunks_kernel(
         *reinterpret_cast<u16x8*>(btl + e / 8 * LP + e % 8 * 8) = btreg[i];
     }
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
+    for (int i = 0; i < XL; ++i) {
       const int e = i * NT + tid;
       *reinterpret_cast<u16x8*>(xl + e / 8 * LP + e % 8 * 8) = xreg[i];
     }
     if (tid < 2 * L) al[tid] = areg;
 #pragma unroll
-    for (int t = 0; t < NK * 2; ++t)
-      if (t < ns) {
-        const float hi4[4] = {S[t][0], S[t][1], S[t][2], S[t][3]};
-        uint16_t* at = sh + (wid * 16 + lo) * NP + t * 16 + hi * 4;
-        st_bf16x4(at, hi4);
-        float lo4[4];
-#pragma unroll
-        for (int r = 0; r < 4; ++r) lo4[r] = hi4[r] - bf16_to_f32(at[r]);
-        st_bf16x4(sl + (wid * 16 + lo) * NP + t * 16 + hi * 4, lo4);
+    for (int t = 0; t < ST; ++t)
+      if (t < nts) {
+        const uint32_t u0 = pack_bf16(S[t][0], S[t][1]);
+        const uint32_t u1 = pack_bf16(S[t][2], S[t][3]);
+        const int at = (pt * 16 + lo) * NP + (nt0 + t) * 16 + hi * 4;
+        *reinterpret_cast<u32x2*>(sh + at) = u32x2{u0, u1};
+        const float rest[4] = {
+            S[t][0] - bf16_to_f32((uint16_t)u0),
+            S[t][1] - bf16_to_f32((uint16_t)(u0 >> 16)),
+            S[t][2] - bf16_to_f32((uint16_t)u1),
+            S[t][3] - bf16_to_f32((uint16_t)(u1 >> 16))};
+        st_bf16x4(sl + at, rest);
       }
     u16x8 cf[NK];
 #pragma unroll
     for (int k = 0; k < NK; ++k) cf[k] = creg[k];
     __syncthreads();
+    // this chunk's gates and the next one's operands are on their way while
+    // the products run
+    const int i = wid * 16 + lo;
+    const int64_t row = row0 + (int64_t)(n - n0) * L + i;
+    const uint16_t* zr =
+        z + min(row, (int64_t)row1 - 1) * m.z_stride + m.z_at + h * m.P + p0;
+    u16x4 zreg[PW];
+    if (m.vec) {
+#pragma unroll
+      for (int t = 0; t < PW; ++t) {
+        zreg[t] = u16x4{0, 0, 0, 0};
+        if (t * 16 + hi * 4 < np)
+          zreg[t] = *reinterpret_cast<const u16x4*>(zr + t * 16 + hi * 4);
+      }
+    }
     if (n + 1 < n1) load(n + 1);
 
     // --- scores, transposed: lane has token i, 8 neighbouring j a group
-    const int i = wid * 16 + lo;
     const float ai = al[i];
     u16x8 mh[2], mlow[2];
 #pragma unroll
@@ -303,9 +375,8 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void ssm_chunks_kernel(
     }
     // --- outputs, transposed: lane has token i, values 4 hi + r
     const float ei = __expf(ai);
-    const int64_t row = row0 + (int64_t)(n - n0) * L + i;
 #pragma unroll
-    for (int t = 0; t < 4; ++t) {
+    for (int t = 0; t < PW; ++t) {
       if (t * 16 >= np) continue;
       floatx4 o = floatx4{0, 0, 0, 0};
       const uint16_t* s1 = sh + (t * 16 + lo) * NP + hi * 8;
@@ -327,16 +398,16 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void ssm_chunks_kernel(
       }
       if (row < row1) {
         const int p = t * 16 + hi * 4;
-        const int64_t zc = row * m.z_stride + m.z_at + h * m.P + p0 + p;
         uint16_t* dst = y + row * m.y_stride + h * m.P + p0 + p;
+        float v[4];
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          v[r] = o[r] + Dh * bf16_to_f32(xl[(p + r) * LP + i]);
         if (m.vec) {
           if (p < np) {
-            const u16x4 zz = *reinterpret_cast<const u16x4*>(z + zc);
-            float v[4];
 #pragma unroll
             for (int r = 0; r < 4; ++r)
-              v[r] = (o[r] + m.D[h] * bf16_to_f32(xl[(p + r) * LP + i])) *
-                     silu_s<uint16_t>(bf16_to_f32(zz[r]));
+              v[r] *= silu_s<uint16_t>(bf16_to_f32(zreg[t][r]));
             st_bf16x4(dst, v);
           }
         } else {
@@ -344,22 +415,21 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void ssm_chunks_kernel(
           for (int r = 0; r < 4; ++r)
             if (p + r < np)
               dst[r] = f32_to_bf16(
-                  (o[r] + m.D[h] * bf16_to_f32(xl[(p + r) * LP + i])) *
-                  silu_s<uint16_t>(bf16_to_f32(z[zc + r])));
+                  v[r] * silu_s<uint16_t>(bf16_to_f32(zr[p + r])));
         }
       }
     }
     // --- state
-    if (wid * 16 < np) {
+    if (pt * 16 < np) {
       const float end = al[L - 1], ee = __expf(end);
 #pragma unroll
-      for (int t = 0; t < NK * 2; ++t)
+      for (int t = 0; t < ST; ++t)
 #pragma unroll
         for (int r = 0; r < 4; ++r) S[t][r] *= ee;
 #pragma unroll
       for (int kk = 0; kk < 2; ++kk) {
         const u16x8 x =
-            ld_u16x8(xl + (wid * 16 + lo) * LP + kk * 32 + hi * 8);
+            ld_u16x8(xl + (pt * 16 + lo) * LP + kk * 32 + hi * 8);
         float v[8];
 #pragma unroll
         for (int q = 0; q < 8; ++q) {
@@ -369,10 +439,10 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void ssm_chunks_kernel(
         u16x8 xh, xlow;
         split8(v, xh, xlow);
 #pragma unroll
-        for (int t = 0; t < NK * 2; ++t)
-          if (t < ns) {
-            const u16x8 a =
-                ld_u16x8(btl + (t * 16 + lo) * LP + kk * 32 + hi * 8);
+        for (int t = 0; t < ST; ++t)
+          if (t < nts) {
+            const u16x8 a = ld_u16x8(btl + ((nt0 + t) * 16 + lo) * LP +
+                                     kk * 32 + hi * 8);
             S[t] = mfma16(a, xh, S[t]);
             S[t] = mfma16(a, xlow, S[t]);
           }
@@ -381,11 +451,11 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void ssm_chunks_kernel(
   }
   if (slot >= 0 && pcol < m.P) {
 #pragma unroll
-    for (int t = 0; t < NK * 2; ++t)
+    for (int t = 0; t < ST; ++t)
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        const int n = t * 16 + hi * 4 + r;
-        if (n < m.N) st[(int64_t)n * m.P] = S[t][r];
+        const int n = (nt0 + t) * 16 + hi * 4 + r;
+        if (t < nts && n < m.N) st[(int64_t)n * m.P] = S[t][r];
       }
   }
 }
@@ -395,8 +465,8 @@ void check(const torch::Tensor& t, torch::ScalarType type, int64_t n) {
               "ssm chunks: operand of ", t.numel(), " values, want ", n);
 }
 
-int chunk_lds(int Np) {
-  return (3 * L * (Np + 8) + Np * LP + 64 * LP) * 2 + 2 * L * 4;
+int chunk_lds(int Np, int PB) {
+  return ((L + 2 * PB) * (Np + 8) + (Np + PB) * LP) * 2 + 2 * L * 4;
 }
 
 }  // namespace
@@ -463,8 +533,10 @@ void conv_chunks(torch::Tensor xt, torch::Tensor b, torch::Tensor bt,
   m.dt_at = dt_at;
   if (n == 0) return;
   auto stream = at::hip::getCurrentHIPStream();
-  const int rows = L + m.taps - 1;
-  const int lds = ((rows * 65 + 3) & ~3) * 4 + L * LP * 2;
+  // 16-byte loads: every block of channels starts on 8 and is whole
+  m.vec = m.P % 8 == 0 && m.N % 8 == 0 && m.C % 8 == 0 && xbc_at % 8 == 0 &&
+          m.z_stride % 8 == 0 && (uintptr_t)z.data_ptr() % 16 == 0;
+  const int lds = (L + m.taps - 1 + 64 + L) * LP * 2;
   const dim3 grid(n, m.H * cdiv(m.P, 64) + 2 * m.G * cdiv(m.Np, 64) +
                          cdiv(m.H, 4));
   hipLaunchKernelGGL(conv_chunks_kernel, grid, dim3(NT), lds, stream,
@@ -522,25 +594,30 @@ void ssm_chunks(torch::Tensor y, torch::Tensor z, int64_t z_at, int64_t vdim,
           (uintptr_t)y.data_ptr() % 8 == 0;
   if (B == 0 || n == 0) return;
   auto stream = at::hip::getCurrentHIPStream();
-  const dim3 grid(m.H, B, cdiv(m.P, 64));
-  const int lds = chunk_lds(m.Np);
-#define HELIX_SSM(NK)                                                        \
+  // few heads and sequences: half the values to a workgroup
+  const int PW = (int64_t)m.H * B * cdiv(m.P, 64) < 256 ? 2 : 4;
+  const dim3 grid(m.H, B, cdiv(m.P, PW * 16));
+  const int lds = chunk_lds(m.Np, PW * 16);
+#define HELIX_SSM_P(NK, PW)                                                  \
   do {                                                                       \
     static const hipError_t big = hipFuncSetAttribute(                       \
-        (const void*)ssm_chunks_kernel<NK>,                                  \
+        (const void*)ssm_chunks_kernel<NK, PW>,                              \
         hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);             \
     TORCH_CHECK(big == hipSuccess, "LDS size refused");                      \
-    hipLaunchKernelGGL((ssm_chunks_kernel<NK>), grid, dim3(NT), lds, stream, \
-                       (uint16_t*)y.data_ptr(),                              \
+    hipLaunchKernelGGL((ssm_chunks_kernel<NK, PW>), grid, dim3(NT), lds,     \
+                       stream, (uint16_t*)y.data_ptr(),                      \
                        (const uint16_t*)z.data_ptr(),                        \
                        (const uint16_t*)xt.data_ptr(),                       \
                        (const uint16_t*)b.data_ptr(),                        \
                        (const uint16_t*)bt.data_ptr(),                       \
                        (const uint16_t*)c.data_ptr(), m);                    \
   } while (0)
-  if (m.Np <= 32) HELIX_SSM(1);
-  else if (m.Np <= 64) HELIX_SSM(2);
-  else if (m.Np <= 128) HELIX_SSM(4);
-  else HELIX_SSM(8);
+#define HELIX_SSM(NK)                                                        \
+  if (PW == 4) HELIX_SSM_P(NK, 4); else HELIX_SSM_P(NK, 2)
+  if (m.Np <= 32) { HELIX_SSM(1); }
+  else if (m.Np <= 64) { HELIX_SSM(2); }
+  else if (m.Np <= 128) { HELIX_SSM(4); }
+  else { HELIX_SSM(8); }
 #undef HELIX_SSM
+#undef HELIX_SSM_P
 }

@@ -12,6 +12,7 @@ import torch
 from . import build
 from . import hybrid_reference as ref
 
+
 def _native():
     return build.load("_C_hybrid")
 
@@ -122,7 +123,7 @@ def latent_epilogue(z: torch.Tensor, p: LatentParams,
 
 
 # Cached rows of a partition at least; enough workgroups to fill the chip.
-LATENT_PART = 128
+LATENT_PART = 64
 LATENT_TARGET_WGS = 512
 
 
@@ -295,7 +296,15 @@ def ssm_prompt(y: torch.Tensor, z: torch.Tensor, p: SSMParams, w: SSMWeights,
                    w.dt_bias, w.A_log, w.D, ring, state, meta.state_slots,
                    meta.positions, meta.cu_seqlens)
         return
-    ch = meta.chunks(SSM_CHUNK)
+    for step in ssm_chunk_steps(y, z, p, w, cache, meta):
+        step()
+
+
+def ssm_chunk_steps(y: torch.Tensor, z: torch.Tensor, p: SSMParams,
+                    w: SSMWeights, cache, meta):
+    """The two launches of a prompt in chunks: operands, then recurrence."""
+    ring, state = cache
+    ch, C = meta.chunks(SSM_CHUNK), _native()
     n, dev = ch.seq.shape[0], z.device
     Pp, Np = -(-p.vdim // 16) * 16, -(-p.state // 32) * 32
     xt = torch.empty(n, p.heads, Pp, SSM_CHUNK, dtype=z.dtype, device=dev)
@@ -304,9 +313,16 @@ def ssm_prompt(y: torch.Tensor, z: torch.Tensor, p: SSMParams, w: SSMWeights,
     bt = torch.empty(n, p.groups, Np, SSM_CHUNK, dtype=z.dtype, device=dev)
     da = torch.empty(n, p.heads, 2, SSM_CHUNK, dtype=torch.float32,
                      device=dev)
-    C.conv_chunks(xt, b, bt, c, da, z, p.xbc_at, p.dt_at, p.vdim, p.state,
-                  w.conv, w.conv_b, w.dt_bias, w.A_log, ring,
-                  meta.state_slots, meta.positions, meta.cu_seqlens, ch.seq,
-                  ch.row, ch.count)
-    C.ssm_chunks(y, z, p.z_at, p.vdim, p.state, xt, b, bt, c, da, w.D, state,
-                 meta.state_slots, meta.positions, meta.cu_seqlens, ch.first)
+
+    def operands():
+        C.conv_chunks(xt, b, bt, c, da, z, p.xbc_at, p.dt_at, p.vdim,
+                      p.state, w.conv, w.conv_b, w.dt_bias, w.A_log, ring,
+                      meta.state_slots, meta.positions, meta.cu_seqlens,
+                      ch.seq, ch.row, ch.count)
+
+    def recurrence():
+        C.ssm_chunks(y, z, p.z_at, p.vdim, p.state, xt, b, bt, c, da, w.D,
+                     state, meta.state_slots, meta.positions,
+                     meta.cu_seqlens, ch.first)
+
+    return operands, recurrence

@@ -53,6 +53,8 @@ DEFAULT_SPECS = {
                           max_model_len=32768),
     "zederax-8b": ModelSpec("zederax-8b", "llm", "zederax-8b"),
     "zederax-1b": ModelSpec("zederax-1b", "llm", "zederax-1b"),
+    "nibezen-8b": ModelSpec("nibezen-8b", "llm", "nibezen-8b"),
+    "nibezen-1b": ModelSpec("nibezen-1b", "llm", "nibezen-1b"),
     "bge-base": ModelSpec("bge-base", "embedding", "bge-base"),
     "siglip-base": ModelSpec("siglip-base", "vision", "siglip-base"),
     "tiny-vit": ModelSpec("tiny-vit", "vision", "tiny-vit"),
@@ -65,6 +67,8 @@ DEFAULT_SPECS = {
     "tiny-gqa": ModelSpec("tiny-gqa", "llm", "tiny-gqa", max_model_len=512,
                           kv_cache_blocks=256),
     "tiny-zederax": ModelSpec("tiny-zederax", "llm", "tiny-zederax",
+                              max_model_len=256, kv_cache_blocks=256),
+    "tiny-nibezen": ModelSpec("tiny-nibezen", "llm", "tiny-nibezen",
                               max_model_len=256, kv_cache_blocks=256),
     "tiny-bert": ModelSpec("tiny-bert", "embedding", "tiny-bert"),
 }

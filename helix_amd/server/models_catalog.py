@@ -30,6 +30,12 @@ STATIC_MODEL_INFO: Dict[str, dict] = {
     "zederax-1b": {"context_length": 8192, "prompt_price_per_m": 0.02,
                    "completion_price_per_m": 0.04, "family": "zederax",
                    "runtime": "helix_amd", "kind": "chat"},
+    "nibezen-8b": {"context_length": 32768, "prompt_price_per_m": 0.05,
+                   "completion_price_per_m": 0.10, "family": "nibezen",
+                   "runtime": "helix_amd", "kind": "chat"},
+    "nibezen-1b": {"context_length": 32768, "prompt_price_per_m": 0.02,
+                   "completion_price_per_m": 0.04, "family": "nibezen",
+                   "runtime": "helix_amd", "kind": "chat"},
     "bge-base": {"context_length": 512, "prompt_price_per_m": 0.005,
                  "completion_price_per_m": 0.0, "family": "bge",
                  "runtime": "helix_amd", "kind": "embedding"},
