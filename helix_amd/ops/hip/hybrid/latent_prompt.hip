@@ -70,25 +70,28 @@ void latent_prompt_kernel(uint16_t* __restrict__ out,
     }
   }
 
+  // Loads without branches, so that all are under way at once: addresses
+  // past the end are clamped. What they bring meets a zero query column, a
+  // zero weight or a value dimension that is not stored.
   u16x8 kreg[NK], vreg[NV / 2];
+  const uint16_t* kh = k + h * m.dim_pad;
+  const uint16_t* vh = vt + (int64_t)h * m.E * m.rows;
   auto load = [&](int t) {
 #pragma unroll
     for (int c = 0; c < NK; ++c) {
-      const int e = c * NT + tid, key = e / (NK * 4), d = e % (NK * 4) * 8;
+      const int e = c * NT + tid, key = e / (NK * 4);
+      const int d = min(e % (NK * 4) * 8, m.head_cols - 8);
       const int64_t r = k0 + min(t + key, klen - 1);
-      kreg[c] = d < m.dim_pad
-                    ? ld_u16x8(k + (r * m.H + h) * m.dim_pad + d)
-                    : (d < m.head_cols
-                           ? ld_u16x8(kr + r * m.kr_stride + d - m.dim_pad)
-                           : zero);
+      const uint16_t* src = d < m.dim_pad
+                                ? kh + r * m.H * m.dim_pad + d
+                                : kr + r * m.kr_stride + d - m.dim_pad;
+      kreg[c] = ld_u16x8(src);
     }
 #pragma unroll
     for (int c = 0; c < NV / 2; ++c) {
-      const int e = c * NT + tid, dim = e / 8, key = e % 8 * 8;
-      const int64_t r = k0 + t + key;
-      vreg[c] = dim < m.E && r + 8 <= m.rows
-                    ? ld_u16x8(vt + ((int64_t)h * m.E + dim) * m.rows + r)
-                    : zero;
+      const int e = c * NT + tid, dim = min(e / 8, m.E - 1);
+      const int64_t r = min(k0 + t + e % 8 * 8, m.rows - 8);
+      vreg[c] = ld_u16x8(vh + dim * m.rows + r);
     }
   };
 

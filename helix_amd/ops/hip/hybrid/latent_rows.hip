@@ -199,18 +199,18 @@ __global__ __launch_bounds__(NT) void absorb_mfma_kernel(
 #pragma unroll
   for (int t = 0; t < 8; ++t) acc[t] = floatx4{0, 0, 0, 0};
   const int k0 = blockIdx.z * 128;
-  for (int d = hi * 8; d < ((dim_pad + 31) & ~31); d += 32) {
-    const bool in = d < dim_pad;
-    const u16x8 b = in ? ld_u16x8(zh + d) : zero;
+  for (int d0 = hi * 8; d0 < ((dim_pad + 31) & ~31); d0 += 32) {
+    // clamped columns meet a zero, clamped rows are not stored
+    const int d = min(d0, dim_pad - 8);
+    const u16x8 raw = ld_u16x8(zh + d), b = d == d0 ? raw : zero;
+    u16x8 a[8];
 #pragma unroll
-    for (int t = 0; t < 8; ++t) {
-      const int k = k0 + t * 16 + lo;
-      const u16x8 a = in && k < rank_pad
-                          ? ld_u16x8(ukt + ((int64_t)h * rank_pad + k) *
-                                               dim_pad + d)
-                          : zero;
-      acc[t] = mfma16(a, b, acc[t]);
-    }
+    for (int t = 0; t < 8; ++t)
+      a[t] = ld_u16x8(ukt + ((int64_t)h * rank_pad +
+                             min(k0 + t * 16 + lo, rank_pad - 1)) * dim_pad +
+                      d);
+#pragma unroll
+    for (int t = 0; t < 8; ++t) acc[t] = mfma16(a[t], b, acc[t]);
   }
   if (r < R) {
 #pragma unroll
@@ -323,10 +323,11 @@ __global__ __launch_bounds__(NT, 2) void latent_rows_kernel(
   auto load = [&](int buf) {
 #pragma unroll
     for (int c = 0; c < NL; ++c) {
-      const int e = c * NT + tid, key = e / (NK * 4), d = e % (NK * 4) * 8;
-      reg[c] = d < m.row
-                   ? ld_u16x8(cache + (int64_t)slots[buf][key] * m.row + d)
-                   : zero;
+      // no branch, so that all loads are under way at once; columns past
+      // the row meet zeros of the query
+      const int e = c * NT + tid, key = e / (NK * 4);
+      const int d = min(e % (NK * 4) * 8, m.row - 8);
+      reg[c] = ld_u16x8(cache + (int64_t)slots[buf][key] * m.row + d);
     }
   };
   // page lookups run two tiles ahead of the rows, so no load waits for one
@@ -571,14 +572,22 @@ __global__ __launch_bounds__(NT) void latent_out_kernel(
           v = ld_u16x8(o + ((int64_t)r * H + h) * K + d);
         } else {
           float a[8] = {0, 0, 0, 0, 0, 0, 0, 0};
-          for (int p = 0; p < parts; ++p) {
-            const float ls = st[(int64_t)p * H * 2 + 1];
-            if (ls == 0.f) continue;          // an empty partition
-            const float w = __expf(st[(int64_t)p * H * 2] - M) * L;
-            float b[8];
-            ldv<8>(part_o + (((int64_t)r * parts + p) * H + h) * K + d, b);
+          const float* po = part_o + ((int64_t)r * parts * H + h) * K + d;
+          for (int p = 0; p < parts; p += 8) {
+            float b[8][8], w[8];
 #pragma unroll
-            for (int j = 0; j < 8; ++j) a[j] += w * b[j];
+            for (int i = 0; i < 8; ++i) {
+              const int64_t q = min(p + i, parts - 1);
+              const float* s = st + q * H * 2;
+              w[i] = p + i < parts && s[1] > 0.f ? __expf(s[0] - M) * L : 0.f;
+              ldv<8>(po + q * H * K, b[i]);
+            }
+#pragma unroll
+            for (int i = 0; i < 8; ++i)
+              if (w[i] > 0.f) {               // not an empty partition
+#pragma unroll
+                for (int j = 0; j < 8; ++j) a[j] += w[i] * b[i][j];
+              }
           }
           v = pack8(a);
         }
@@ -595,7 +604,7 @@ __global__ __launch_bounds__(NT) void latent_out_kernel(
     const uint16_t* ur = uv + ((int64_t)h * E + min(e0 + lo, E - 1)) * K;
 #pragma unroll 4
     for (int k = 0; k < pitch - 8; k += 32) {
-      const u16x8 a = k + hi * 8 < K ? ld_u16x8(ur + k + hi * 8) : zero;
+      const u16x8 a = ld_u16x8(ur + min(k + hi * 8, K - 8));
 #pragma unroll
       for (int t = 0; t < RT; ++t)
         acc[t] = mfma16(a, ld_u16x8(ol + (t * 16 + lo) * pitch + k + hi * 8),
@@ -905,7 +914,10 @@ void latent_out(torch::Tensor out, OptT o, OptT part, OptT ml,
   const int pitch = ((K + 31) & ~31) + 8;
   const int vec = E % 4 == 0 && out.stride(0) % 4 == 0 &&
                   (uintptr_t)out.data_ptr() % 8 == 0;
-  const int zs = std::min(cdiv(E, 64), R <= 64 ? 8 : 1);
+  // few rows: more workgroups, unless each would merge partitions again
+  const int tiles = cdiv(R, 16) * H;
+  const int zs = std::min(cdiv(E, 64), parts > 1 ? std::max(1, 128 / tiles)
+                                                 : (R <= 64 ? 8 : 1));
 #define HELIX_OUT(RT)                                                        \
   hipLaunchKernelGGL((latent_out_kernel<RT>), dim3(cdiv(R, RT * 16), H, zs), \
                      dim3(NT), RT * 16 * pitch * 2, stream,                  \
@@ -918,7 +930,7 @@ void latent_out(torch::Tensor out, OptT o, OptT part, OptT ml,
                      gate.has_value() ? (const uint16_t*)gate->data_ptr()    \
                                       : nullptr,                             \
                      gs, R, H, E, K, parts, vec)
-  if (R > 16 && K <= 512) HELIX_OUT(2);
+  if (R > 16 && K <= 512 && parts == 1) HELIX_OUT(2);
   else {
     TORCH_CHECK(K <= 1536, "latent size ", K);
     HELIX_OUT(1);

@@ -242,7 +242,10 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void ssm_chunks_kernel(
   float* al = (float*)(sl + PB * NP);         // [64] sums, [64] steps
   float* dl = al + L;
 
-  const int seq = blockIdx.y, h = blockIdx.x, p0 = blockIdx.z * PB;
+  // neighbouring heads share B and C: an XCD gets a contiguous range
+  const int h = m.H % 8 ? blockIdx.x
+                        : (blockIdx.x & 7) * (m.H / 8) + (blockIdx.x >> 3);
+  const int seq = blockIdx.y, p0 = blockIdx.z * PB;
   const int g = h / (m.H / m.G);
   const int tid = threadIdx.x, wid = tid / WAVE, lane = tid & (WAVE - 1);
   const int lo = lane & 15, hi = lane >> 4;
@@ -251,8 +254,6 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void ssm_chunks_kernel(
   const int slot = m.slots[seq];
   const int n0 = m.first[seq], n1 = m.first[seq + 1];
   const int ks = m.Np / 32, per = m.Np / 8;
-  const u16x8 zero = {0, 0, 0, 0, 0, 0, 0, 0};
-
   // this wave's 16 columns of the state: lane has column lo, rows 4 hi + r
   // of the nts row tiles from nt0 on
   const int pt = wid % PW, pcol = p0 + pt * 16 + lo;
@@ -270,31 +271,26 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void ssm_chunks_kernel(
 
   u16x8 breg[NK], btreg[NK], xreg[XL], creg[NK];
   float areg = 0.f;
+  // No branches, so that all loads are under way at once: indices past the
+  // end are clamped and their values not stored.
   auto load = [&](int n) {
+    const int64_t at = (int64_t)n * L * m.G * m.Np;
+    const uint16_t* bn = b + at + g * m.Np;
+    const uint16_t* btn = bt + at + (int64_t)g * m.Np * L;
+    const uint16_t* cn =
+        c + at + ((int64_t)(wid * 16 + lo) * m.G + g) * m.Np + hi * 8;
 #pragma unroll
     for (int i = 0; i < NK; ++i) {
-      const int e = i * NT + tid;
-      breg[i] = btreg[i] = zero;
-      if (e < L * per)
-        breg[i] = ld_u16x8(
-            b + (((int64_t)n * L + e / per) * m.G + g) * m.Np + e % per * 8);
-      if (e < m.Np * 8)
-        btreg[i] =
-            ld_u16x8(bt + ((int64_t)n * m.G + g) * m.Np * L + e * 8);
-      creg[i] = i < ks ? ld_u16x8(c + (((int64_t)n * L + wid * 16 + lo) *
-                                           m.G + g) * m.Np +
-                                  i * 32 + hi * 8)
-                       : zero;
+      const int e = min(i * NT + tid, L * per - 1);
+      breg[i] = ld_u16x8(bn + (int64_t)(e / per) * m.G * m.Np + e % per * 8);
+      btreg[i] = ld_u16x8(btn + e * 8);
+      creg[i] = ld_u16x8(cn + min(i, ks - 1) * 32);
     }
+    const uint16_t* xn = xt + (((int64_t)n * m.H + h) * m.Pp + p0) * L;
 #pragma unroll
-    for (int i = 0; i < XL; ++i) {
-      const int e = i * NT + tid;
-      xreg[i] = e < rowsp * 8
-                    ? ld_u16x8(xt + (((int64_t)n * m.H + h) * m.Pp + p0) * L +
-                               e * 8)
-                    : zero;
-    }
-    if (tid < 2 * L) areg = m.da[((int64_t)n * m.H + h) * 2 * L + tid];
+    for (int i = 0; i < XL; ++i)
+      xreg[i] = ld_u16x8(xn + min(i * NT + tid, rowsp * 8 - 1) * 8);
+    areg = m.da[((int64_t)n * m.H + h) * 2 * L + (tid & (2 * L - 1))];
   };
 
   const float Dh = m.D[h];
@@ -342,11 +338,9 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void ssm_chunks_kernel(
     u16x4 zreg[PW];
     if (m.vec) {
 #pragma unroll
-      for (int t = 0; t < PW; ++t) {
-        zreg[t] = u16x4{0, 0, 0, 0};
-        if (t * 16 + hi * 4 < np)
-          zreg[t] = *reinterpret_cast<const u16x4*>(zr + t * 16 + hi * 4);
-      }
+      for (int t = 0; t < PW; ++t)
+        zreg[t] = *reinterpret_cast<const u16x4*>(
+            zr + min(t * 16 + hi * 4, np - 4));
     }
     if (n + 1 < n1) load(n + 1);
 
@@ -355,7 +349,6 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void ssm_chunks_kernel(
     u16x8 mh[2], mlow[2];
 #pragma unroll
     for (int jp = 0; jp < 2; ++jp) {
-      mh[jp] = mlow[jp] = zero;
       if (jp > (wid >> 1)) continue;
       float v[8];
 #pragma unroll
