@@ -111,8 +111,8 @@ void latent_prompt_kernel(uint16_t* __restrict__ out,
 #pragma unroll
     for (int c = 0; c < NK; ++c) {
       const int e = c * NT + tid;
-      *reinterpret_cast<u16x8*>(kl + e / (NK * 4) * KP + e % (NK * 4) * 8) =
-          kreg[c];
+      *reinterpret_cast<u16x8*>(kl + paired_row(e / (NK * 4)) * KP +
+                                e % (NK * 4) * 8) = kreg[c];
     }
 #pragma unroll
     for (int c = 0; c < NV / 2; ++c) {
@@ -129,7 +129,7 @@ void latent_prompt_kernel(uint16_t* __restrict__ out,
 #pragma unroll
       for (int j = 0; j < 2; ++j) {
         s[g][j][0] = s[g][j][1] = floatx4{0, 0, 0, 0};
-        const uint16_t* row = kl + (g * 32 + paired_row(lo, j)) * KP + hi * 8;
+        const uint16_t* row = kl + (g * 32 + j * 16 + lo) * KP + hi * 8;
 #pragma unroll
         for (int c = 0; c < NK; ++c) {
           const u16x8 a = ld_u16x8(row + c * 32);

@@ -13,7 +13,7 @@
 // matrix, the weighted x) enters as two bf16 terms, 17 significant bits.
 //
 // Layouts per chunk: xt [H, Pp, 64], b and c [64, G, Np], bt [G, Np, 64],
-// da [H, 2, 64] (A_t and dt_t). Tokens past a portion's end and state
+// da [H, 3, 64] (A_t, dt_t and e^(A_63 - A_t) dt_t). Tokens past a portion's end and state
 // columns past N are zero.
 #include "tile.h"
 #include <torch/extension.h>
@@ -67,9 +67,10 @@ __global__ __launch_bounds__(NT) void conv_chunks_kernel(
       const float up = __shfl_up(a, off, WAVE);
       if (t >= off) a += up;
     }
-    float* o = da + ((int64_t)n * m.H + h) * 2 * L;
+    float* o = da + ((int64_t)n * m.H + h) * 3 * L;
     o[t] = a;
     o[L + t] = dt;
+    o[2 * L + t] = __expf(__shfl(a, WAVE - 1, WAVE) - a) * dt;
     return;
   }
 
@@ -239,8 +240,8 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void ssm_chunks_kernel(
   uint16_t* xl = btl + m.Np * LP;             // [PB values][LP]
   uint16_t* sh = xl + PB * LP;                // [PB values][NP]
   uint16_t* sl = sh + PB * NP;
-  float* al = (float*)(sl + PB * NP);         // [64] sums, [64] steps
-  float* dl = al + L;
+  float* al = (float*)(sl + PB * NP);         // sums, steps, weights: [64]
+  float *dl = al + L, *wl = dl + L;
 
   // neighbouring heads share B and C: an XCD gets a contiguous range
   const int h = m.H % 8 ? blockIdx.x
@@ -290,7 +291,7 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void ssm_chunks_kernel(
 #pragma unroll
     for (int i = 0; i < XL; ++i)
       xreg[i] = ld_u16x8(xn + min(i * NT + tid, rowsp * 8 - 1) * 8);
-    areg = m.da[((int64_t)n * m.H + h) * 2 * L + (tid & (2 * L - 1))];
+    areg = m.da[((int64_t)n * m.H + h) * 3 * L + min(tid, 3 * L - 1)];
   };
 
   const float Dh = m.D[h];
@@ -301,7 +302,8 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void ssm_chunks_kernel(
     for (int i = 0; i < NK; ++i) {
       const int e = i * NT + tid;
       if (e < L * per)
-        *reinterpret_cast<u16x8*>(bl + e / per * NP + e % per * 8) = breg[i];
+        *reinterpret_cast<u16x8*>(bl + paired_row(e / per) * NP +
+                                  e % per * 8) = breg[i];
       if (e < m.Np * 8)
         *reinterpret_cast<u16x8*>(btl + e / 8 * LP + e % 8 * 8) = btreg[i];
     }
@@ -310,7 +312,7 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void ssm_chunks_kernel(
       const int e = i * NT + tid;
       *reinterpret_cast<u16x8*>(xl + e / 8 * LP + e % 8 * 8) = xreg[i];
     }
-    if (tid < 2 * L) al[tid] = areg;
+    if (tid < 3 * L) al[tid] = areg;
 #pragma unroll
     for (int t = 0; t < ST; ++t)
       if (t < nts) {
@@ -354,15 +356,16 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void ssm_chunks_kernel(
 #pragma unroll
       for (int s = 0; s < 2; ++s) {
         floatx4 d = floatx4{0, 0, 0, 0};
-        const uint16_t* br = bl + (jp * 32 + paired_row(lo, s)) * NP + hi * 8;
+        const uint16_t* br = bl + (jp * 32 + s * 16 + lo) * NP + hi * 8;
 #pragma unroll
         for (int k = 0; k < NK; ++k)
           if (k < ks) d = mfma16(ld_u16x8(br + k * 32), cf[k], d);
+        const int j = jp * 32 + hi * 8 + s * 4;
+        const f32x4 aj = *reinterpret_cast<const f32x4*>(al + j);
+        const f32x4 dj = *reinterpret_cast<const f32x4*>(dl + j);
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int j = jp * 32 + hi * 8 + s * 4 + r;
-          v[s * 4 + r] = j <= i ? d[r] * __expf(ai - al[j]) * dl[j] : 0.f;
-        }
+        for (int r = 0; r < 4; ++r)
+          v[s * 4 + r] = j + r <= i ? d[r] * __expf(ai - aj[r]) * dj[r] : 0.f;
       }
       split8(v, mh[jp], mlow[jp]);
     }
@@ -414,7 +417,7 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void ssm_chunks_kernel(
     }
     // --- state
     if (pt * 16 < np) {
-      const float end = al[L - 1], ee = __expf(end);
+      const float ee = __expf(al[L - 1]);
 #pragma unroll
       for (int t = 0; t < ST; ++t)
 #pragma unroll
@@ -423,12 +426,10 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void ssm_chunks_kernel(
       for (int kk = 0; kk < 2; ++kk) {
         const u16x8 x =
             ld_u16x8(xl + (pt * 16 + lo) * LP + kk * 32 + hi * 8);
-        float v[8];
+        float v[8], w[8];
+        ldv<8>(wl + kk * 32 + hi * 8, w);
 #pragma unroll
-        for (int q = 0; q < 8; ++q) {
-          const int j = kk * 32 + hi * 8 + q;
-          v[q] = bf16_to_f32(x[q]) * (__expf(end - al[j]) * dl[j]);
-        }
+        for (int q = 0; q < 8; ++q) v[q] = bf16_to_f32(x[q]) * w[q];
         u16x8 xh, xlow;
         split8(v, xh, xlow);
 #pragma unroll
@@ -459,7 +460,7 @@ void check(const torch::Tensor& t, torch::ScalarType type, int64_t n) {
 }
 
 int chunk_lds(int Np, int PB) {
-  return ((L + 2 * PB) * (Np + 8) + (Np + PB) * LP) * 2 + 2 * L * 4;
+  return ((L + 2 * PB) * (Np + 8) + (Np + PB) * LP) * 2 + 3 * L * 4;
 }
 
 }  // namespace
@@ -497,7 +498,7 @@ void conv_chunks(torch::Tensor xt, torch::Tensor b, torch::Tensor bt,
   check(b, BF, n * L * m.G * m.Np);
   check(c, BF, b.numel());
   check(bt, BF, b.numel());
-  check(da, F32, n * m.H * 2 * L);
+  check(da, F32, n * m.H * 3 * L);
   check(conv, F32, (int64_t)m.C * m.taps);
   check(conv_b, F32, m.C);
   check(dt_bias, F32, m.H);
@@ -562,7 +563,7 @@ void ssm_chunks(torch::Tensor y, torch::Tensor z, int64_t z_at, int64_t vdim,
   check(b, BF, n * L * m.G * m.Np);
   check(c, BF, b.numel());
   check(bt, BF, b.numel());
-  check(da, F32, n * m.H * 2 * L);
+  check(da, F32, n * m.H * 3 * L);
   check(D, F32, m.H);
   check(state, F32, state.size(0) * m.H * m.N * m.P);
   check(slots, I32, B);

@@ -16,10 +16,12 @@ __device__ __forceinline__ floatx4 mfma16(u16x8 a, u16x8 b, floatx4 c) {
       0);
 }
 
-// Row of a 32-row group that row `lo` of half `sub` stands for, so that the
-// two results' lanes hold 8 neighbouring rows: lane hi has 8 hi + 4 sub + r.
-__device__ __forceinline__ int paired_row(int lo, int sub) {
-  return (lo >> 2) * 8 + sub * 4 + (lo & 3);
+// Where row r of a tile is stored in LDS when its products should leave 8
+// neighbouring rows to a lane: rows 8 a + 4 s + b of a group of 32 go to
+// 16 s + 4 a + b, so an A operand of half s is 16 rows in a row (no bank
+// conflicts) and lane hi ends up with rows 8 hi + 4 s + r of its result.
+__device__ __forceinline__ int paired_row(int r) {
+  return (r & ~31) | (r & 4) << 2 | (r & 24) >> 1 | (r & 3);
 }
 
 __device__ __forceinline__ u16x8 pack8(const float* v) {

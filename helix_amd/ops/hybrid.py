@@ -311,7 +311,7 @@ def ssm_chunk_steps(y: torch.Tensor, z: torch.Tensor, p: SSMParams,
     b = torch.empty(n, SSM_CHUNK, p.groups, Np, dtype=z.dtype, device=dev)
     c = torch.empty_like(b)
     bt = torch.empty(n, p.groups, Np, SSM_CHUNK, dtype=z.dtype, device=dev)
-    da = torch.empty(n, p.heads, 2, SSM_CHUNK, dtype=torch.float32,
+    da = torch.empty(n, p.heads, 3, SSM_CHUNK, dtype=torch.float32,
                      device=dev)
 
     def operands():
