@@ -90,13 +90,12 @@ def kernels(z: NibezenConfig, device, decode_batch: int = 256,
         cache = rand(B * nb, 1, bs, p.row)
         q = rand(B, H, p.row)
         parts = hybrid.latent_parts(B, H, keys)
-        o = part = ml = None
-        if parts == 1:
-            o = rand(B, H, p.rank_pad)
-        else:
+        o, part, ml = rand(B, H, p.rank_pad), None, None
+        if parts > 1:
             part = rand(B, parts, H, p.rank_pad, dtype=torch.float32)
             ml = torch.empty(B, parts, H, 2, device=device)
-        t = _time(lambda: C.latent_rows(o, part, ml, q, cache, bt, None,
+        one = o if parts == 1 else None
+        t = _time(lambda: C.latent_rows(one, part, ml, q, cache, bt, None,
                                         lens, p.rank_pad, p.scale, p.window))
         new = _row(t, 2.0 * B * keys * p.row,
                    2.0 * B * keys * H * (p.row + p.rank_pad))
@@ -109,12 +108,16 @@ def kernels(z: NibezenConfig, device, decode_batch: int = 256,
         pair(f"decode_attention_b{B}_l{L}", new, like)
         zz = rand(B, mod.in_proj.weight.shape[0])
         gate, dst = zz[:, mod.gate_at:mod.gate_at + H], rand(B, H * E)
+
+        def value_out():
+            if parts > 1:
+                C.latent_merge(o, part, ml)
+            C.latent_out(dst, o, mod.uv, gate)
         for name, fn, wts, act in (
                 ("absorb", lambda: C.latent_absorb(
                     q, zz, 0, p.head_cols, p.dim_pad, mod.uk, mod.ukt,
                     p.rank_pad), H * D * K, H * (D + K)),
-                ("value_out", lambda: C.latent_out(
-                    dst, o, part, ml, mod.uv, gate), H * E * K,
+                ("value_out", value_out, H * E * K,
                     H * (E + K * (1 if parts == 1 else 2 * parts)))):
             new = _row(_time(fn), 2.0 * (wts + B * act), 2.0 * B * wts)
             x, w = rand(B, W), rand(wts // W, W)

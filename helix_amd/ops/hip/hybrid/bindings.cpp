@@ -23,7 +23,8 @@ void latent_rows(OptT o, OptT part, OptT ml, T q, T cache, T block_tables,
                  int64_t window);
 void latent_rows_plain(T o, T q, T cache, T block_tables, OptT row_seq,
                        T row_len, double scale, int64_t window);
-void latent_out(T out, OptT o, OptT part, OptT ml, T uv, OptT gate);
+void latent_merge(T o, T part, T ml);
+void latent_out(T out, T o, T uv, OptT gate);
 bool latent_prompt_fits(T z, int64_t dim_pad, int64_t rot_pad, int64_t vdim);
 void latent_prompt(T out, T z, int64_t q_at, int64_t head_cols,
                    int64_t heads, T k, T kr, T vt, T cu, T start, T length,
@@ -55,6 +56,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         "Paged latent attention, single query rows (MFMA)");
   m.def("latent_rows_plain", &latent_rows_plain,
         "Paged latent attention, single query rows of any size");
+  m.def("latent_merge", &latent_merge, "Partitions of a row into one");
   m.def("latent_out", &latent_out, "Values out of latent space, gate");
   m.def("latent_prompt_fits", &latent_prompt_fits);
   m.def("latent_prompt", &latent_prompt, "Latent attention of prompts (MFMA)");

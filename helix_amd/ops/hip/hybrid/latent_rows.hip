@@ -11,7 +11,7 @@
 // rows waits in LDS; it is the A operand of the scores as it lies and, read
 // with the transposing LDS load, that of the values. A workgroup's 4 waves
 // split rows x heads for the scores and the latent's dimensions for the
-// values. Partitions of long rows are merged by the out kernel.
+// values. Partitions of long rows are merged by a kernel of their own.
 //
 // Cache row: [latent, padded to 8 | shared rotated key part, padded to 8].
 #include "tile.h"
@@ -534,66 +534,83 @@ __global__ __launch_bounds__(NT) void latent_rows_plain_kernel(
   }
 }
 
+// -------------------------------------------------------------------- merge
+
+// o'[r, h] from its partitions, a workgroup per (row, head): the waves take
+// every fourth partition, 8 of them under way at once.
+__global__ __launch_bounds__(NT) void latent_merge_kernel(
+    uint16_t* __restrict__ o, const float* __restrict__ part_o,
+    const float* __restrict__ ml, int H, int K, int parts) {
+  __shared__ float sum[NT / WAVE][512];
+  const int r = blockIdx.x, h = blockIdx.y;
+  const int wid = __builtin_amdgcn_readfirstlane(threadIdx.x / WAVE);
+  const int lane = threadIdx.x & (WAVE - 1);
+  const float* st = ml + ((int64_t)r * parts * H + h) * 2;
+  float M = NEG, l = 0.f;
+  for (int p = lane; p < parts; p += WAVE)
+    M = fmaxf(M, st[(int64_t)p * H * 2]);
+  M = wave_reduce_max(M);
+  for (int p = lane; p < parts; p += WAVE)
+    l += st[(int64_t)p * H * 2 + 1] * __expf(st[(int64_t)p * H * 2] - M);
+  const float inv = 1.f / wave_reduce_sum(l);
+  for (int d0 = 0; d0 < K; d0 += 512) {
+    const int d = min(d0 + lane * 8, K - 8);
+    const float* po = part_o + ((int64_t)r * parts * H + h) * K + d;
+    float a[8] = {0, 0, 0, 0, 0, 0, 0, 0};
+    for (int p = wid; p < parts; p += 8 * (NT / WAVE)) {
+      float b[8][8], w[8];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const int64_t q = p + i * (NT / WAVE);
+        w[i] = 0.f;
+        if (q < parts) {                      // the same for all lanes
+          const float* s = st + q * H * 2;
+          w[i] = s[1] > 0.f ? __expf(s[0] - M) * inv : 0.f;
+          ldv<8>(po + q * H * K, b[i]);
+        }
+      }
+#pragma unroll
+      for (int i = 0; i < 8; ++i)
+        if (w[i] > 0.f) {                     // not an empty partition
+#pragma unroll
+          for (int j = 0; j < 8; ++j) a[j] += w[i] * b[i][j];
+        }
+    }
+    stv<8>(&sum[wid][lane * 8], a);
+    __syncthreads();
+    if (wid == 0 && d0 + lane * 8 < K) {
+#pragma unroll
+      for (int w = 1; w < NT / WAVE; ++w)
+#pragma unroll
+        for (int j = 0; j < 8; ++j) a[j] += sum[w][lane * 8 + j];
+      *reinterpret_cast<u16x8*>(o + ((int64_t)r * H + h) * K + d) = pack8(a);
+    }
+    __syncthreads();
+  }
+}
+
 // ---------------------------------------------------------------------- out
 
 // out[r, h E + e] = gate * sum_k uv[h E + e, k] o'[r, h, k]. A workgroup has
-// RT tiles of 16 rows of one head; o' (merged from its partitions) waits in
-// LDS, the waves split the value dimensions.
+// RT tiles of 16 rows of one head; o' waits in LDS, the waves split the
+// value dimensions.
 template <int RT>
 __global__ __launch_bounds__(NT) void latent_out_kernel(
     uint16_t* __restrict__ out, int64_t out_stride,
-    const uint16_t* __restrict__ o, const float* __restrict__ part_o,
-    const float* __restrict__ ml, const uint16_t* __restrict__ uv,
+    const uint16_t* __restrict__ o, const uint16_t* __restrict__ uv,
     const uint16_t* __restrict__ gate, int64_t gate_stride, int R, int H,
-    int E, int K, int parts, int vec) {
+    int E, int K, int vec) {
   extern __shared__ __attribute__((aligned(16))) uint16_t ol[];
-  const int pitch = ((K + 31) & ~31) + 8;
+  const int pitch = ((K + 31) & ~31) + 8, per = (pitch - 8) / 8;
   const int h = blockIdx.y, r0 = blockIdx.x * RT * 16;
   const int wid = threadIdx.x / WAVE, lane = threadIdx.x & (WAVE - 1);
   const int lo = lane & 15, hi = lane >> 4;
   const u16x8 zero = {0, 0, 0, 0, 0, 0, 0, 0};
-  for (int i = wid; i < RT * 16; i += NT / WAVE) {
-    const int r = r0 + i;
-    float M = NEG, L = 0.f;
-    const float* st = nullptr;
-    if (o == nullptr && r < R) {
-      st = ml + ((int64_t)r * parts * H + h) * 2;
-      for (int p = lane; p < parts; p += WAVE)
-        M = fmaxf(M, st[(int64_t)p * H * 2]);
-      M = wave_reduce_max(M);
-      for (int p = lane; p < parts; p += WAVE)
-        L += st[(int64_t)p * H * 2 + 1] * __expf(st[(int64_t)p * H * 2] - M);
-      L = 1.f / wave_reduce_sum(L);
-    }
-    for (int d = lane * 8; d < pitch - 8; d += WAVE * 8) {
-      u16x8 v = zero;
-      if (r < R && d < K) {
-        if (o != nullptr) {
-          v = ld_u16x8(o + ((int64_t)r * H + h) * K + d);
-        } else {
-          float a[8] = {0, 0, 0, 0, 0, 0, 0, 0};
-          const float* po = part_o + ((int64_t)r * parts * H + h) * K + d;
-          for (int p = 0; p < parts; p += 8) {
-            float b[8][8], w[8];
-#pragma unroll
-            for (int i = 0; i < 8; ++i) {
-              const int64_t q = min(p + i, parts - 1);
-              const float* s = st + q * H * 2;
-              w[i] = p + i < parts && s[1] > 0.f ? __expf(s[0] - M) * L : 0.f;
-              ldv<8>(po + q * H * K, b[i]);
-            }
-#pragma unroll
-            for (int i = 0; i < 8; ++i)
-              if (w[i] > 0.f) {               // not an empty partition
-#pragma unroll
-                for (int j = 0; j < 8; ++j) a[j] += w[i] * b[i][j];
-              }
-          }
-          v = pack8(a);
-        }
-      }
-      *reinterpret_cast<u16x8*>(ol + i * pitch + d) = v;
-    }
+  for (int i = threadIdx.x; i < RT * 16 * per; i += NT) {
+    const int t = i / per, d = i % per * 8;
+    const u16x8 v = ld_u16x8(o + ((int64_t)min(r0 + t, R - 1) * H + h) * K +
+                             min(d, K - 8));
+    *reinterpret_cast<u16x8*>(ol + t * pitch + d) = d < K ? v : zero;
   }
   __syncthreads();
   for (int e0 = (blockIdx.z * 4 + wid) * 16; e0 < E;
@@ -871,15 +888,30 @@ void latent_rows_plain(torch::Tensor o, torch::Tensor q, torch::Tensor cache,
                        (const float*)cache.data_ptr(), m);
 }
 
-void latent_out(torch::Tensor out, OptT o, OptT part, OptT ml,
-                torch::Tensor uv, OptT gate) {
+void latent_merge(torch::Tensor o, torch::Tensor part, torch::Tensor ml) {
+  TORCH_CHECK(part.dim() == 4 && part.is_contiguous() &&
+              part.scalar_type() == torch::kFloat32);
+  const int R = part.size(0), parts = part.size(1), H = part.size(2);
+  const int K = part.size(3);
+  TORCH_CHECK(o.is_contiguous() && is_bf16(o) &&
+              o.numel() == (int64_t)R * H * K && K % 8 == 0);
+  TORCH_CHECK(ml.is_contiguous() && ml.scalar_type() == torch::kFloat32 &&
+              ml.numel() == (int64_t)R * parts * H * 2);
+  if (R == 0) return;
+  hipLaunchKernelGGL(latent_merge_kernel, dim3(R, H), dim3(NT), 0,
+                     at::hip::getCurrentHIPStream(), (uint16_t*)o.data_ptr(),
+                     part.data_ptr<float>(), ml.data_ptr<float>(), H, K,
+                     parts);
+}
+
+void latent_out(torch::Tensor out, torch::Tensor o, torch::Tensor uv,
+                OptT gate) {
   check_type(out);
-  TORCH_CHECK(o.has_value() != part.has_value());
-  const torch::Tensor& src = o.has_value() ? *o : *part;
-  const int R = src.size(0), H = src.size(-2), K = src.size(-1);
-  const int parts = o.has_value() ? 1 : src.size(1);
-  TORCH_CHECK(src.is_contiguous() && uv.dim() == 2 && uv.is_contiguous() &&
-              uv.size(1) == K && uv.size(0) % H == 0 && K % 8 == 0);
+  TORCH_CHECK(o.dim() == 3 && o.is_contiguous() &&
+              o.scalar_type() == out.scalar_type());
+  const int R = o.size(0), H = o.size(1), K = o.size(2);
+  TORCH_CHECK(uv.dim() == 2 && uv.is_contiguous() && uv.size(1) == K &&
+              uv.size(0) % H == 0 && K % 8 == 0);
   const int E = uv.size(0) / H;
   TORCH_CHECK(out.size(0) == R && out.size(1) == H * E && out.stride(1) == 1);
   TORCH_CHECK(uv.scalar_type() == out.scalar_type());
@@ -893,45 +925,31 @@ void latent_out(torch::Tensor out, OptT o, OptT part, OptT ml,
   if (R == 0) return;
   auto stream = at::hip::getCurrentHIPStream();
   if (!is_bf16(out)) {
-    TORCH_CHECK(o.has_value() && o->scalar_type() == out.scalar_type());
     hipLaunchKernelGGL((latent_out_plain_kernel<float>), dim3(R, H), dim3(NT),
                        0, stream, (float*)out.data_ptr(), out.stride(0),
-                       (const float*)o->data_ptr(),
+                       (const float*)o.data_ptr(),
                        (const float*)uv.data_ptr(),
                        gate.has_value() ? (const float*)gate->data_ptr()
                                         : nullptr,
                        gs, H, E, K);
     return;
   }
-  if (part.has_value()) {
-    TORCH_CHECK(ml.has_value() && ml->is_contiguous() &&
-                ml->numel() == (int64_t)R * parts * H * 2 &&
-                ml->scalar_type() == torch::kFloat32 &&
-                part->scalar_type() == torch::kFloat32);
-  } else {
-    TORCH_CHECK(is_bf16(*o));
-  }
   const int pitch = ((K + 31) & ~31) + 8;
   const int vec = E % 4 == 0 && out.stride(0) % 4 == 0 &&
                   (uintptr_t)out.data_ptr() % 8 == 0;
-  // few rows: more workgroups, unless each would merge partitions again
-  const int tiles = cdiv(R, 16) * H;
-  const int zs = std::min(cdiv(E, 64), parts > 1 ? std::max(1, 128 / tiles)
-                                                 : (R <= 64 ? 8 : 1));
+  const int zs = std::min(cdiv(E, 64), R <= 64 ? 8 : 1);
 #define HELIX_OUT(RT)                                                        \
   hipLaunchKernelGGL((latent_out_kernel<RT>), dim3(cdiv(R, RT * 16), H, zs), \
                      dim3(NT), RT * 16 * pitch * 2, stream,                  \
                      (uint16_t*)out.data_ptr(), out.stride(0),               \
-                     o.has_value() ? (const uint16_t*)o->data_ptr()          \
-                                   : nullptr,                                \
-                     part.has_value() ? part->data_ptr<float>() : nullptr,   \
-                     ml.has_value() ? ml->data_ptr<float>() : nullptr,       \
+                     (const uint16_t*)o.data_ptr(),                          \
                      (const uint16_t*)uv.data_ptr(),                         \
                      gate.has_value() ? (const uint16_t*)gate->data_ptr()    \
                                       : nullptr,                             \
-                     gs, R, H, E, K, parts, vec)
-  if (R > 16 && K <= 512 && parts == 1) HELIX_OUT(2);
-  else {
+                     gs, R, H, E, K, vec)
+  if (R > 16 && K <= 512) {
+    HELIX_OUT(2);
+  } else {
     TORCH_CHECK(K <= 1536, "latent size ", K);
     HELIX_OUT(1);
   }

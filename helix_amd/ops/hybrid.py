@@ -161,16 +161,14 @@ def latent_attn_rows(out: torch.Tensor, z: torch.Tensor, p: LatentParams,
     q = torch.empty(R, H, p.row, dtype=z.dtype, device=dev)
     C.latent_absorb(q, z, p.q_at, p.head_cols, p.dim_pad, uk, ukt,
                     p.rank_pad)
+    o = torch.empty(R, H, p.rank_pad, dtype=z.dtype, device=dev)
+    parts = latent_parts(R, H, p.max_keys(max_len))
     if not C.latent_rows_fits(q, p.rank_pad):
-        o = torch.empty(R, H, p.rank_pad, dtype=z.dtype, device=dev)
         C.latent_rows_plain(o, q, cache, block_tables, row_seq, row_len,
                             p.scale, p.window)
-        C.latent_out(out, o, None, None, uv, gate)
-        return
-    parts = latent_parts(R, H, p.max_keys(max_len))
-    o = part = ml = None
-    if parts == 1:
-        o = torch.empty(R, H, p.rank_pad, dtype=z.dtype, device=dev)
+    elif parts == 1:
+        C.latent_rows(o, None, None, q, cache, block_tables, row_seq,
+                      row_len, p.rank_pad, p.scale, p.window)
     else:
         need = latent_scratch_floats(R, p, max_len)
         if workspace is None or workspace.numel() < need:
@@ -178,9 +176,10 @@ def latent_attn_rows(out: torch.Tensor, z: torch.Tensor, p: LatentParams,
         n = R * parts * H
         part = workspace[:n * p.rank_pad].view(R, parts, H, p.rank_pad)
         ml = workspace[n * p.rank_pad:need].view(R, parts, H, 2)
-    C.latent_rows(o, part, ml, q, cache, block_tables, row_seq, row_len,
-                  p.rank_pad, p.scale, p.window)
-    C.latent_out(out, o, part, ml, uv, gate)
+        C.latent_rows(None, part, ml, q, cache, block_tables, row_seq,
+                      row_len, p.rank_pad, p.scale, p.window)
+        C.latent_merge(o, part, ml)
+    C.latent_out(out, o, uv, gate)
 
 
 # Prompt portions up to this many rows per sequence run as single rows: they

@@ -112,6 +112,7 @@ def estimate_model_bytes(spec: ModelSpec, block_size: int = 16) -> int:
     else:
         kv = kv_block * spec.max_num_seqs * \
             (spec.max_model_len // block_size + 1)
+    kv += KVCache.state_bytes(cfg.kv_layers(), spec.max_num_seqs)
     return weights + kv + (1 << 30)    # +1 GiB activations/graphs headroom
 
 
