@@ -19,7 +19,7 @@ from helix_amd.engine.sampling_params import SamplingParams
 from helix_amd.models import registry
 from helix_amd.models.meta import (CONTEXT_TAIL, DecodeMeta, MixedMeta,
                                    PrefillMeta, StateLayer)
-from helix_amd.models.latent import LatentAttention, LatentSpec, RotarySpec
+from helix_amd.models.latent import LatentAttention, LatentSpec
 from helix_amd.models.nibezen import (PRESETS, NibezenConfig,
                                       NibezenForCausalLM)
 from helix_amd.models.ssm import Mamba2Mixer, SSMSpec
@@ -261,10 +261,8 @@ def latent_case(case, n, dtype, seed=0):
     return w, m, h
 
 
-def build_latent(case, w, m, dtype, dev, seed_scaling=True):
-    H, D, R, E, K, window, dims = case
-    spec = LatentSpec.from_json(m)
-    mod = LatentAttention(spec, 64, EPS)
+def build_latent(w, m, dtype, dev):
+    mod = LatentAttention(LatentSpec.from_json(m), 64, EPS)
     for name, dst in mod.targets("").items():
         dst.copy_(w[name].float())
     return mod.to(dtype).to(dev)
@@ -299,7 +297,7 @@ def test_latent_attention(dev, dtype, case):
     w, m = cases[0][:2]
     hs = [c[2] for c in cases]
     want = [want_latent(w, m, h) for h in hs]
-    mod = build_latent(case, w, m, dtype, dev)
+    mod = build_latent(w, m, dtype, dev)
     tables, pool = page_tables(n, bs, gen(3))
     kl = mod.spec.cache_layer()
 
@@ -351,7 +349,7 @@ def test_long_rows_in_partitions(dev, dtype, window):
     n, bs = 1203, 16
     w, m, h = latent_case(case, n, dtype, seed=4)
     want = want_latent(w, m, h)
-    mod = build_latent(case, w, m, dtype, dev)
+    mod = build_latent(w, m, dtype, dev)
     tables, pool = page_tables([n], bs, gen(5))
     kl = mod.spec.cache_layer()
     cache = (torch.zeros(pool, *kl.k_shape(bs), dtype=dtype, device=dev),
@@ -514,7 +512,7 @@ def test_rows_without_a_slot_leave_states_alone(dev):
         assert torch.equal(t, k)
 
 
-def test_state_carries_far(dev="cpu"):
+def test_state_carries_far():
     """With slow decays a token from the first chunk still shows at the end:
     the cases above see a state that is lost between chunks."""
     w, m, h = ssm_case(SSM[1], 150, F32)
@@ -805,9 +803,9 @@ def test_greedy_generation(folders, dev, mixed):
     folder, cfg, w = folders["varied"]
     prompts = [prompt(cfg, n, 40 + n) for n in (50, 3, 61)]
     prompts.append(prompts[0][:32] + prompt(cfg, 9, 3))     # shared prefix
-    want = _GREEDY.setdefault("want", None) or [
-        oracle_greedy(cfg, w, p, 14) for p in prompts]
-    _GREEDY["want"] = want
+    if "want" not in _GREEDY:
+        _GREEDY["want"] = [oracle_greedy(cfg, w, p, 14) for p in prompts]
+    want = _GREEDY["want"]
     sp = SamplingParams(temperature=0.0, max_tokens=14, ignore_eos=True)
     for kw in (dict(max_prefill_tokens=4096),
                dict(max_prefill_tokens=24),
