@@ -59,6 +59,17 @@ def iter_safetensors(ckpt_dir: str) -> Iterator[Tuple[str, torch.Tensor]]:
                 yield name, f.get_tensor(name)
 
 
+def tensor_shapes(ckpt_dir: str) -> Dict[str, Tuple[int, ...]]:
+    """Shape of every tensor of a checkpoint folder."""
+    from safetensors import safe_open
+    out = {}
+    for path in sorted(glob.glob(os.path.join(ckpt_dir, "*.safetensors"))):
+        with safe_open(path, framework="pt", device="cpu") as f:
+            for name in f.keys():
+                out[name] = tuple(f.get_slice(name).get_shape())
+    return out
+
+
 # HF Llama checkpoint name -> (our param, role). Roles q/k/v and
 # gate/up are packed into the fused projections.
 def _map_hf_name(name: str):

@@ -23,7 +23,8 @@ from typing import List, Optional, Tuple, Union
 import torch
 import torch.nn as nn
 
-from helix_amd.models.base import Float32Kept, round_up
+from helix_amd.models.base import (Float32Kept, LayerRun, LoopSpec, round_up,
+                                   unroll)
 from helix_amd.models.latent import LatentAttention, LatentSpec, RotarySpec
 from helix_amd.models.llama import HLinear
 from helix_amd.models.ssm import Mamba2Mixer, SSMSpec
@@ -40,20 +41,6 @@ class LayerSpec:
 
 
 @dataclass(frozen=True)
-class LoopSpec:
-    """Layers start .. stop-1 run `times` times in a row."""
-    start: int
-    stop: int
-    times: int
-
-
-@dataclass(frozen=True)
-class LayerRun:
-    layer: int
-    loop_pass: int = -1          # number of the pass that begins here, or -1
-
-
-@dataclass(frozen=True)
 class NibezenConfig:
     name: str
     vocab_size: int
@@ -65,10 +52,8 @@ class NibezenConfig:
     max_position: int = 1 << 20  # nothing in the design bounds it
 
     def __post_init__(self):
-        l = self.loop
-        if l is not None and not (0 <= l.start < l.stop <= len(self.layers)
-                                  and l.times >= 1):
-            raise ValueError(f"loop {l} over {len(self.layers)} layers")
+        if self.loop is not None:
+            self.loop.check(len(self.layers))
 
     @property
     def num_layers(self) -> int:
@@ -76,12 +61,7 @@ class NibezenConfig:
 
     def runs(self) -> List[LayerRun]:
         """The layers in the order they run."""
-        l = self.loop or LoopSpec(0, 0, 0)
-        out = [LayerRun(i) for i in range(l.start)]
-        for t in range(l.times):
-            out += [LayerRun(i, t if i == l.start else -1)
-                    for i in range(l.start, l.stop)]
-        return out + [LayerRun(i) for i in range(l.stop, self.num_layers)]
+        return unroll(self.loop, self.num_layers)
 
     def kv_layers(self, tp_size: int = 1) -> list:
         return [self.layers[r.layer].mixer.cache_layer()

@@ -10,23 +10,29 @@ import json
 import os
 from typing import Callable, Dict, Optional
 
-from helix_amd.models import llama, nibezen, zederax
+from helix_amd.models import llama, motolix, nibezen, zederax
 from helix_amd.models.llama import LlamaConfig, LlamaForCausalLM
+from helix_amd.models.motolix import MotolixConfig, MotolixForCausalLM
 from helix_amd.models.nibezen import NibezenConfig, NibezenForCausalLM
 from helix_amd.models.zederax import ZederaxConfig, ZederaxForCausalLM
 
 MODEL_CLASSES = {LlamaConfig: LlamaForCausalLM,
+                 MotolixConfig: MotolixForCausalLM,
                  NibezenConfig: NibezenForCausalLM,
                  ZederaxConfig: ZederaxForCausalLM}
 
 # config.json architecture -> reader(dict, name) of the configuration
 CONFIG_READERS: Dict[str, Callable] = {
+    "Motolix": MotolixConfig.from_json,
     "Nibezen": NibezenConfig.from_json,
     "Zederax": ZederaxConfig.from_json,
     "LlamaForCausalLM": LlamaConfig.from_json,
     "MistralForCausalLM": LlamaConfig.from_json,
     "Qwen2ForCausalLM": LlamaConfig.from_json,
 }
+
+# designs whose config.json leaves some sizes to the tensors' shapes
+SIZED_BY_TENSORS = {"Motolix"}
 
 
 def is_folder(model: str) -> bool:
@@ -35,7 +41,8 @@ def is_folder(model: str) -> bool:
 
 def get_config(model: str):
     """Configuration of a preset or of a checkpoint folder."""
-    families = (llama.PRESETS, nibezen.PRESETS, zederax.PRESETS)
+    families = (llama.PRESETS, motolix.PRESETS, nibezen.PRESETS,
+                zederax.PRESETS)
     for presets in families:
         if model in presets:
             return presets[model]
@@ -49,7 +56,11 @@ def get_config(model: str):
     if arch not in CONFIG_READERS:
         raise ValueError(f"{model}: unknown architecture {arch!r}")
     name = os.path.basename(os.path.normpath(model))
-    return CONFIG_READERS[arch](d, name=name)
+    sizes = {}
+    if arch in SIZED_BY_TENSORS:
+        from helix_amd.engine import weights
+        sizes["shapes"] = weights.tensor_shapes(model)
+    return CONFIG_READERS[arch](d, name=name, **sizes)
 
 
 def model_class(cfg):

@@ -14,7 +14,8 @@ import torch
 
 from . import build
 from . import reference as ref
-from .reference import make_cos_sin_cache, yarn_frequencies  # re-export
+from .reference import (banded_frequencies, make_cos_sin_cache,  # re-export
+                        yarn_frequencies)
 
 _C = None
 _C_ERR: str | None = None

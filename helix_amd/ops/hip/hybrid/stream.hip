@@ -4,9 +4,7 @@
 //   x_out <- v;  h = v / sqrt(mean(v^2) + eps) * w
 //
 // One workgroup per token; the row stays in registers between sum and norm.
-#include "tile.h"
-#include <torch/extension.h>
-#include <ATen/hip/HIPContext.h>
+#include "../glu.h"
 
 using namespace helix;
 using OptT = c10::optional<torch::Tensor>;
@@ -149,48 +147,6 @@ void launch_residual(torch::Tensor h, OptT y, OptT embed, Stream s, int T) {
 #undef HELIX_RES
 }
 
-// ---------------------------------------------------------------- silu * up
-
-template <typename S, int N>
-__global__ void silu_mul_kernel(S* __restrict__ out, const S* __restrict__ z,
-                                int64_t z_stride, int up_at, int F,
-                                int64_t total) {
-  const int64_t i = ((int64_t)blockIdx.x * blockDim.x + threadIdx.x);
-  if (i >= total) return;
-  const int nv = F / N;
-  const int64_t t = i / nv;
-  const int d = (int)(i - t * nv) * N;
-  const S* zr = z + t * z_stride;
-  if constexpr (N == 1) {
-    st1(out + t * F + d, silu_s<S>(ld1(zr + d)) * ld1(zr + up_at + d));
-  } else {
-    float g[N], u[N];
-    ldv<N>(zr + d, g);
-    ldv<N>(zr + up_at + d, u);
-#pragma unroll
-    for (int j = 0; j < N; ++j) g[j] = silu_s<S>(g[j]) * u[j];
-    stv<N>(out + t * F + d, g);
-  }
-}
-
-template <typename S>
-void launch_silu(torch::Tensor out, torch::Tensor z, int up_at) {
-  const int64_t T = out.size(0);
-  const int F = out.size(1);
-  auto stream = at::hip::getCurrentHIPStream();
-  const bool vec = F % 8 == 0 && up_at % 8 == 0 && z.stride(0) % 8 == 0;
-  const int64_t total = T * F / (vec ? 8 : 1);
-  const dim3 grid((total + 255) / 256);
-  if (vec)
-    hipLaunchKernelGGL((silu_mul_kernel<S, 8>), grid, dim3(256), 0, stream,
-                       (S*)out.data_ptr(), (const S*)z.data_ptr(),
-                       z.stride(0), up_at, F, total);
-  else
-    hipLaunchKernelGGL((silu_mul_kernel<S, 1>), grid, dim3(256), 0, stream,
-                       (S*)out.data_ptr(), (const S*)z.data_ptr(),
-                       z.stride(0), up_at, F, total);
-}
-
 // ------------------------------------------------------------- grouped norm
 
 // One workgroup per (row, group); NV vectors of 8 per thread.
@@ -326,15 +282,7 @@ void residual_norm(torch::Tensor h, OptT x, OptT y, OptT ls, double mult,
 }
 
 void silu_mul(torch::Tensor out, torch::Tensor z, int64_t up_at) {
-  TORCH_CHECK(out.is_contiguous() && supported(out) && z.stride(1) == 1);
-  TORCH_CHECK(z.scalar_type() == out.scalar_type() &&
-              z.size(0) == out.size(0));
-  TORCH_CHECK(out.size(1) <= up_at && up_at + out.size(1) <= z.size(1));
-  if (out.numel() == 0) return;
-  if (z.scalar_type() == torch::kBFloat16)
-    launch_silu<uint16_t>(out, z, up_at);
-  else
-    launch_silu<float>(out, z, up_at);
+  launch_glu<Silu>(out, z, up_at);
 }
 
 void group_rms_norm(torch::Tensor out, torch::Tensor y, int64_t groups,

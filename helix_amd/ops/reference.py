@@ -112,6 +112,27 @@ def yarn_frequencies(dims: int, base: float,
             0.1 * math.log(factor) + 1.0)
 
 
+def banded_frequencies(dims: int, base: float,
+                       scaling: dict | None = None) -> torch.Tensor:
+    """float64 frequency of each of the dims/2 pairs. With scaling (factor,
+    low, high, original), pairs that turn less than `low` times over the
+    original context are slowed down by factor, those that turn more than
+    `high` times are left alone, with a blend by the number of turns
+    between."""
+    import math
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    freq = float(base) ** (-2.0 * i / dims)
+    if not scaling:
+        return freq
+    low, high = float(scaling["low"]), float(scaling["high"])
+    slow = freq / float(scaling["factor"])
+    turns = float(scaling["original"]) * freq / (2 * math.pi)
+    s = (turns - low) / (high - low) if high != low else torch.zeros_like(i)
+    mid = (1 - s) * slow + s * freq
+    return torch.where(turns < low, slow,
+                       torch.where(turns > high, freq, mid))
+
+
 def silu_and_mul(x: torch.Tensor) -> torch.Tensor:
     i = x.shape[-1] // 2
     g, u = x[..., :i].float(), x[..., i:].float()
