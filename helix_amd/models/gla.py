@@ -16,7 +16,6 @@ from dataclasses import dataclass
 import torch
 import torch.nn as nn
 
-from helix_amd.engine.weights import Placement
 from helix_amd.models.base import Float32Kept, round_up
 from helix_amd.models.meta import MixedMeta, StateLayer
 from helix_amd.ops import gated
@@ -63,7 +62,7 @@ class GLASpec:
 class GatedLinearAttention(Float32Kept):
     """Everything between the fused projections; at: first column of each
     input in the fused projection."""
-    kept = ("a2", "a2_b", "norm_w")
+    kept = ("a2_b", "norm_w")
 
     def __init__(self, spec: GLASpec, at: dict, eps: float,
                  out_scale: float = 1.0):
@@ -73,7 +72,7 @@ class GatedLinearAttention(Float32Kept):
         self.params = gated.GLAParams(
             spec.heads, spec.dim, spec.vdim, spec.rank, at["q"], at["k"],
             at["v"], at["g"], at["a1"], spec.tau, eps, out_scale)
-        self.a2 = nn.Parameter(torch.zeros(spec.rank, n))
+        self.a2 = nn.Parameter(torch.zeros(n, round_up(spec.rank, 32)))
         self.a2_b = nn.Parameter(torch.zeros(n))
         self.norm_w = nn.Parameter(torch.ones(spec.vdim))
 
@@ -100,8 +99,7 @@ class GatedLinearAttention(Float32Kept):
     def targets(self, prefix: str) -> dict:
         s = self.spec
         return {
-            prefix + "a2": Placement((s.heads * s.dim, s.rank), [
-                (self.a2.data, lambda t: t.t())]),
+            prefix + "a2": self.a2.data[:, :s.rank],
             prefix + "a2.b": self.a2_b.data,
             prefix + "norm": self.norm_w.data,
         }

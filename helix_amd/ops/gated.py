@@ -258,7 +258,8 @@ class GLAParams:
 
 @dataclass
 class GLAWeights:
-    """fp32: a2 [rank, heads * dim] (transposed), a2_b, norm [vdim]."""
+    """a2 [heads * dim, rank padded to 32] in the storage type; fp32: a2_b,
+    norm [vdim]."""
     a2: torch.Tensor
     a2_b: torch.Tensor
     norm: torch.Tensor
@@ -270,7 +271,8 @@ GLA_CHUNK = 64
 
 def _gla_step(y, z, p: GLAParams, w: GLAWeights, state, slots, positions,
               cu=None):
-    _native().gla_step(y, z, *p.columns, p.vdim, w.a2, w.a2_b, w.norm, p.tau,
+    _native().gla_step(y, z, *p.columns, p.vdim, p.rank, w.a2, w.a2_b, w.norm,
+                       p.tau,
                        p.q_scale, p.out_scale, p.eps, state, slots,
                        positions, cu)
 
@@ -324,8 +326,8 @@ def gla_chunk_steps(y, z, p: GLAParams, w: GLAWeights, state, meta):
 
     def operands():
         C.gla_operands(qe, ke, am, vt, ec, z, p.q_at, p.k_at, p.v_at, p.a_at,
-                       p.dim, p.vdim, w.a2, w.a2_b, p.tau, p.q_scale, ch.row,
-                       ch.count)
+                       p.dim, p.vdim, p.rank, w.a2, w.a2_b, p.tau, p.q_scale,
+                       ch.row, ch.count)
 
     def recurrence():
         C.gla_chunks(o, qe, ke, am, vt, ec, p.vdim, state, meta.state_slots,

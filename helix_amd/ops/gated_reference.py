@@ -114,7 +114,7 @@ def gla_span(y, z, p, w, state, slot, start):
         row = z[t].float()
         q, k = (row[at:at + H * D].view(H, D) for at in (p.q_at, p.k_at))
         v, g = (row[at:at + H * E].view(H, E) for at in (p.v_at, p.g_at))
-        a = row[p.a_at:p.a_at + p.rank] @ w.a2 + w.a2_b
+        a = w.a2[:, :p.rank].float() @ row[p.a_at:p.a_at + p.rank] + w.a2_b
         a = torch.exp(F.logsigmoid(a) / p.tau).view(H, D)
         keep = a[:, :, None] * keep + k[:, :, None] * v[:, None, :]
         o = (keep * (q * p.q_scale)[:, :, None]).sum(1)

@@ -30,14 +30,14 @@ void attn_prompt(T out, T q, T kc, T vc, T bt, T cu, T seq_lens,
                  int64_t max_q, double scale, double out_scale, bool sigmoid,
                  OptT temp, OptT bias, OptT vcs);
 void gla_step(T y, T z, int64_t q_at, int64_t k_at, int64_t v_at,
-              int64_t g_at, int64_t a_at, int64_t vdim, T a2, T a2_b, T norm,
-              double tau, double q_scale, double out_scale, double eps,
+              int64_t g_at, int64_t a_at, int64_t vdim, int64_t rank, T a2,
+              T a2_b, T norm, double tau, double q_scale, double out_scale, double eps,
               T state, T slots, T pos, OptT cu);
 bool gla_chunks_fit(T z, int64_t dim);
 void gla_operands(T qe, T ke, T am, T vt, T ec, T z, int64_t q_at,
                   int64_t k_at, int64_t v_at, int64_t a_at, int64_t dim,
-                  int64_t vdim, T a2, T a2_b, double tau, double q_scale,
-                  T row, T count);
+                  int64_t vdim, int64_t rank, T a2, T a2_b, double tau,
+                  double q_scale, T row, T count);
 void gla_chunks(T o, T qe, T ke, T am, T vt, T ec, int64_t vdim, T state,
                 T slots, T pos, T cu, T first);
 void head_norm_gate(T y, T o, T g, T w, double scale, double eps);

@@ -42,7 +42,14 @@ struct Epilogue {
 
 template <typename S, int N>
 __device__ __forceinline__ void get(const S* p, float* v) {
-  if constexpr (N == 1) v[0] = ld1(p); else ldv<N>(p, v);
+  if constexpr (N == 1) {
+    v[0] = ld1(p);
+  } else if constexpr (N == 2) {
+    v[0] = ld1(p);
+    v[1] = ld1(p + 1);
+  } else {
+    ldv<N>(p, v);
+  }
 }
 template <typename S, int N>
 __device__ __forceinline__ void put(S* p, const float* v) {
@@ -64,95 +71,131 @@ __device__ __forceinline__ float row_inv(const S* z, int n, float eps,
   return inv;
 }
 
-// Heads of [D] from z (norm inv and w apply if w is given), turned and
-// handed to store(head, dim, values).
+// Unit u of head h of one row z [heads][D]: N pairs of the turned part, or N
+// dimensions of the rest. store(dim, values) takes the results.
 template <typename S, int N, class Store>
-__device__ __forceinline__ void turn_heads(const S* z, int heads, int D,
-                                           const float2* cs, int n,
-                                           float inv, const float* w,
-                                           Store store) {
-  // units: N pairs of the turned part, N dimensions of the rest
-  const int pu = n / N, units = pu + (D - 2 * n) / N;
-  for (int i = threadIdx.x; i < heads * units; i += NT) {
-    const int h = i / units, u = i % units;
-    const int d = u < pu ? u * N : 2 * n + (u - pu) * N;
-    const int at = h * D + d;
-    float a[N], b[N];
-    get<S, N>(z + at, a);
+__device__ __forceinline__ void turn_unit(const S* z, int h, int u, int D,
+                                          const float2* cs, int n, float inv,
+                                          const float* w, Store store) {
+  const int pu = n / N;
+  const int d = u < pu ? u * N : 2 * n + (u - pu) * N;
+  const int at = h * D + d;
+  float a[N], b[N];
+  get<S, N>(z + at, a);
+  if (w != nullptr) {
+    float g[N];
+    get<float, N>(w + at, g);
+#pragma unroll
+    for (int j = 0; j < N; ++j) a[j] *= inv * g[j];
+  }
+  if (u < pu) {
+    get<S, N>(z + at + n, b);
     if (w != nullptr) {
       float g[N];
-      get<float, N>(w + at, g);
+      get<float, N>(w + at + n, g);
 #pragma unroll
-      for (int j = 0; j < N; ++j) a[j] *= inv * g[j];
+      for (int j = 0; j < N; ++j) b[j] *= inv * g[j];
     }
-    if (u < pu) {
-      get<S, N>(z + at + n, b);
-      if (w != nullptr) {
-        float g[N];
-        get<float, N>(w + at + n, g);
+    float r[2 * N];
+    get<float, 2 * N>((const float*)(cs + d), r);
 #pragma unroll
-        for (int j = 0; j < N; ++j) b[j] *= inv * g[j];
-      }
-#pragma unroll
-      for (int j = 0; j < N; ++j) {
-        const float2 r = cs[d + j];
-        const float p = a[j] * r.x - b[j] * r.y;
-        b[j] = b[j] * r.x + a[j] * r.y;
-        a[j] = p;
-      }
-      store(h, d + n, b);
+    for (int j = 0; j < N; ++j) {
+      const float p = a[j] * r[2 * j] - b[j] * r[2 * j + 1];
+      b[j] = b[j] * r[2 * j] + a[j] * r[2 * j + 1];
+      a[j] = p;
     }
-    store(h, d, a);
+    store(d + n, b);
   }
+  store(d, a);
 }
 
+// Units of a head: the turned pairs, then the rest.
+__device__ __forceinline__ int units_of(int D, int n, int N) {
+  return n / N + (D - 2 * n) / N;
+}
+
+constexpr int PER = 16;                       // tokens of a workgroup at most
+
 // The first T workgroups have a token's queries each, the others keys and
-// values of `per` tokens, so that a page's values are written together.
+// values of `per` neighbouring tokens. Values go out token by token of one
+// dimension, so that a page's 16-byte runs are written at once.
 template <typename S, int N>
 __global__ __launch_bounds__(NT) void attn_epilogue_kernel(
     S* __restrict__ q, S* __restrict__ kc, S* __restrict__ vc,
     const S* __restrict__ z, Epilogue m) {
-  __shared__ float red[16];
+  __shared__ float red[16], invs[PER];
+  __shared__ int64_t slots[PER];
+  const int pad = m.Dp - m.D;
   if (blockIdx.x < m.T) {
     const int64_t t = blockIdx.x;
     const S* zq = z + t * m.z_stride + m.q_at;
     float inv = 1.f;
     if (m.qw != nullptr) inv = row_inv<S, N>(zq, m.H * m.D, m.eps, red);
     S* qt = q + t * m.H * m.Dp;
-    turn_heads<S, N>(zq, m.H, m.D, m.cs + t * m.nk, m.nk, inv, m.qw,
-                     [&](int h, int d, const float* v) {
-                       put<S, N>(qt + h * m.Dp + d, v);
-                     });
-    const int pad = m.Dp - m.D;
+    const int units = units_of(m.D, m.nk, N);
+    for (int i = threadIdx.x; i < m.H * units; i += NT) {
+      const int h = i / units;
+      turn_unit<S, N>(zq, h, i - h * units, m.D, m.cs + t * m.nk, m.nk, inv,
+                      m.qw, [&](int d, const float* v) {
+                        put<S, N>(qt + h * m.Dp + d, v);
+                      });
+    }
     for (int i = threadIdx.x; i < m.H * pad; i += NT)
       st1(qt + i / pad * m.Dp + m.D + i % pad, 0.f);
     return;
   }
-  const int64_t first = (blockIdx.x - m.T) * m.per;
-  for (int64_t t = first; t < min(first + m.per, m.T); ++t) {
-    const int64_t slot = m.slots[t];
-    if (slot < 0) continue;                   // the same for all threads
-    const int64_t page = slot / m.bs;
-    const int at = (int)(slot % m.bs);
-    const S* zk = z + t * m.z_stride + m.k_at;
-    float inv = 1.f;
-    if (m.kw != nullptr) inv = row_inv<S, N>(zk, m.G * m.D, m.eps, red);
-    S* kt = kc + (page * m.G * m.bs + at) * m.Dp;
-    turn_heads<S, N>(zk, m.G, m.D, m.cs + t * m.nk, m.nk, inv, m.kw,
-                     [&](int g, int d, const float* v) {
-                       put<S, N>(kt + (int64_t)g * m.bs * m.Dp + d, v);
-                     });
-    const int pad = m.Dp - m.D;
-    for (int i = threadIdx.x; i < m.G * pad; i += NT)
-      st1(kt + (int64_t)(i / pad) * m.bs * m.Dp + m.D + i % pad, 0.f);
-    S* vt = vc + page * m.G * m.E * m.bs + at;
-    turn_heads<S, N>(z + t * m.z_stride + m.v_at, m.G, m.E,
-                     m.vcs + t * m.nv, m.nv, 1.f, nullptr,
-                     [&](int g, int d, const float* v) {
+  const int64_t t0 = (blockIdx.x - m.T) * m.per;
+  const int nt = (int)min((int64_t)m.per, m.T - t0);
+  if ((int)threadIdx.x < nt) slots[threadIdx.x] = m.slots[t0 + threadIdx.x];
+  if (m.kw != nullptr) {
+    const int lane = threadIdx.x & (WAVE - 1), n = m.G * m.D;
+    for (int t = threadIdx.x / WAVE; t < nt; t += NT / WAVE) {
+      const S* zk = z + (t0 + t) * m.z_stride + m.k_at;
+      float ss = 0.f;
+      for (int i = lane * N; i < n; i += WAVE * N) {
+        float v[N];
+        get<S, N>(zk + i, v);
 #pragma unroll
-                       for (int j = 0; j < N; ++j)
-                         st1(vt + ((int64_t)g * m.E + d + j) * m.bs, v[j]);
-                     });
+        for (int j = 0; j < N; ++j) ss += v[j] * v[j];
+      }
+      ss = wave_reduce_sum(ss);
+      if (lane == 0) invs[t] = 1.f / sqrtf(ss / n + m.eps);
+    }
+  }
+  __syncthreads();
+  {
+    const int units = units_of(m.D, m.nk, N), all = m.G * units;
+    for (int i = threadIdx.x; i < nt * all; i += NT) {
+      const int t = i / all, g = (i - t * all) / units;
+      const int64_t slot = slots[t];
+      if (slot < 0) continue;
+      S* kt = kc + ((slot / m.bs * m.G + g) * m.bs + slot % m.bs) * m.Dp;
+      turn_unit<S, N>(z + (t0 + t) * m.z_stride + m.k_at, g,
+                      i - t * all - g * units, m.D, m.cs + (t0 + t) * m.nk,
+                      m.nk, m.kw != nullptr ? invs[t] : 1.f, m.kw,
+                      [&](int d, const float* v) { put<S, N>(kt + d, v); });
+    }
+    for (int i = threadIdx.x; i < nt * m.G * pad; i += NT) {
+      const int t = i / (m.G * pad), g = i / pad % m.G;
+      const int64_t slot = slots[t];
+      if (slot >= 0)
+        st1(kc + ((slot / m.bs * m.G + g) * m.bs + slot % m.bs) * m.Dp +
+                m.D + i % pad, 0.f);
+    }
+  }
+  const int units = units_of(m.E, m.nv, N);
+  for (int i = threadIdx.x; i < nt * m.G * units; i += NT) {
+    const int t = i % nt, u = i / nt, g = u / units;
+    const int64_t slot = slots[t];
+    if (slot < 0) continue;
+    S* vt = vc + (slot / m.bs * m.G + g) * m.E * m.bs + slot % m.bs;
+    turn_unit<S, N>(z + (t0 + t) * m.z_stride + m.v_at, g, u - g * units,
+                    m.E, m.vcs + (t0 + t) * m.nv, m.nv, 1.f, nullptr,
+                    [&](int d, const float* v) {
+#pragma unroll
+                      for (int j = 0; j < N; ++j)
+                        st1(vt + (int64_t)(d + j) * m.bs, v[j]);
+                    });
   }
 }
 
@@ -241,7 +284,7 @@ void attn_epilogue(torch::Tensor q, torch::Tensor kc, torch::Tensor vc,
   m.v_at = v_at;
   m.eps = (float)eps;
   if (m.T == 0) return;
-  m.per = m.T > 1024 ? m.bs : 1;
+  m.per = m.T > 1024 ? PER : 1;
   if (z.scalar_type() == torch::kBFloat16) launch<uint16_t>(q, kc, vc, z, m);
   else if (z.scalar_type() == torch::kFloat32) launch<float>(q, kc, vc, z, m);
   else TORCH_CHECK(false, "attention epilogue: bf16 or fp32");

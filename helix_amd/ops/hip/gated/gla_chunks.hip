@@ -7,10 +7,11 @@
 //   A_ij = sum_d q_i[d] k_j[d] e^(c_i[d] - c_j[d])
 //   S  <- diag(e^(c_63)) S + sum_j (k_j e^(c_63 - c_j)) v_j^T
 //
-// gla_operands makes a chunk's operands. No exponent there is ever positive,
-// however fast a channel decays: A's blocks of 16 x 16 off the diagonal take
-// the start of the later block as reference, those on it multiply keys by
-// one decay after another in fp32. gla_chunks carries a head's state from
+// gla_operands makes a chunk's operands. No power there overflows,
+// however fast a channel decays: A's blocks of 16 x 16 take the start of the
+// later block as reference. On the diagonal keys then have positive ones;
+// where a channel decays by more than 2^-100 in 16 tokens, that block is
+// summed pair by pair in fp32. gla_chunks carries a head's state from
 // chunk to chunk in fp32 registers. v enters the products as the bf16 it is,
 // whatever has a decay or the state in it as two bf16 terms (17 bits).
 //
@@ -31,14 +32,15 @@ constexpr int LP = L + 8;
 constexpr int SL = 32;                        // channels worked on at a time
 constexpr int PV = 36;                        // pitch, rows read as vectors
 constexpr int PS = 33;                        // pitch, columns read
-constexpr int PA = 68;
+constexpr float LOG2E_ = 1.4426950408889634f;
 
 struct Operands {
-  const float *a2, *a2_b;      // [rank, H * D], [H * D]
+  const uint16_t* a2;          // [H * D, rank_pad]
+  const float* a2_b;           // [H * D]
   const int *row, *count;      // per chunk
   int64_t z_stride;
-  int q_at, k_at, v_at, a_at, H, D, Dp, E, Pp, rank, vec;
-  float inv_tau, q_scale;
+  int q_at, k_at, v_at, a_at, H, D, Dp, E, Pp, rank, rank_pad, vec;
+  float unit, q_scale;         // unit: 1 / tau
 };
 
 // Columns c0 .. c0 + 31 of the chunk's rows, 8 per thread; nothing past
@@ -60,19 +62,29 @@ __device__ __forceinline__ void load_slice(float* v, const uint16_t* z,
   }
 }
 
-// grid (chunks, heads)
+__device__ __forceinline__ float exp2_(float x) {
+  return __builtin_amdgcn_exp2f(x);
+}
+
+// log2(1 + 2^x)
+__device__ __forceinline__ float softplus2(float x) {
+  return fmaxf(x, 0.f) +
+         __builtin_amdgcn_logf(1.f + exp2_(-fabsf(x)));
+}
+
+// Most a channel may decay within 16 tokens (as a power of two) for the
+// diagonal blocks to be products.
+constexpr float STEEP = -100.f;
+
+// grid (chunks, heads). Decays are kept as base-2 logarithms.
 __global__ __launch_bounds__(NT) void gla_operands_kernel(
     uint16_t* __restrict__ qe, uint16_t* __restrict__ ke,
     uint16_t* __restrict__ am, uint16_t* __restrict__ vt,
     float* __restrict__ ec, const uint16_t* __restrict__ z, Operands m) {
-  extern __shared__ __attribute__((aligned(16))) float sh[];
-  float* qs = sh;                             // [64][PV] queries
-  float* al = qs + L * PV;                    // [64][PV] decays
-  float* ks = al + L * PV;                    // [64][PS] keys (later values)
-  float* cs = ks + L * PS;                    // [64][PS] log decays, summed
-  float* pre = cs + L * PS;                   // [8][SL]
-  float* a1 = pre + 8 * SL;                   // [64][rank]
-  float* as = sh;                             // [64][PA] in the end
+  __shared__ __attribute__((aligned(16))) float qs[L * PV];
+  __shared__ float ks[L * PS];                // keys (later values)
+  __shared__ float cs[L * PS];                // log decays, summed
+  __shared__ float ends[4][SL];               // of every 16 tokens
   const int n = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   const int wid = tid / WAVE, lane = tid & (WAVE - 1);
   const int lo = lane & 15, hi = lane >> 4;
@@ -81,66 +93,90 @@ __global__ __launch_bounds__(NT) void gla_operands_kernel(
   const int64_t nh = (int64_t)n * m.H + h;
   uint16_t* qo = qe + nh * 2 * L * m.Dp;
   uint16_t* ko = ke + nh * 2 * L * m.Dp;
-
-  for (int i = tid; i < L * m.rank; i += NT) {
-    const int t = i / m.rank, r = i % m.rank;
-    a1[i] = t < count ? bf16_to_f32(zr[t * m.z_stride + m.a_at + r]) : 0.f;
-  }
-
-  floatx4 off[2];                             // blocks wid, wid + 4 of six
-  off[0] = off[1] = floatx4{0, 0, 0, 0};
-  float dg[16];                               // diagonal block wid, column j
+  // the score blocks (I, J <= I) of this wave; heads start elsewhere, so
+  // that the long rows do not all meet on one SIMD
+  const int I = (wid + h) & 3;
+  floatx4 acc[4];
 #pragma unroll
-  for (int i = 0; i < 16; ++i) dg[i] = 0.f;
-  const int j = lane >> 2, dq = (lane & 3) * 8;
+  for (int i = 0; i < 4; ++i) acc[i] = floatx4{0, 0, 0, 0};
 
   for (int d0 = 0; d0 < m.Dp; d0 += SL) {
     float v[8], w[8];
     const int t = tid / 4, s = tid % 4 * 8;
     load_slice(v, zr + m.q_at + h * m.D, m.z_stride, d0, m.D, count, m.vec);
     load_slice(w, zr + m.k_at + h * m.D, m.z_stride, d0, m.D, count, m.vec);
+    // decays: wave w has tokens 16 w .., a lane 4 tokens of two channels
+    floatx4 x[2] = {floatx4{0, 0, 0, 0}, floatx4{0, 0, 0, 0}};
+    const int ta = wid * 16 + lo;
+    for (int r = hi * 8; r < m.rank_pad; r += 32) {
+      u16x8 a = {0, 0, 0, 0, 0, 0, 0, 0};
+      if (ta < count && r < m.rank) {
+        const uint16_t* ap = zr + ta * m.z_stride + m.a_at + r;
+        if (m.vec && r + 8 <= m.rank) {
+          a = ld_u16x8(ap);
+        } else {
+#pragma unroll
+          for (int i = 0; i < 8; ++i)
+            if (r + i < m.rank) a[i] = ap[i];
+        }
+      }
+#pragma unroll
+      for (int u = 0; u < 2; ++u) {
+        const int c = min(d0 + u * 16 + lo, m.D - 1);
+        const u16x8 b =
+            ld_u16x8(m.a2 + (int64_t)(h * m.D + c) * m.rank_pad + r);
+        x[u] = mfma16(a, b, x[u]);
+      }
+    }
+    float part[2];
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      const int c = d0 + u * 16 + lo;
+      const float bias = c < m.D ? m.a2_b[h * m.D + c] : 0.f;
+      float sum = 0.f;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const bool in = c < m.D && wid * 16 + hi * 4 + r < count;
+        // log2(sigmoid(y)^(1/tau)) = -softplus2(-y log2(e)) / tau
+        const float g = -softplus2(-(x[u][r] + bias) * LOG2E_) * m.unit;
+        sum += in ? g : 0.f;
+        x[u][r] = sum;
+      }
+      float up = __shfl_up(sum, 16, WAVE);
+      if (hi >= 1) sum += up;
+      up = __shfl_up(sum, 32, WAVE);
+      if (hi >= 2) sum += up;
+      part[u] = sum - x[u][3];                // of the lanes before
+    }
     __syncthreads();                          // the last slice is done
+#pragma unroll
+    for (int u = 0; u < 2; ++u)
+      if (hi == 3) ends[wid][u * 16 + lo] = part[u] + x[u][3];
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
       v[i] *= m.q_scale;
       ks[t * PS + s + i] = w[i];
     }
     stv<8>(qs + t * PV + s, v);
-    {
-      // decays: a thread has 8 tokens of a channel
-      const int d = tid % SL, tg = tid / SL, c = d0 + d;
-      float x[8], sum = 0.f;
-      const float bias = c < m.D ? m.a2_b[h * m.D + c] : 0.f;
+    __syncthreads();
+    bool steep = false;
 #pragma unroll
-      for (int i = 0; i < 8; ++i) x[i] = bias;
-      if (c < m.D)
-        for (int r = 0; r < m.rank; ++r) {
-          const float wr = m.a2[(int64_t)r * m.H * m.D + h * m.D + c];
+    for (int u = 0; u < 2; ++u) {
+      float base = part[u];
 #pragma unroll
-          for (int i = 0; i < 8; ++i)
-            x[i] += a1[(tg * 8 + i) * m.rank + r] * wr;
-        }
+      for (int i = 0; i < 3; ++i)
+        if (i < wid) base += ends[i][u * 16 + lo];
 #pragma unroll
-      for (int i = 0; i < 8; ++i) {
-        const int tt = tg * 8 + i;
-        const float g = tt < count && c < m.D
-                            ? -softplus(-x[i]) * m.inv_tau : 0.f;
-        sum += g;
-        al[tt * PV + d] = expf(g);
-        x[i] = sum;
-      }
-      pre[tg * SL + d] = sum;
-      __syncthreads();
-      float base = 0.f;
-      for (int i = 0; i < tg; ++i) base += pre[i * SL + d];
-#pragma unroll
-      for (int i = 0; i < 8; ++i) cs[(tg * 8 + i) * PS + d] = base + x[i];
+      for (int r = 0; r < 4; ++r)
+        cs[(wid * 16 + hi * 4 + r) * PS + u * 16 + lo] = base + x[u][r];
+      steep |= ends[I][u * 16 + lo] < STEEP;
     }
+    steep = __any(steep);
     __syncthreads();
     // queries and keys with their decays
     u16x8 a, b;
 #pragma unroll
-    for (int i = 0; i < 8; ++i) v[i] *= expf(cs[t * PS + s + i]);
+    for (int i = 0; i < 8; ++i) v[i] *= exp2_(cs[t * PS + s + i]);
     split8(v, a, b);
     *reinterpret_cast<u16x8*>(qo + t * m.Dp + d0 + s) = a;
     *reinterpret_cast<u16x8*>(qo + (L + t) * m.Dp + d0 + s) = b;
@@ -148,87 +184,64 @@ __global__ __launch_bounds__(NT) void gla_operands_kernel(
     const float end = cs[(L - 1) * PS + kd];
 #pragma unroll
     for (int i = 0; i < 8; ++i)
-      w[i] = ks[(kt + i) * PS + kd] * expf(end - cs[(kt + i) * PS + kd]);
+      w[i] = ks[(kt + i) * PS + kd] * exp2_(end - cs[(kt + i) * PS + kd]);
     split8(w, a, b);
     *reinterpret_cast<u16x8*>(ko + (d0 + kd) * L + kt) = a;
     *reinterpret_cast<u16x8*>(ko + (m.Dp + d0 + kd) * L + kt) = b;
-    if (tid < SL) ec[nh * m.Dp + d0 + tid] = expf(cs[(L - 1) * PS + tid]);
+    if (tid < SL) ec[nh * m.Dp + d0 + tid] = exp2_(cs[(L - 1) * PS + tid]);
 
-    // diagonal block: key j meets queries i >= j, decaying on the way
-    float kk[8];
+    // scores: rows j of a block's result, columns i
+    const int i = I * 16 + lo;
+    float ref[8], q[8];
 #pragma unroll
-    for (int i = 0; i < 8; ++i) kk[i] = ks[(wid * 16 + j) * PS + dq + i];
-#pragma unroll
-    for (int i = 0; i < 16; ++i) {
-      float q[8], g[8], sum = 0.f;
-      ldv<8>(qs + (wid * 16 + i) * PV + dq, q);
-      ldv<8>(al + (wid * 16 + i) * PV + dq, g);
-#pragma unroll
-      for (int c = 0; c < 8; ++c) {
-        kk[c] *= i > j ? g[c] : 1.f;
-        sum += q[c] * kk[c];
-      }
-      dg[i] += i >= j ? sum : 0.f;
+    for (int c = 0; c < 8; ++c) {
+      const int d = hi * 8 + c;
+      ref[c] = I > 0 ? cs[(I * 16 - 1) * PS + d] : 0.f;
+      q[c] = qs[i * PV + d] * exp2_(cs[i * PS + d] - ref[c]);
     }
-    // blocks (I, J), I > J: rows j of the result, columns i
+    u16x8 qh, ql;
+    split8(q, qh, ql);
 #pragma unroll
-    for (int u = 0; u < 2; ++u) {
-      const int blk = wid + u * 4;
-      if (blk >= 6) continue;
-      const int I = blk < 1 ? 1 : (blk < 3 ? 2 : 3);
-      const int J = blk - I * (I - 1) / 2;
-      float q[8], k[8];
+    for (int J = 0; J < 4; ++J) {
+      if (J > I || (J == I && steep)) continue;
+      const int j = J * 16 + lo;
+      float k[8];
 #pragma unroll
-      for (int c = 0; c < 8; ++c) {
-        const int d = hi * 8 + c;
-        const float ref = cs[(I * 16 - 1) * PS + d];
-        q[c] = qs[(I * 16 + lo) * PV + d] *
-               expf(cs[(I * 16 + lo) * PS + d] - ref);
-        k[c] = ks[(J * 16 + lo) * PS + d] *
-               expf(ref - cs[(J * 16 + lo) * PS + d]);
-      }
-      u16x8 qh, ql, kh, kl;
-      split8(q, qh, ql);
+      for (int c = 0; c < 8; ++c)
+        k[c] = ks[j * PS + hi * 8 + c] *
+               exp2_(ref[c] - cs[j * PS + hi * 8 + c]);
+      u16x8 kh, kl;
       split8(k, kh, kl);
-      off[u] = mfma16(kh, qh, off[u]);
-      off[u] = mfma16(kh, ql, off[u]);
-      off[u] = mfma16(kl, qh, off[u]);
+      acc[J] = mfma16(kh, qh, acc[J]);
+      acc[J] = mfma16(kh, ql, acc[J]);
+      acc[J] = mfma16(kl, qh, acc[J]);
     }
+    if (steep)
+#pragma unroll
+      for (int J = 0; J < 4; ++J)
+        if (J == I)
+          for (int d = 0; d < SL; ++d) {
+            const float qd = qs[i * PV + d], cd = cs[i * PS + d];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+              const int j = J * 16 + hi * 4 + r;
+              if (j <= i)
+                acc[J][r] += qd * ks[j * PS + d] * exp2_(cd - cs[j * PS + d]);
+            }
+          }
   }
 
-  // the score matrix, through LDS
-  __syncthreads();
-  for (int i = tid; i < L * PA; i += NT) as[i] = 0.f;
-  __syncthreads();
+  uint16_t* ao = am + nh * 2 * L * L + (I * 16 + lo) * L + hi * 4;
 #pragma unroll
-  for (int i = 0; i < 16; ++i) {
-    float x = dg[i];
-    x += __shfl_xor(x, 1, WAVE);
-    x += __shfl_xor(x, 2, WAVE);
-    if ((lane & 3) == 0) as[(wid * 16 + i) * PA + wid * 16 + j] = x;
-  }
+  for (int J = 0; J < 4; ++J) {
+    float x[4], rest[4];
 #pragma unroll
-  for (int u = 0; u < 2; ++u) {
-    const int blk = wid + u * 4;
-    if (blk >= 6) continue;
-    const int I = blk < 1 ? 1 : (blk < 3 ? 2 : 3);
-    const int J = blk - I * (I - 1) / 2;
-    *reinterpret_cast<floatx4*>(as + (I * 16 + lo) * PA + J * 16 + hi * 4) =
-        off[u];
-  }
-  __syncthreads();
-  uint16_t* ao = am + nh * 2 * L * L;
-  {
-    const int i = tid / 4, c0 = tid % 4 * 16;
-#pragma unroll
-    for (int c = 0; c < 16; c += 8) {
-      float v[8];
-      ldv<8>(as + i * PA + c0 + c, v);
-      u16x8 a, b;
-      split8(v, a, b);
-      *reinterpret_cast<u16x8*>(ao + i * L + c0 + c) = a;
-      *reinterpret_cast<u16x8*>(ao + (L + i) * L + c0 + c) = b;
+    for (int r = 0; r < 4; ++r) {
+      x[r] = J < I || (J == I && hi * 4 + r <= lo) ? acc[J][r] : 0.f;
+      rest[r] = x[r] - bf16_to_f32(f32_to_bf16(x[r]));
     }
+    st_bf16x4(ao + J * 16, x);
+    st_bf16x4(ao + L * L + J * 16, rest);
   }
   // values, transposed
   for (int e0 = 0; e0 < m.Pp; e0 += SL) {
@@ -521,7 +534,7 @@ bool gla_chunks_fit(torch::Tensor z, int64_t dim) {
 void gla_operands(torch::Tensor qe, torch::Tensor ke, torch::Tensor am,
                   torch::Tensor vt, torch::Tensor ec, torch::Tensor z,
                   int64_t q_at, int64_t k_at, int64_t v_at, int64_t a_at,
-                  int64_t dim, int64_t vdim, torch::Tensor a2,
+                  int64_t dim, int64_t vdim, int64_t rank, torch::Tensor a2,
                   torch::Tensor a2_b, double tau, double q_scale,
                   torch::Tensor row, torch::Tensor count) {
   check_operands(qe, ke, am, vt, ec, dim, vdim);
@@ -532,8 +545,10 @@ void gla_operands(torch::Tensor qe, torch::Tensor ke, torch::Tensor am,
   m.Dp = qe.size(4);
   m.E = vdim;
   m.Pp = vt.size(2);
-  m.rank = a2.size(0);
-  check(a2, torch::kFloat32, (int64_t)m.rank * m.H * m.D);
+  m.rank = rank;
+  m.rank_pad = a2.size(1);
+  check(a2, torch::kBFloat16, (int64_t)m.rank_pad * m.H * m.D);
+  TORCH_CHECK(rank >= 1 && rank <= m.rank_pad && m.rank_pad % 32 == 0);
   check(a2_b, torch::kFloat32, (int64_t)m.H * m.D);
   check(row, torch::kInt32, n);
   check(count, torch::kInt32, n);
@@ -541,7 +556,7 @@ void gla_operands(torch::Tensor qe, torch::Tensor ke, torch::Tensor am,
   const int64_t width = z.size(1);
   TORCH_CHECK(q_at + m.H * m.D <= width && k_at + m.H * m.D <= width &&
               v_at + m.H * m.E <= width && a_at + m.rank <= width);
-  m.a2 = a2.data_ptr<float>();
+  m.a2 = (const uint16_t*)a2.data_ptr();
   m.a2_b = a2_b.data_ptr<float>();
   m.row = row.data_ptr<int>();
   m.count = count.data_ptr<int>();
@@ -550,19 +565,13 @@ void gla_operands(torch::Tensor qe, torch::Tensor ke, torch::Tensor am,
   m.k_at = k_at;
   m.v_at = v_at;
   m.a_at = a_at;
-  m.inv_tau = (float)(1.0 / tau);
+  m.unit = (float)(1.0 / tau);
   m.q_scale = (float)q_scale;
   m.vec = m.D % 8 == 0 && m.E % 8 == 0 && q_at % 8 == 0 && k_at % 8 == 0 &&
-          v_at % 8 == 0 && m.z_stride % 8 == 0 &&
+          v_at % 8 == 0 && a_at % 8 == 0 && m.z_stride % 8 == 0 &&
           (uintptr_t)z.data_ptr() % 16 == 0;
   if (n == 0) return;
-  const int lds = (2 * L * PV + 2 * L * PS + 8 * SL + L * m.rank) * 4;
-  TORCH_CHECK(m.rank >= 1 && lds <= 160 * 1024, "rank ", m.rank);
-  static const hipError_t big = hipFuncSetAttribute(
-      (const void*)gla_operands_kernel,
-      hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
-  TORCH_CHECK(big == hipSuccess, "LDS size refused");
-  hipLaunchKernelGGL(gla_operands_kernel, dim3(n, m.H), dim3(NT), lds,
+  hipLaunchKernelGGL(gla_operands_kernel, dim3(n, m.H), dim3(NT), 0,
                      at::hip::getCurrentHIPStream(), (uint16_t*)qe.data_ptr(),
                      (uint16_t*)ke.data_ptr(), (uint16_t*)am.data_ptr(),
                      (uint16_t*)vt.data_ptr(), ec.data_ptr<float>(),

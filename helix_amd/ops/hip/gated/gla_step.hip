@@ -18,14 +18,14 @@ using OptT = c10::optional<torch::Tensor>;
 namespace {
 
 struct Step {
-  const float* a2;             // [rank, H * D]
+  const void* a2;              // [H * D, rank_pad], storage type
   const float *a2_b, *norm;    // [H * D], [E]
   float* state;                // [slots, H, D, Ep]
   const int* slots;
   const int64_t* pos;          // per row
   const int* cu;               // spans: [B + 1] rows; null: a token each
   int64_t z_stride, y_stride;
-  int q_at, k_at, v_at, g_at, a_at, H, D, E, Ep, rank;
+  int q_at, k_at, v_at, g_at, a_at, H, D, E, Ep, rank, rank_pad;
   float inv_tau, q_scale, out_scale, eps;
 };
 
@@ -36,6 +36,7 @@ __global__ __launch_bounds__(TX* TY) void gla_step_kernel(
   constexpr int NT = TX * TY, NW = NT / WAVE;
   __shared__ float qs[TY * NI], ks[TY * NI], as[TY * NI], vs[TX * 4];
   __shared__ float part[NW][TX * 4], red[32];
+  extern __shared__ float a1[];               // [rank_pad]
   const int b = blockIdx.x, h = blockIdx.y;
   const int tid = threadIdx.x, tx = tid % TX, ty = tid / TX;
   const int row0 = m.cu ? m.cu[b] : b, row1 = m.cu ? m.cu[b + 1] : b + 1;
@@ -58,13 +59,21 @@ __global__ __launch_bounds__(TX* TY) void gla_step_kernel(
 
   for (int row = row0; row < row1; ++row) {
     const S* zr = z + row * m.z_stride;
+    for (int r = tid; r < m.rank_pad; r += NT)
+      a1[r] = r < m.rank ? ld1(zr + m.a_at + r) : 0.f;
+    __syncthreads();
     for (int d = tid; d < TY * NI; d += NT) {
       float a = 1.f, q = 0.f, k = 0.f;
       if (d < m.D) {
         const int c = h * m.D + d;
         float x = m.a2_b[c];
-        for (int r = 0; r < m.rank; ++r)
-          x += ld1(zr + m.a_at + r) * m.a2[(int64_t)r * m.H * m.D + c];
+        const S* w = (const S*)m.a2 + (int64_t)c * m.rank_pad;
+        for (int r = 0; r < m.rank_pad; r += 8) {
+          float u[8];
+          ldv<8>(w + r, u);
+#pragma unroll
+          for (int i = 0; i < 8; ++i) x += a1[r + i] * u[i];
+        }
         a = expf(-softplus(-x) * m.inv_tau);
         q = ld1(zr + m.q_at + c) * m.q_scale;
         k = ld1(zr + m.k_at + c);
@@ -130,7 +139,8 @@ void launch(torch::Tensor y, torch::Tensor z, Step m, int B) {
   const dim3 grid(B, m.H);
 #define HELIX_GLA(TX, TY, NI)                                                \
   hipLaunchKernelGGL((gla_step_kernel<S, TX, TY, NI>), grid, dim3(TX * TY),  \
-                     0, at::hip::getCurrentHIPStream(), (S*)y.data_ptr(),    \
+                     m.rank_pad * 4, at::hip::getCurrentHIPStream(),         \
+                     (S*)y.data_ptr(),                                       \
                      (const S*)z.data_ptr(), m)
 #define HELIX_GLA_D(TX, TY)                                                  \
   if (m.D <= TY * 2) HELIX_GLA(TX, TY, 2);                                   \
@@ -150,7 +160,7 @@ void launch(torch::Tensor y, torch::Tensor z, Step m, int B) {
 // z and y rows: one token of sequence r each, or (with cu) the concatenated
 // tokens of cu.numel() - 1 sequences.
 void gla_step(torch::Tensor y, torch::Tensor z, int64_t q_at, int64_t k_at,
-              int64_t v_at, int64_t g_at, int64_t a_at, int64_t vdim,
+              int64_t v_at, int64_t g_at, int64_t a_at, int64_t vdim, int64_t rank,
               torch::Tensor a2, torch::Tensor a2_b, torch::Tensor norm,
               double tau, double q_scale, double out_scale, double eps,
               torch::Tensor state, torch::Tensor slots, torch::Tensor pos,
@@ -162,7 +172,12 @@ void gla_step(torch::Tensor y, torch::Tensor z, int64_t q_at, int64_t k_at,
   m.D = state.size(2);
   m.Ep = state.size(3);
   m.E = vdim;
-  m.rank = a2.size(0);
+  m.rank = rank;
+  m.rank_pad = a2.size(1);
+  TORCH_CHECK(a2.dim() == 2 && a2.is_contiguous() &&
+              a2.size(0) == (int64_t)m.H * m.D && m.rank_pad % 8 == 0 &&
+              rank >= 1 && rank <= m.rank_pad && m.rank_pad <= 4096 &&
+              a2.scalar_type() == z.scalar_type());
   TORCH_CHECK(m.D <= 256 && m.E <= 256, "heads of at most 256 x 256, got ",
               m.D, " x ", m.E);
   TORCH_CHECK(m.Ep % 4 == 0 && m.Ep >= m.E && m.E > 0 && m.D > 0);
@@ -173,7 +188,7 @@ void gla_step(torch::Tensor y, torch::Tensor z, int64_t q_at, int64_t k_at,
   TORCH_CHECK(q_at + m.H * m.D <= width && k_at + m.H * m.D <= width &&
               v_at + m.H * m.E <= width && g_at + m.H * m.E <= width &&
               a_at + m.rank <= width);
-  m.a2 = f32(a2, (int64_t)m.rank * m.H * m.D);
+  m.a2 = a2.data_ptr();
   m.a2_b = f32(a2_b, (int64_t)m.H * m.D);
   m.norm = f32(norm, m.E);
   m.state = (float*)f32(state, state.numel());

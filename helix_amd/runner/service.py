@@ -55,6 +55,8 @@ DEFAULT_SPECS = {
     "zederax-1b": ModelSpec("zederax-1b", "llm", "zederax-1b"),
     "nibezen-8b": ModelSpec("nibezen-8b", "llm", "nibezen-8b"),
     "nibezen-1b": ModelSpec("nibezen-1b", "llm", "nibezen-1b"),
+    "motolix-8b": ModelSpec("motolix-8b", "llm", "motolix-8b"),
+    "motolix-1b": ModelSpec("motolix-1b", "llm", "motolix-1b"),
     "bge-base": ModelSpec("bge-base", "embedding", "bge-base"),
     "siglip-base": ModelSpec("siglip-base", "vision", "siglip-base"),
     "tiny-vit": ModelSpec("tiny-vit", "vision", "tiny-vit"),
@@ -69,6 +71,8 @@ DEFAULT_SPECS = {
     "tiny-zederax": ModelSpec("tiny-zederax", "llm", "tiny-zederax",
                               max_model_len=256, kv_cache_blocks=256),
     "tiny-nibezen": ModelSpec("tiny-nibezen", "llm", "tiny-nibezen",
+                              max_model_len=256, kv_cache_blocks=256),
+    "tiny-motolix": ModelSpec("tiny-motolix", "llm", "tiny-motolix",
                               max_model_len=256, kv_cache_blocks=256),
     "tiny-bert": ModelSpec("tiny-bert", "embedding", "tiny-bert"),
 }

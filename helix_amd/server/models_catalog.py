@@ -36,6 +36,12 @@ STATIC_MODEL_INFO: Dict[str, dict] = {
     "nibezen-1b": {"context_length": 32768, "prompt_price_per_m": 0.02,
                    "completion_price_per_m": 0.04, "family": "nibezen",
                    "runtime": "helix_amd", "kind": "chat"},
+    "motolix-8b": {"context_length": 32768, "prompt_price_per_m": 0.05,
+                   "completion_price_per_m": 0.10, "family": "motolix",
+                   "runtime": "helix_amd", "kind": "chat"},
+    "motolix-1b": {"context_length": 32768, "prompt_price_per_m": 0.02,
+                   "completion_price_per_m": 0.04, "family": "motolix",
+                   "runtime": "helix_amd", "kind": "chat"},
     "bge-base": {"context_length": 512, "prompt_price_per_m": 0.005,
                  "completion_price_per_m": 0.0, "family": "bge",
                  "runtime": "helix_amd", "kind": "embedding"},
