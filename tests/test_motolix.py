@@ -263,7 +263,8 @@ LAYERS = {
     "sigmoid large": {"type": "attention", "mixer": attn(2, 1, 200, 200, 50)},
     "sigmoid plain": {"type": "attention", "mixer": attn(2, 2, 264, 264, 8)},
     "sigmoid unrotated": {"type": "attention", "mixer": attn(3, 1, 16, 16, 0)},
-    "parallel": parallel(attn(4, 2, 24, 40, 16), gla(3, 24, 20, 4.0)),
+    "parallel": parallel(attn(4, 2, 24, 40, 4, 0.6, 1e8),
+                         gla(3, 24, 20, 4.0)),
     "parallel small": parallel(attn(1, 1, 6, 2, 2), gla(1, 1, 1, 1.0), 1., 1.),
     "parallel odd": parallel(attn(3, 1, 10, 14, 10), gla(2, 37, 51, 2.0)),
     "parallel 64": parallel(attn(8, 2, 64, 64, 64, scaling=SCALING),
