@@ -198,10 +198,8 @@ def attn_rows(out: torch.Tensor, q: torch.Tensor, p: AttnParams, kv_cache,
     if workspace is None or workspace.numel() < need:
         workspace = torch.empty(need, dtype=torch.float32, device=q.device)
     n = R * parts * p.heads
-    part = workspace[:n * p.vdim].view(R, parts, p.heads, p.vdim)
-    ml = workspace[n * p.vdim:need]
-    if (n * p.vdim) % 2:
-        raise ValueError("odd scratch")
+    ml = workspace[:2 * n]
+    part = workspace[2 * n:need].view(R, parts, p.heads, p.vdim)
     C.attn_rows(None, part, ml, q, k, v, block_tables, row_seq, row_len,
                 p.scale, p.out_scale, p.sigmoid, p.temp, p.bias, vcs)
     C.attn_merge(out, part, ml, p.out_scale, p.sigmoid, vcs)

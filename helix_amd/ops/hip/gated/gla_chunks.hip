@@ -45,21 +45,21 @@ struct Operands {
 
 // Columns c0 .. c0 + 31 of the chunk's rows, 8 per thread; nothing past
 // column n or row count.
-__device__ __forceinline__ void load_slice(float* v, const uint16_t* z,
-                                           int64_t stride, int c0, int n,
-                                           int count, bool vec) {
+__device__ __forceinline__ u16x8 load_slice(const uint16_t* z, int64_t stride,
+                                            int c0, int n, int count,
+                                            bool vec) {
   const int t = threadIdx.x / 4, d = c0 + threadIdx.x % 4 * 8;
-#pragma unroll
-  for (int i = 0; i < 8; ++i) v[i] = 0.f;
-  if (t >= count) return;
+  u16x8 v = {0, 0, 0, 0, 0, 0, 0, 0};
+  if (t >= count) return v;
   const uint16_t* p = z + t * stride + d;
   if (vec) {
-    if (d < n) ldv<8>(p, v);
+    if (d < n) v = ld_u16x8(p);
   } else {
 #pragma unroll
     for (int i = 0; i < 8; ++i)
-      if (d + i < n) v[i] = bf16_to_f32(p[i]);
+      if (d + i < n) v[i] = p[i];
   }
+  return v;
 }
 
 __device__ __forceinline__ float exp2_(float x) {
@@ -100,34 +100,61 @@ __global__ __launch_bounds__(NT) void gla_operands_kernel(
 #pragma unroll
   for (int i = 0; i < 4; ++i) acc[i] = floatx4{0, 0, 0, 0};
 
+  // inputs of the decays: wave w has tokens 16 w ..
+  auto rank_terms = [&](int r) {
+    u16x8 a = {0, 0, 0, 0, 0, 0, 0, 0};
+    const int t = wid * 16 + lo;
+    if (t < count && r < m.rank) {
+      const uint16_t* ap = zr + t * m.z_stride + m.a_at + r;
+      if (m.vec && r + 8 <= m.rank) {
+        a = ld_u16x8(ap);
+      } else {
+#pragma unroll
+        for (int i = 0; i < 8; ++i)
+          if (r + i < m.rank) a[i] = ap[i];
+      }
+    }
+    return a;
+  };
+  const u16x8 a0 = rank_terms(hi * 8);
+  const uint16_t *zq = zr + m.q_at + h * m.D, *zk = zr + m.k_at + h * m.D;
+  // a slice's queries, keys and decay weights are under way one slice ahead
+  u16x8 qreg, kreg, b0[2];
+  auto load = [&](int d0) {
+    qreg = load_slice(zq, m.z_stride, d0, m.D, count, m.vec);
+    kreg = load_slice(zk, m.z_stride, d0, m.D, count, m.vec);
+#pragma unroll
+    for (int u = 0; u < 2; ++u)
+      b0[u] = ld_u16x8(m.a2 + (int64_t)(h * m.D + min(d0 + u * 16 + lo,
+                                                      m.D - 1)) *
+                                  m.rank_pad + hi * 8);
+  };
+
+  load(0);
   for (int d0 = 0; d0 < m.Dp; d0 += SL) {
     float v[8], w[8];
     const int t = tid / 4, s = tid % 4 * 8;
-    load_slice(v, zr + m.q_at + h * m.D, m.z_stride, d0, m.D, count, m.vec);
-    load_slice(w, zr + m.k_at + h * m.D, m.z_stride, d0, m.D, count, m.vec);
-    // decays: wave w has tokens 16 w .., a lane 4 tokens of two channels
-    floatx4 x[2] = {floatx4{0, 0, 0, 0}, floatx4{0, 0, 0, 0}};
-    const int ta = wid * 16 + lo;
-    for (int r = hi * 8; r < m.rank_pad; r += 32) {
-      u16x8 a = {0, 0, 0, 0, 0, 0, 0, 0};
-      if (ta < count && r < m.rank) {
-        const uint16_t* ap = zr + ta * m.z_stride + m.a_at + r;
-        if (m.vec && r + 8 <= m.rank) {
-          a = ld_u16x8(ap);
-        } else {
 #pragma unroll
-          for (int i = 0; i < 8; ++i)
-            if (r + i < m.rank) a[i] = ap[i];
-        }
-      }
+    for (int i = 0; i < 8; ++i) {
+      v[i] = bf16_to_f32(qreg[i]);
+      w[i] = bf16_to_f32(kreg[i]);
+    }
+    // a lane has 4 tokens of two channels
+    floatx4 x[2];
+#pragma unroll
+    for (int u = 0; u < 2; ++u)
+      x[u] = mfma16(a0, b0[u], floatx4{0, 0, 0, 0});
+    for (int r = 32 + hi * 8; r < m.rank_pad; r += 32) {
+      const u16x8 a = rank_terms(r);
 #pragma unroll
       for (int u = 0; u < 2; ++u) {
         const int c = min(d0 + u * 16 + lo, m.D - 1);
-        const u16x8 b =
-            ld_u16x8(m.a2 + (int64_t)(h * m.D + c) * m.rank_pad + r);
-        x[u] = mfma16(a, b, x[u]);
+        x[u] = mfma16(
+            a, ld_u16x8(m.a2 + (int64_t)(h * m.D + c) * m.rank_pad + r),
+            x[u]);
       }
     }
+    if (d0 + SL < m.Dp) load(d0 + SL);
     float part[2];
 #pragma unroll
     for (int u = 0; u < 2; ++u) {
@@ -231,6 +258,8 @@ __global__ __launch_bounds__(NT) void gla_operands_kernel(
           }
   }
 
+  const uint16_t* zv = zr + m.v_at + h * m.E;
+  u16x8 vreg = load_slice(zv, m.z_stride, 0, m.E, count, m.vec);
   uint16_t* ao = am + nh * 2 * L * L + (I * 16 + lo) * L + hi * 4;
 #pragma unroll
   for (int J = 0; J < 4; ++J) {
@@ -246,10 +275,13 @@ __global__ __launch_bounds__(NT) void gla_operands_kernel(
   // values, transposed
   for (int e0 = 0; e0 < m.Pp; e0 += SL) {
     float v[8];
-    load_slice(v, zr + m.v_at + h * m.E, m.z_stride, e0, m.E, count, m.vec);
+    const u16x8 raw = vreg;
+    if (e0 + SL < m.Pp) vreg = load_slice(zv, m.z_stride, e0 + SL, m.E, count,
+                                          m.vec);
     __syncthreads();
 #pragma unroll
-    for (int i = 0; i < 8; ++i) ks[tid / 4 * PS + tid % 4 * 8 + i] = v[i];
+    for (int i = 0; i < 8; ++i)
+      ks[tid / 4 * PS + tid % 4 * 8 + i] = bf16_to_f32(raw[i]);
     __syncthreads();
     const int e = e0 + tid / 8, t = tid % 8 * 8;
 #pragma unroll

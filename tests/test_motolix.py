@@ -352,7 +352,8 @@ def test_mixer_batches_and_single_tokens(dev, dtype, name):
 
 @pytest.mark.parametrize("dev", DEVICES)
 @pytest.mark.parametrize("dtype", [F32, BF16])
-@pytest.mark.parametrize("name", ["sigmoid", "parallel 64"])
+@pytest.mark.parametrize("name", ["sigmoid", "sigmoid odd", "sigmoid wide",
+                                  "parallel odd", "parallel 64"])
 def test_long_rows_in_partitions(dev, dtype, name):
     """A single token far into a sequence: its keys are cut into partitions
     on the GPU, and only a far one stands out."""
