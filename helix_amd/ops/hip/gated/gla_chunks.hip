@@ -302,10 +302,19 @@ struct Chunks {
   int H, D, Dp, E, Ep, Pp, vec;
 };
 
+// A chunk's operands on their way to one thread.
+template <int NK, int XL>
+struct Stage {
+  u16x8 k[NK * 2], q[2][NK], a[2][2], x[XL];
+  float e;
+};
+
 // NK: 32-wide steps of the key channels; PW: 16-value tiles of a workgroup.
 // Wave w has tokens 16 w .. of the output, and of the state the value tile
-// w % PW in its share of the rows.
-template <int NK, int PW>
+// w % PW in its share of the rows. FULL: every tile is a whole one, so
+// nothing branches and the products of different tiles overlap (a chunk
+// waits for the one before, so the chunk's own latency is the time).
+template <int NK, int PW, bool FULL>
 __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void gla_chunks_kernel(
     uint16_t* __restrict__ o, const uint16_t* __restrict__ qe,
     const uint16_t* __restrict__ ke, const uint16_t* __restrict__ am,
@@ -347,8 +356,7 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void gla_chunks_kernel(
       S[t][r] = carried && t < nts && n < m.D ? st[(int64_t)n * m.Ep] : 0.f;
     }
 
-  u16x8 kreg[KR], qreg[2][NK], areg[2][2], xreg[XL];
-  float ereg = 0.f;
+  Stage<NK, XL> in;
   // No branches, so that all loads are under way at once: indices past the
   // end are clamped and their values not stored or not used.
   auto load = [&](int n) {
@@ -356,23 +364,23 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void gla_chunks_kernel(
     const uint16_t* kn = ke + nh * 2 * L * m.Dp;
 #pragma unroll
     for (int i = 0; i < KR; ++i)
-      kreg[i] = ld_u16x8(kn + min(i * NT + tid, m.Dp * 16 - 1) * 8);
+      in.k[i] = ld_u16x8(kn + min(i * NT + tid, m.Dp * 16 - 1) * 8);
     const uint16_t* qn = qe + (nh * 2 * L + wid * 16 + lo) * m.Dp + hi * 8;
 #pragma unroll
     for (int s = 0; s < 2; ++s) {
 #pragma unroll
       for (int k = 0; k < NK; ++k)
-        qreg[s][k] = ld_u16x8(qn + (int64_t)s * L * m.Dp + min(k, ks - 1) * 32);
+        in.q[s][k] = ld_u16x8(qn + (int64_t)s * L * m.Dp + min(k, ks - 1) * 32);
       const uint16_t* an =
           am + ((nh * 2 + s) * L + wid * 16 + lo) * L + hi * 8;
-      areg[s][0] = ld_u16x8(an);
-      areg[s][1] = ld_u16x8(an + 32);
+      in.a[s][0] = ld_u16x8(an);
+      in.a[s][1] = ld_u16x8(an + 32);
     }
     const uint16_t* xn = vt + (nh * m.Pp + p0) * L;
 #pragma unroll
     for (int i = 0; i < XL; ++i)
-      xreg[i] = ld_u16x8(xn + min(i * NT + tid, rowsp * 8 - 1) * 8);
-    ereg = m.ec[nh * m.Dp + min(tid, m.Dp - 1)];
+      in.x[i] = ld_u16x8(xn + min(i * NT + tid, rowsp * 8 - 1) * 8);
+    in.e = m.ec[nh * m.Dp + min(tid, m.Dp - 1)];
   };
 
   load(n0);
@@ -381,18 +389,18 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void gla_chunks_kernel(
 #pragma unroll
     for (int i = 0; i < KR; ++i) {
       const int e = i * NT + tid;
-      if (e < m.Dp * 16)
-        *reinterpret_cast<u16x8*>(kl + e / 8 * LP + e % 8 * 8) = kreg[i];
+      if (FULL || e < m.Dp * 16)
+        *reinterpret_cast<u16x8*>(kl + e / 8 * LP + e % 8 * 8) = in.k[i];
     }
 #pragma unroll
     for (int i = 0; i < XL; ++i) {
       const int e = i * NT + tid;
-      *reinterpret_cast<u16x8*>(xl + e / 8 * LP + e % 8 * 8) = xreg[i];
+      *reinterpret_cast<u16x8*>(xl + e / 8 * LP + e % 8 * 8) = in.x[i];
     }
-    if (tid < m.Dp) el[tid] = ereg;
+    if (tid < m.Dp) el[tid] = in.e;
 #pragma unroll
     for (int t = 0; t < ST; ++t)
-      if (t < nts) {
+      if (FULL || t < nts) {
         const uint32_t u0 = pack_bf16(S[t][0], S[t][1]);
         const uint32_t u1 = pack_bf16(S[t][2], S[t][3]);
         const int at = (pt * 16 + lo) * NP + (nt0 + t) * 16 + hi * 4;
@@ -408,9 +416,9 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void gla_chunks_kernel(
 #pragma unroll
     for (int s = 0; s < 2; ++s) {
 #pragma unroll
-      for (int k = 0; k < NK; ++k) qf[s][k] = qreg[s][k];
-      af[s][0] = areg[s][0];
-      af[s][1] = areg[s][1];
+      for (int k = 0; k < NK; ++k) qf[s][k] = in.q[s][k];
+      af[s][0] = in.a[s][0];
+      af[s][1] = in.a[s][1];
     }
     __syncthreads();
     if (n + 1 < n1) load(n + 1);
@@ -420,13 +428,13 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void gla_chunks_kernel(
     const int64_t row = row0 + (int64_t)(n - n0) * L + i;
 #pragma unroll
     for (int t = 0; t < PW; ++t) {
-      if (t * 16 >= np) continue;
+      if (!FULL && t * 16 >= np) continue;
       floatx4 d = floatx4{0, 0, 0, 0};
       const uint16_t* s1 = sh + (t * 16 + lo) * NP + hi * 8;
       const uint16_t* s2 = sl + (t * 16 + lo) * NP + hi * 8;
 #pragma unroll
       for (int k = 0; k < NK; ++k)
-        if (k < ks) {
+        if (FULL || k < ks) {
           const u16x8 a = ld_u16x8(s1 + k * 32);
           d = mfma16(a, qf[0][k], d);
           d = mfma16(a, qf[1][k], d);
@@ -434,7 +442,7 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void gla_chunks_kernel(
         }
 #pragma unroll
       for (int jp = 0; jp < 2; ++jp) {
-        if (jp > (wid >> 1)) continue;
+        if (!FULL && jp > (wid >> 1)) continue;  // zero there
         const u16x8 a = ld_u16x8(xl + (t * 16 + lo) * LP + jp * 32 + hi * 8);
         d = mfma16(a, af[0][jp], d);
         d = mfma16(a, af[1][jp], d);
@@ -453,10 +461,10 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void gla_chunks_kernel(
       }
     }
     // --- state
-    if (pt * 16 < np) {
+    if (FULL || pt * 16 < np) {
 #pragma unroll
       for (int t = 0; t < ST; ++t)
-        if (t < nts) {
+        if (FULL || t < nts) {
           const f32x4 ee = *reinterpret_cast<const f32x4*>(
               el + (nt0 + t) * 16 + hi * 4);
 #pragma unroll
@@ -468,7 +476,7 @@ __global__ __launch_bounds__(NT, NK > 4 ? 1 : 2) void gla_chunks_kernel(
             ld_u16x8(xl + (pt * 16 + lo) * LP + kk * 32 + hi * 8);
 #pragma unroll
         for (int t = 0; t < ST; ++t)
-          if (t < nts) {
+          if (FULL || t < nts) {
             const uint16_t* a =
                 kl + ((nt0 + t) * 16 + lo) * LP + kk * 32 + hi * 8;
             S[t] = mfma16(ld_u16x8(a), x, S[t]);
@@ -649,13 +657,15 @@ void gla_chunks(torch::Tensor o, torch::Tensor qe, torch::Tensor ke,
   const dim3 grid(m.H, B, cdiv(m.E, PB));
   const int lds =
       (2 * m.Dp * LP + PB * LP + 2 * PB * (m.Dp + 8)) * 2 + m.Dp * 4;
-#define HELIX_GC_P(NK, PW)                                                   \
+  const bool full = m.E % PB == 0 && (m.Dp & (m.Dp - 1)) == 0;
+#define HELIX_GC_F(NK, PW, FULL)                                             \
   do {                                                                       \
     static const hipError_t big = hipFuncSetAttribute(                       \
-        (const void*)gla_chunks_kernel<NK, PW>,                              \
+        (const void*)gla_chunks_kernel<NK, PW, FULL>,                        \
         hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);             \
     TORCH_CHECK(big == hipSuccess, "LDS size refused");                      \
-    hipLaunchKernelGGL((gla_chunks_kernel<NK, PW>), grid, dim3(NT), lds,     \
+    hipLaunchKernelGGL((gla_chunks_kernel<NK, PW, FULL>), grid, dim3(NT),    \
+                       lds,                                                  \
                        at::hip::getCurrentHIPStream(),                       \
                        (uint16_t*)o.data_ptr(),                              \
                        (const uint16_t*)qe.data_ptr(),                       \
@@ -663,14 +673,17 @@ void gla_chunks(torch::Tensor o, torch::Tensor qe, torch::Tensor ke,
                        (const uint16_t*)am.data_ptr(),                       \
                        (const uint16_t*)vt.data_ptr(), m);                   \
   } while (0)
+#define HELIX_GC_P(NK, PW)                                                   \
+  if (full) HELIX_GC_F(NK, PW, true); else HELIX_GC_F(NK, PW, false)
 #define HELIX_GC(NK)                                                         \
-  if (PW == 4) HELIX_GC_P(NK, 4); else HELIX_GC_P(NK, 2)
+  if (PW == 4) { HELIX_GC_P(NK, 4); } else { HELIX_GC_P(NK, 2); }
   if (m.Dp <= 32) { HELIX_GC(1); }
   else if (m.Dp <= 64) { HELIX_GC(2); }
   else if (m.Dp <= 128) { HELIX_GC(4); }
   else { HELIX_GC(8); }
 #undef HELIX_GC
 #undef HELIX_GC_P
+#undef HELIX_GC_F
 }
 
 void head_norm_gate(torch::Tensor y, torch::Tensor o, torch::Tensor g,
