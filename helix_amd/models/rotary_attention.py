@@ -89,12 +89,6 @@ class AttnSpec:
         if self.value_rotary is not None and self.vdim % 2:
             raise ValueError(f"values of {self.vdim} cannot turn in pairs")
 
-    @classmethod
-    def from_json(cls, m: dict, **kinds) -> "AttnSpec":
-        return cls(heads=m["heads"], kv_heads=m["kv_heads"], dim=m["dim"],
-                   vdim=m["vdim"], scale=float(m["scale"]),
-                   rotary=HalvesRotary.from_json(m.get("rot")), **kinds)
-
     @property
     def value_rotary(self) -> Optional[HalvesRotary]:
         """All of a value, with the keys' base and no scaling."""
