@@ -10,7 +10,7 @@ from __future__ import annotations
 
 import time
 import zlib
-from dataclasses import dataclass, field
+from dataclasses import dataclass, field, replace
 from enum import Enum
 from typing import Callable, Dict, List, Optional
 
@@ -103,6 +103,10 @@ class LLMEngine:
         self.device = torch.device(device)
         self.model_cfg = model.cfg if model is not None \
             else registry.get_config(cfg.model)
+        # learned positions bound the length of a sequence
+        limit = getattr(self.model_cfg, "position_limit", None)
+        if limit is not None and cfg.max_model_len > limit:
+            cfg = self.cfg = replace(cfg, max_model_len=limit)
         self.tp_size = tp_size
         self.tp_rank = tp_rank
         self.tp_group = tp_group

@@ -1,8 +1,9 @@
 """Mixers that read the same rows and whose scaled results add up: one fused
 projection in, one out, whose accumulator does the addition.
 
-A member is a spec (inputs(), out_size, bias, cache_layer()) with its module
-(forward(out, z, cache, meta, tables) fills its columns of the buffer that
+A member is a spec (inputs(), out_size, bias, cache_layer(); shared_kv if it
+has no cache of its own) with its module (forward(out, z, cache, meta, tables)
+fills its columns of the buffer that
 the output projection reads; its scale is applied there, in fp32).
 """
 from __future__ import annotations
@@ -14,16 +15,20 @@ import torch
 import torch.nn as nn
 
 from helix_amd.models.base import round_up
-from helix_amd.models.gla import GatedLinearAttention, GLASpec
+from helix_amd.models.gla import (GatedLinearAttention, GLASpec,
+                                  LightningAttention, LightningSpec)
 from helix_amd.models.llama import HLinear
 from helix_amd.models.rotary_attention import AttnSpec, RotaryAttention
+from helix_amd.models.selective import SelectiveScan, SelectiveSpec
 
-MODULES = {AttnSpec: RotaryAttention, GLASpec: GatedLinearAttention}
+MODULES = {AttnSpec: RotaryAttention, GLASpec: GatedLinearAttention,
+           LightningSpec: LightningAttention, SelectiveSpec: SelectiveScan}
+MixerSpec = Union[AttnSpec, GLASpec, LightningSpec, SelectiveSpec]
 
 
 @dataclass(frozen=True)
 class Member:
-    spec: Union[AttnSpec, GLASpec]
+    spec: MixerSpec
     prefix: str = ""             # of its checkpoint names
     scale: float = 1.0
 
@@ -41,7 +46,9 @@ class GroupSpec:
         return any(m.spec.bias for m in self.members)
 
     def cache_layers(self) -> list:
-        return [m.spec.cache_layer() for m in self.members]
+        """Of the members that have a cache of their own."""
+        return [m.spec.cache_layer() for m in self.members
+                if not m.spec.shared_kv]
 
     def num_weights(self, width: int) -> int:
         return sum(width * (sum(n for _, n in m.spec.inputs())
@@ -80,6 +87,7 @@ class MixerGroup(nn.Module):
         return max(c.scratch_floats(max_batch, max_len) for c in self.cores)
 
     def forward(self, h, caches, meta, tables):
+        """caches: one entry per member, of its own or shared."""
         z = self.in_proj(h)
         width = self.out_proj.weight.shape[1]
         buf = torch.empty(h.shape[0], width, dtype=h.dtype, device=h.device)

@@ -10,19 +10,22 @@ import json
 import os
 from typing import Callable, Dict, Optional
 
-from helix_amd.models import llama, motolix, nibezen, zederax
+from helix_amd.models import dibizen, llama, motolix, nibezen, zederax
+from helix_amd.models.dibizen import DibizenConfig, DibizenForCausalLM
 from helix_amd.models.llama import LlamaConfig, LlamaForCausalLM
 from helix_amd.models.motolix import MotolixConfig, MotolixForCausalLM
 from helix_amd.models.nibezen import NibezenConfig, NibezenForCausalLM
 from helix_amd.models.zederax import ZederaxConfig, ZederaxForCausalLM
 
-MODEL_CLASSES = {LlamaConfig: LlamaForCausalLM,
+MODEL_CLASSES = {DibizenConfig: DibizenForCausalLM,
+                 LlamaConfig: LlamaForCausalLM,
                  MotolixConfig: MotolixForCausalLM,
                  NibezenConfig: NibezenForCausalLM,
                  ZederaxConfig: ZederaxForCausalLM}
 
 # config.json architecture -> reader(dict, name) of the configuration
 CONFIG_READERS: Dict[str, Callable] = {
+    "Dibizen": DibizenConfig.from_json,
     "Motolix": MotolixConfig.from_json,
     "Nibezen": NibezenConfig.from_json,
     "Zederax": ZederaxConfig.from_json,
@@ -41,8 +44,8 @@ def is_folder(model: str) -> bool:
 
 def get_config(model: str):
     """Configuration of a preset or of a checkpoint folder."""
-    families = (llama.PRESETS, motolix.PRESETS, nibezen.PRESETS,
-                zederax.PRESETS)
+    families = (dibizen.PRESETS, llama.PRESETS, motolix.PRESETS,
+                nibezen.PRESETS, zederax.PRESETS)
     for presets in families:
         if model in presets:
             return presets[model]

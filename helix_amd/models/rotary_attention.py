@@ -1,10 +1,12 @@
-"""Attention over paged keys and values with rotated positions.
+"""Attention over paged keys and values, with rotated positions or none.
 
 Per head: score = (q . k) * scale over rotated q and k; weights are a softmax
 or (sigmoid) each 1 / (1 + e^-(temp * score + bias)), not normalised. q and k
 may be RMS-normed over their whole projections, values may be the unrotated
 keys, and may travel rotated: cached turned by their position, results turned
-back by the query's.
+back by the query's. A query may have a temperature that grows with its
+position, results a gate per value; a layer without projections of its own
+for keys and values reads those of another layer's cache.
 """
 from __future__ import annotations
 
@@ -48,8 +50,8 @@ class HalvesRotary:
 
 
 class RotaryTables:
-    """Cosines and sines of a step's positions, made once for all layers
-    that turn alike."""
+    """What depends on a step's positions alone, made once for all layers
+    that share it: cosines and sines, query temperatures."""
 
     def __init__(self, positions: torch.Tensor):
         self.positions = positions
@@ -61,6 +63,30 @@ class RotaryTables:
         if rotary not in self.made:
             self.made[rotary] = gated.rotary_table(self.positions, freqs)
         return self.made[rotary]
+
+    def temperature(self, t: Optional["QueryTemperature"]):
+        if t is None:
+            return None
+        if t not in self.made:
+            self.made[t] = gated.query_temperature(self.positions, t.coef,
+                                                   t.every)
+        return self.made[t]
+
+
+@dataclass(frozen=True)
+class QueryTemperature:
+    """A query at position p is multiplied by
+    1 + coef * ln(floor((p + 1) / every) + 1)."""
+    coef: float
+    every: float
+
+    def __post_init__(self):
+        if self.every <= 0:
+            raise ValueError(f"query temperature every {self.every} tokens")
+
+    @classmethod
+    def from_json(cls, d: Optional[dict]) -> Optional["QueryTemperature"]:
+        return None if not d else cls(float(d["coef"]), float(d["every"]))
 
 
 @dataclass(frozen=True)
@@ -76,11 +102,17 @@ class AttnSpec:
     bias: bool = False           # in the projections
     qk_norm: bool = False        # over the whole projections
     turn_values: bool = False
+    q_temp: Optional[QueryTemperature] = None
+    gate: bool = False           # sigmoid per value on the results
+    shared_kv: bool = False      # no keys and values of its own
 
     def __post_init__(self):
         if self.heads % self.kv_heads:
             raise ValueError(f"{self.heads} heads over {self.kv_heads} "
                              "key/value heads")
+        if self.shared_kv and (self.tied_values or self.qk_norm):
+            raise ValueError("shared keys and values have no projections "
+                             "to tie or to norm")
         if self.tied_values and self.dim != self.vdim:
             raise ValueError(f"keys of {self.dim} as values of {self.vdim}")
         if self.rotary is not None and self.rotary.dims > self.dim:
@@ -98,9 +130,14 @@ class AttnSpec:
 
     def inputs(self) -> list:
         """(checkpoint name, columns) of what is projected from a row."""
-        out = [("q", self.heads * self.dim), ("k", self.kv_heads * self.dim)]
-        return out if self.tied_values else \
-            out + [("v", self.kv_heads * self.vdim)]
+        out = [("q", self.heads * self.dim)]
+        if not self.shared_kv:
+            out.append(("k", self.kv_heads * self.dim))
+            if not self.tied_values:
+                out.append(("v", self.kv_heads * self.vdim))
+        if self.gate:
+            out.append(("g", self.out_size))
+        return out
 
     @property
     def out_size(self) -> int:
@@ -143,9 +180,10 @@ class RotaryAttention(Float32Kept):
                                  else rot.frequencies(), persistent=False)
         self._shape = dict(
             heads=H, kv_heads=G, dim=D, vdim=spec.vdim,
-            dim_pad=round_up(D, 8), q_at=at["q"], k_at=at["k"],
-            v_at=at["k" if spec.tied_values else "v"], scale=spec.scale,
-            out_scale=out_scale, sigmoid=spec.sigmoid)
+            dim_pad=round_up(D, 8), q_at=at["q"], k_at=at.get("k", -1),
+            v_at=at.get("k" if spec.tied_values else "v", -1),
+            scale=spec.scale, out_scale=out_scale, sigmoid=spec.sigmoid)
+        self.gate_at = at.get("g", -1)
 
     @property
     def params(self) -> gated.AttnParams:
@@ -165,21 +203,31 @@ class RotaryAttention(Float32Kept):
         q = gated.attn_epilogue(z, p, kv_cache, meta.slot_mapping,
                                 tables.get(s.rotary, self.freqs), vcs,
                                 self.q_norm, self.k_norm, self.eps)
+        # one entry per row of the batch, as out and q
+        by_row = dict(vcs=vcs, row_scale=tables.temperature(s.q_temp),
+                      gate=z[:, self.gate_at:self.gate_at + s.out_size]
+                      if s.gate else None)
+
+        def rows(of: slice) -> dict:
+            return {k: None if t is None else t[of]
+                    for k, t in by_row.items()}
+
         if isinstance(meta, MixedMeta):
             n = meta.num_decode
-            a, b = (None, None) if vcs is None else (vcs[:n], vcs[n:])
-            self._rows(out[:n], q[:n], p, kv_cache, meta.decode, a)
-            gated.attn_prompt(out[n:], q[n:], p, kv_cache, meta.prefill, b)
+            self._rows(out[:n], q[:n], p, kv_cache, meta.decode,
+                       rows(slice(0, n)))
+            gated.attn_prompt(out[n:], q[n:], p, kv_cache, meta.prefill,
+                              **rows(slice(n, None)))
         elif meta.is_prefill:
-            gated.attn_prompt(out, q, p, kv_cache, meta, vcs)
+            gated.attn_prompt(out, q, p, kv_cache, meta, **by_row)
         else:
-            self._rows(out, q, p, kv_cache, meta, vcs)
+            self._rows(out, q, p, kv_cache, meta, by_row)
 
     @staticmethod
-    def _rows(out, q, p, kv_cache, meta, vcs):
+    def _rows(out, q, p, kv_cache, meta, by_row):
         gated.attn_rows(out, q, p, kv_cache, meta.block_tables,
-                        meta.seq_lens, meta.max_len, vcs,
-                        workspace=meta.workspace)
+                        meta.seq_lens, meta.max_len,
+                        workspace=meta.workspace, **by_row)
 
     def targets(self, prefix: str) -> dict:
         named = {"q.norm": self.q_norm, "k.norm": self.k_norm,

@@ -1,7 +1,7 @@
 """In-tree build of the native extensions, on demand.
 
 A source checkout has no built libraries; a program that needs one calls
-ensure() before it imports helix_amd.ops. Only the named extension is
+ensure() before it imports helix_amd.ops. Only the named extensions are
 compiled (gfx950, cross-compilation needs no GPU).
 """
 from __future__ import annotations
@@ -20,12 +20,13 @@ def is_built(name: str) -> bool:
     return bool(glob.glob(os.path.join(ROOT, "helix_amd", f"{name}.*.so")))
 
 
-def ensure(name: str) -> None:
-    """Compile extension `name` unless its library is there. The compiler's
-    output goes to standard error."""
-    if is_built(name):
+def ensure(names: str) -> None:
+    """Compile the extensions (names with commas between them) whose library
+    is not there. The compiler's output goes to standard error."""
+    names = ",".join(n for n in names.split(",") if not is_built(n))
+    if not names:
         return
-    env = dict(os.environ, PYTORCH_ROCM_ARCH="gfx950", HELIX_BUILD_ONLY=name)
+    env = dict(os.environ, PYTORCH_ROCM_ARCH="gfx950", HELIX_BUILD_ONLY=names)
     subprocess.run([sys.executable, "setup.py", "build_ext", "--inplace"],
                    cwd=ROOT, env=env, check=True, stdout=sys.stderr)
 

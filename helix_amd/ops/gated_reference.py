@@ -50,6 +50,11 @@ def rotary_table(positions, freqs):
     return torch.stack([torch.cos(a), torch.sin(a)], -1).float()
 
 
+def query_temperature(positions, coef, every):
+    n = torch.floor((positions + 1).double() / every) + 1
+    return (1 + coef * torch.log(n)).float()
+
+
 def _turn(v, cs):
     """v [T, heads, D]: pairs (i, i + n) by table cs [T, n, 2]."""
     if cs is None:
@@ -69,6 +74,8 @@ def attn_epilogue(q, kc, vc, z, p, slots, cs, vcs, q_norm, k_norm, eps):
 
     q.zero_()
     q[..., :p.dim] = _turn(part(p.q_at, p.heads, p.dim, q_norm), cs)
+    if p.k_at < 0:
+        return
     k = F.pad(_turn(part(p.k_at, p.kv_heads, p.dim, k_norm), cs),
               (0, p.dim_pad - p.dim))
     v = _turn(part(p.v_at, p.kv_heads, p.vdim), vcs)
@@ -79,7 +86,8 @@ def attn_epilogue(q, kc, vc, z, p, slots, cs, vcs, q_norm, k_norm, eps):
     vc[s // bs, :, :, s % bs] = v[live].to(vc.dtype)
 
 
-def attn_rows(out, q, p, kc, vc, block_tables, row_len, vcs, row_seq):
+def attn_rows(out, q, p, kc, vc, block_tables, row_len, vcs, row_seq,
+              row_scale, gate):
     bs, per = kc.shape[2], p.heads // p.kv_heads
     for r in range(q.shape[0]):
         n = int(row_len[r])
@@ -89,6 +97,8 @@ def attn_rows(out, q, p, kc, vc, block_tables, row_len, vcs, row_seq):
         v = vc[pages].permute(1, 2, 0, 3).flatten(2)[..., :n].float()
         s = torch.matmul(k.repeat_interleave(per, 0),
                          q[r].float()[:, :, None])[..., 0] * p.scale
+        if row_scale is not None:
+            s = s * row_scale[r]
         if p.temp is not None:
             s = s * p.temp[:, None]
         if p.bias is not None:
@@ -98,7 +108,10 @@ def attn_rows(out, q, p, kc, vc, block_tables, row_len, vcs, row_seq):
         if vcs is not None:
             back = vcs[r:r + 1] * torch.tensor([1.0, -1.0])
             o = _turn(o[None], back)[0]
-        out[r] = (p.out_scale * o).reshape(-1).to(out.dtype)
+        o = (p.out_scale * o).reshape(-1)
+        if gate is not None:
+            o = o * torch.sigmoid(gate[r].float())
+        out[r] = o.to(out.dtype)
 
 
 # ------------------------------------------------------ gated linear attention
@@ -120,5 +133,31 @@ def gla_span(y, z, p, w, state, slot, start):
         o = (keep * (q * p.q_scale)[:, :, None]).sum(1)
         o = F.rms_norm(o, (E,), w.norm, p.eps) * F.silu(g)
         y[t] = (p.out_scale * o).reshape(-1).to(y.dtype)
+    if live:
+        state[slot, ..., :E] = keep
+
+
+# --------------------------------------- linear attention, a decay per head
+
+def decay_span(y, z, p, w, state, slot, start):
+    """Tokens of one sequence, as gla_span."""
+    H, D, E = p.heads, p.dim, p.vdim
+    live = slot >= 0
+    keep = state[slot, ..., :E].clone() if live and start > 0 else \
+        torch.zeros(H, D, E)
+
+    def part(at, size):
+        v = F.silu(z[:, at:at + H * size].float()).to(z.dtype)
+        return v.float().unflatten(1, (H, size))
+
+    q, k, v = part(p.q_at, D), part(p.k_at, D), part(p.v_at, E)
+    a = w.decay[:, None, None]
+    o = torch.empty(z.shape[0], H * E)
+    for t in range(z.shape[0]):
+        keep = a * keep + k[t][:, :, None] * v[t][:, None, :]
+        o[t] = (keep * q[t][:, :, None]).sum(1).reshape(-1)
+    g = z[:, p.g_at:p.g_at + H * E].float()
+    o = F.rms_norm(o.to(z.dtype).float(), (H * E,), w.norm, p.eps)
+    y.copy_((o * torch.sigmoid(g)).to(y.dtype))
     if live:
         state[slot, ..., :E] = keep

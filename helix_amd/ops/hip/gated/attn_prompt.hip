@@ -51,17 +51,19 @@ void attn_prompt_kernel(uint16_t* __restrict__ out,
   const int lo = lane & 15, hi = lane >> 4;
   const u16x8 zero = {0, 0, 0, 0, 0, 0, 0, 0};
   u16x8 qf[2][NK];
+  float mul[2];
 #pragma unroll
   for (int u = 0; u < 2; ++u) {
     const int qi = min(q0 + wid * 32 + u * 16 + lo, qlen - 1);
-    const uint16_t* qr = q + ((int64_t)(row0 + qi) * A.H + h) * A.Dp;
+    const uint16_t* qr = q + (row0 + qi) * A.q_stride + h * A.Dp;
 #pragma unroll
     for (int s = 0; s < NK; ++s) {
       const int d = s * 32 + hi * 8;
       qf[u][s] = d < A.Dp ? ld_u16x8(qr + d) : zero;
     }
+    mul[u] = head_mul(A, h) * row_mul(A, row0 + qi);
   }
-  const float mul = head_mul(A, h), add = head_add(A, h);
+  const float add = head_add(A, h);
   const int half = (A.E + 1) / 2;
 
   // Loads without branches, so that all are under way at once: what lies
@@ -148,7 +150,7 @@ void attn_prompt_kernel(uint16_t* __restrict__ out,
       for (int w = 0; w < 2; ++w)
 #pragma unroll
         for (int i = 0; i < 8; ++i) {
-          float v = s[w][i >> 2][u][i & 3] * mul + add;
+          float v = s[w][i >> 2][u][i & 3] * mul[u] + add;
           if (edge) {
             const int key = t + w * 32 + hi * 8 + i;
             if (key > qi || key >= klen) v = NEG;
@@ -221,6 +223,28 @@ void attn_prompt_kernel(uint16_t* __restrict__ out,
         y[i] = acc[d + 1][u][i] * f;
         if (pair + i < half) turn_back(A, r, pair + i, x[i], y[i]);
       }
+      if (A.gate != nullptr) {
+        const int at = h * A.E + pair;
+        const uint16_t* gp = (const uint16_t*)A.gate + r * A.gate_stride + at;
+        if (m.vec) {
+          float gx[4], gy[4];
+          ldv<4>(gp, gx);
+          ldv<4>(gp + half, gy);
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            x[i] *= sigmoid_s<uint16_t>(gx[i]);
+            y[i] *= sigmoid_s<uint16_t>(gy[i]);
+          }
+        } else {
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            if (pair + i >= half) continue;
+            x[i] *= gate_of<uint16_t>(A, r, at + i);
+            if (half + pair + i < A.E)
+              y[i] *= gate_of<uint16_t>(A, r, at + half + i);
+          }
+        }
+      }
       if (m.vec) {
         st_bf16x4(dst + pair, x);
         st_bf16x4(dst + half + pair, y);
@@ -244,14 +268,15 @@ void attn_prompt(torch::Tensor out, torch::Tensor q, torch::Tensor kc,
                  torch::Tensor vc, torch::Tensor bt, torch::Tensor cu,
                  torch::Tensor seq_lens, int64_t max_q, double scale,
                  double out_scale, bool sigmoid, OptT temp, OptT bias,
-                 OptT vcs) {
-  TORCH_CHECK(q.dim() == 3 && q.is_contiguous() &&
-              q.scalar_type() == kc.scalar_type());
+                 OptT vcs, OptT row_scale, OptT gate) {
+  TORCH_CHECK(q.dim() == 3 && q.scalar_type() == kc.scalar_type());
   const int64_t T = q.size(0), H = q.size(1);
   const int B = seq_lens.numel();
   Prompt m{};
-  m.a = attn_args(kc, vc, bt, T, H, scale, out_scale, temp, bias, vcs);
-  TORCH_CHECK(q.size(2) == m.a.Dp && attn_fits(q, m.a.E));
+  m.a = attn_args(kc, vc, bt, T, H, scale, out_scale, temp, bias, vcs,
+                  row_scale, gate);
+  query_rows(m.a, q);
+  TORCH_CHECK(attn_fits(q, m.a.E));
   for (const auto& t : {cu, seq_lens})
     TORCH_CHECK(t.scalar_type() == torch::kInt32 && t.is_contiguous());
   TORCH_CHECK(cu.numel() == B + 1 && bt.size(0) >= B);
@@ -265,7 +290,8 @@ void attn_prompt(torch::Tensor out, torch::Tensor q, torch::Tensor kc,
   m.q_tiles = cdiv((int)max_q, QT);
   m.seqs = B;
   m.vec = m.a.E % 8 == 0 && out.stride(0) % 4 == 0 &&
-          (uintptr_t)out.data_ptr() % 8 == 0;
+          (uintptr_t)out.data_ptr() % 8 == 0 && m.a.gate_stride % 4 == 0 &&
+          (uintptr_t)m.a.gate % 8 == 0;
   const dim3 grid(8 * cdiv(B * H, 8) * m.q_tiles);
 #define HELIX_AP(NK, NV)                                                     \
   do {                                                                       \

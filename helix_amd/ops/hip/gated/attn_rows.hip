@@ -28,6 +28,17 @@ struct Rows {
   int per, parts;              // query heads per key/value head
 };
 
+// Both values of a pair of head h, gated.
+template <typename S>
+__device__ __forceinline__ void store_pair(const Attn& A, S* out, int64_t row,
+                                           int h, int pair, int half, float a,
+                                           float b) {
+  const int at = h * A.E + pair;
+  S* o = out + row * A.out_stride + at;
+  st1(o, a * gate_of<S>(A, row, at));
+  if (half + pair < A.E) st1(o + half, b * gate_of<S>(A, row, at + half));
+}
+
 template <int NK, int NV, bool SIG>
 __global__ __launch_bounds__(NT, NV > 8 ? 1 : 2) void attn_rows_kernel(
     uint16_t* __restrict__ out, const uint16_t* __restrict__ q,
@@ -52,13 +63,13 @@ __global__ __launch_bounds__(NT, NV > 8 ? 1 : 2) void attn_rows_kernel(
 
   const u16x8 zero = {0, 0, 0, 0, 0, 0, 0, 0};
   u16x8 qf[NK];
-  const uint16_t* qr = q + ((int64_t)row * A.H + h0 + min(lo, nh - 1)) * A.Dp;
+  const uint16_t* qr = q + row * A.q_stride + (h0 + min(lo, nh - 1)) * A.Dp;
 #pragma unroll
   for (int c = 0; c < NK; ++c) {
     const int d = c * 32 + hi * 8;
     qf[c] = lo < nh && d < A.Dp ? ld_u16x8(qr + d) : zero;
   }
-  const float mul = head_mul(A, h0 + min(lo, nh - 1));
+  const float mul = head_mul(A, h0 + min(lo, nh - 1)) * row_mul(A, row);
   const float add = head_add(A, h0 + min(lo, nh - 1));
 
   // A lane's keys are in the group of 8 numbered lo / 4 (keys as operand)
@@ -202,9 +213,7 @@ __global__ __launch_bounds__(NT, NV > 8 ? 1 : 2) void attn_rows_kernel(
     }
     const float inv = A.out_scale / ll;
     turn_back(A, row, pair, a, b);
-    uint16_t* o = out + row * A.out_stride + h * A.E;
-    o[pair] = f32_to_bf16(a * inv);
-    if (half + pair < A.E) o[half + pair] = f32_to_bf16(b * inv);
+    store_pair(A, out, row, h, pair, half, a * inv, b * inv);
   }
 }
 
@@ -240,9 +249,7 @@ __global__ __launch_bounds__(NT) void attn_merge_kernel(
   }
   const float inv = A.out_scale / (sig ? 1.f : ll);
   turn_back(A, row, pair, a, b);
-  uint16_t* o = out + row * A.out_stride + h * A.E;
-  o[pair] = f32_to_bf16(a * inv);
-  if (two) o[half + pair] = f32_to_bf16(b * inv);
+  store_pair(A, out, row, h, pair, half, a * inv, b * inv);
 }
 
 // Any size and type: a workgroup per (row, head), a thread per key, then a
@@ -261,10 +268,10 @@ __global__ __launch_bounds__(NT) void attn_plain_kernel(
   const int wid = tid / WAVE, lane = tid & (WAVE - 1);
   const int* bt = A.bt + (int64_t)seq * A.max_blocks;
   for (int d = tid; d < A.Dp; d += NT)
-    qs[d] = ld1(q + ((int64_t)row * A.H + h) * A.Dp + d);
+    qs[d] = ld1(q + row * A.q_stride + h * A.Dp + d);
   for (int e = tid; e < A.E; e += NT) os[e] = 0.f;
   const float mul =
-      A.scale * (A.temp != nullptr ? A.temp[h] : 1.f);
+      A.scale * (A.temp != nullptr ? A.temp[h] : 1.f) * row_mul(A, row);
   const float add = A.bias != nullptr ? A.bias[h] : 0.f;
   float mm = NEG, ll = 0.f;
   for (int t = 0; t < len; t += NT) {
@@ -317,23 +324,20 @@ __global__ __launch_bounds__(NT) void attn_plain_kernel(
   for (int pair = tid; pair < half; pair += NT) {
     float a = os[pair], b = half + pair < A.E ? os[half + pair] : 0.f;
     turn_back(A, row, pair, a, b);
-    S* o = out + row * A.out_stride + h * A.E;
-    st1(o + pair, a * inv);
-    if (half + pair < A.E) st1(o + half + pair, b * inv);
+    store_pair(A, out, row, h, pair, half, a * inv, b * inv);
   }
 }
 
 Rows row_args(const torch::Tensor& q, const torch::Tensor& kc,
               const torch::Tensor& vc, const torch::Tensor& bt, OptT row_seq,
               const torch::Tensor& row_len, double scale, double out_scale,
-              OptT temp, OptT bias, OptT vcs) {
-  TORCH_CHECK(q.dim() == 3 && q.is_contiguous() &&
-              q.scalar_type() == kc.scalar_type());
+              OptT temp, OptT bias, OptT vcs, OptT row_scale, OptT gate) {
+  TORCH_CHECK(q.dim() == 3 && q.scalar_type() == kc.scalar_type());
   const int64_t R = q.size(0);
   Rows m{};
   m.a = attn_args(kc, vc, bt, R, q.size(1), scale, out_scale, temp, bias,
-                  vcs);
-  TORCH_CHECK(q.size(2) == m.a.Dp);
+                  vcs, row_scale, gate);
+  query_rows(m.a, q);
   TORCH_CHECK(row_len.scalar_type() == torch::kInt32 &&
               row_len.is_contiguous() && row_len.numel() == R);
   m.row_len = row_len.data_ptr<int>();
@@ -394,9 +398,9 @@ void attn_rows(OptT out, OptT part, OptT ml, torch::Tensor q,
                torch::Tensor kc, torch::Tensor vc, torch::Tensor bt,
                OptT row_seq, torch::Tensor row_len, double scale,
                double out_scale, bool sigmoid, OptT temp, OptT bias,
-               OptT vcs) {
+               OptT vcs, OptT row_scale, OptT gate) {
   Rows m = row_args(q, kc, vc, bt, row_seq, row_len, scale, out_scale, temp,
-                    bias, vcs);
+                    bias, vcs, row_scale, gate);
   TORCH_CHECK(attn_fits(q, m.a.E));
   TORCH_CHECK(out.has_value() != part.has_value());
   uint16_t* o = nullptr;
@@ -421,7 +425,7 @@ void attn_rows(OptT out, OptT part, OptT ml, torch::Tensor q,
 }
 
 void attn_merge(torch::Tensor out, torch::Tensor part, torch::Tensor ml,
-                double out_scale, bool sigmoid, OptT vcs) {
+                double out_scale, bool sigmoid, OptT vcs, OptT gate) {
   Rows m{};
   TORCH_CHECK(part.dim() == 4 && part.is_contiguous() && ml.is_contiguous() &&
               part.scalar_type() == torch::kFloat32 &&
@@ -434,11 +438,7 @@ void attn_merge(torch::Tensor out, torch::Tensor part, torch::Tensor ml,
   TORCH_CHECK(out.dim() == 2 && out.size(0) == R &&
               out.size(1) == m.a.H * m.a.E && out.stride(1) == 1 &&
               out.scalar_type() == torch::kBFloat16);
-  if (vcs.has_value()) {
-    TORCH_CHECK(m.a.E % 2 == 0 && vcs->scalar_type() == torch::kFloat32 &&
-                vcs->is_contiguous() && vcs->numel() == R * m.a.E);
-    m.a.vcs = (const float2*)vcs->data_ptr<float>();
-  }
+  row_operands(m.a, R, torch::kBFloat16, vcs, gate);
   m.a.out_stride = out.stride(0);
   m.a.out_scale = (float)out_scale;
   m.part = part.data_ptr<float>();
@@ -453,9 +453,10 @@ void attn_merge(torch::Tensor out, torch::Tensor part, torch::Tensor ml,
 void attn_plain(torch::Tensor out, torch::Tensor q, torch::Tensor kc,
                 torch::Tensor vc, torch::Tensor bt, OptT row_seq,
                 torch::Tensor row_len, double scale, double out_scale,
-                bool sigmoid, OptT temp, OptT bias, OptT vcs) {
+                bool sigmoid, OptT temp, OptT bias, OptT vcs,
+                OptT row_scale, OptT gate) {
   Rows m = row_args(q, kc, vc, bt, row_seq, row_len, scale, out_scale, temp,
-                    bias, vcs);
+                    bias, vcs, row_scale, gate);
   set_out(m, out, q);
   if (q.size(0) == 0) return;
   const int lds = (m.a.Dp + NT + m.a.E) * sizeof(float);

@@ -37,6 +37,7 @@ struct Epilogue {
   const int64_t* slots;
   int64_t z_stride, T;
   int q_at, k_at, v_at, H, G, D, Dp, E, nk, nv, bs, per;
+  int q_rows, kv_rows;         // tokens whose queries / keys are wanted
   float eps;
 };
 
@@ -116,7 +117,7 @@ __device__ __forceinline__ int units_of(int D, int n, int N) {
 
 constexpr int PER = 16;                       // tokens of a workgroup at most
 
-// The first T workgroups have a token's queries each, the others keys and
+// The first q_rows workgroups have a token's queries each, the others keys and
 // values of `per` neighbouring tokens. Values go out token by token of one
 // dimension, so that a page's 16-byte runs are written at once.
 template <typename S, int N>
@@ -126,7 +127,7 @@ __global__ __launch_bounds__(NT) void attn_epilogue_kernel(
   __shared__ float red[16], invs[PER];
   __shared__ int64_t slots[PER];
   const int pad = m.Dp - m.D;
-  if (blockIdx.x < m.T) {
+  if ((int)blockIdx.x < m.q_rows) {
     const int64_t t = blockIdx.x;
     const S* zq = z + t * m.z_stride + m.q_at;
     float inv = 1.f;
@@ -144,7 +145,7 @@ __global__ __launch_bounds__(NT) void attn_epilogue_kernel(
       st1(qt + i / pad * m.Dp + m.D + i % pad, 0.f);
     return;
   }
-  const int64_t t0 = (blockIdx.x - m.T) * m.per;
+  const int64_t t0 = (int64_t)(blockIdx.x - m.q_rows) * m.per;
   const int nt = (int)min((int64_t)m.per, m.T - t0);
   if ((int)threadIdx.x < nt) slots[threadIdx.x] = m.slots[t0 + threadIdx.x];
   if (m.kw != nullptr) {
@@ -199,18 +200,30 @@ __global__ __launch_bounds__(NT) void attn_epilogue_kernel(
   }
 }
 
+// fp32: factor of a query's scores by its position,
+// 1 + coef * ln(floor((p + 1) / every) + 1).
+__global__ void query_temperature_kernel(float* __restrict__ out,
+                                         const int64_t* __restrict__ pos,
+                                         float coef, double every, int T) {
+  const int t = blockIdx.x * NT + threadIdx.x;
+  if (t >= T) return;
+  const double n = floor((double)(pos[t] + 1) / every) + 1.0;
+  out[t] = 1.f + coef * logf((float)n);
+}
+
 template <typename S>
-void launch(torch::Tensor q, torch::Tensor kc, torch::Tensor vc,
+void launch(OptT q, torch::Tensor kc, torch::Tensor vc,
             torch::Tensor z, Epilogue m) {
   auto stream = at::hip::getCurrentHIPStream();
-  const dim3 grid(m.T + (m.T + m.per - 1) / m.per);
+  const dim3 grid(m.q_rows + (m.kv_rows + m.per - 1) / m.per);
+  S* qp = q.has_value() ? (S*)q->data_ptr() : nullptr;
   const bool vec = m.nk % 8 == 0 && m.nv % 8 == 0 && m.D % 8 == 0 &&
                    m.E % 8 == 0 && m.q_at % 8 == 0 && m.k_at % 8 == 0 &&
                    m.v_at % 8 == 0 && m.z_stride % 8 == 0 &&
                    (uintptr_t)z.data_ptr() % 16 == 0;
 #define HELIX_EP(N)                                                          \
   hipLaunchKernelGGL((attn_epilogue_kernel<S, N>), grid, dim3(NT), 0,        \
-                     stream, (S*)q.data_ptr(), (S*)kc.data_ptr(),            \
+                     stream, qp, (S*)kc.data_ptr(),                          \
                      (S*)vc.data_ptr(), (const S*)z.data_ptr(), m)
   if (vec) HELIX_EP(8);
   else HELIX_EP(1);
@@ -250,26 +263,48 @@ void rotary_table(torch::Tensor cs, torch::Tensor pos, torch::Tensor freqs) {
                      freqs.data_ptr<double>(), (int)n, total);
 }
 
-void attn_epilogue(torch::Tensor q, torch::Tensor kc, torch::Tensor vc,
+void query_temperature(torch::Tensor out, torch::Tensor pos, double coef,
+                       double every) {
+  const int T = pos.numel();
+  TORCH_CHECK(out.scalar_type() == torch::kFloat32 && out.is_contiguous() &&
+              out.numel() == T && every > 0);
+  TORCH_CHECK(pos.scalar_type() == torch::kInt64 && pos.is_contiguous());
+  if (T == 0) return;
+  hipLaunchKernelGGL(query_temperature_kernel, dim3((T + NT - 1) / NT),
+                     dim3(NT), 0, at::hip::getCurrentHIPStream(),
+                     out.data_ptr<float>(), pos.data_ptr<int64_t>(),
+                     (float)coef, every, T);
+}
+
+void attn_epilogue(OptT q, torch::Tensor kc, torch::Tensor vc,
                    torch::Tensor z, int64_t q_at, int64_t k_at, int64_t v_at,
-                   int64_t dim, torch::Tensor slots, OptT cs, OptT vcs,
-                   OptT qw, OptT kw, double eps) {
+                   int64_t heads, int64_t dim, torch::Tensor slots, OptT cs,
+                   OptT vcs, OptT qw, OptT kw, double eps, bool write_kv) {
   Epilogue m{};
-  TORCH_CHECK(q.dim() == 3 && kc.dim() == 4 && vc.dim() == 4);
+  TORCH_CHECK(kc.dim() == 4 && vc.dim() == 4);
   m.T = z.size(0);
-  m.H = q.size(1);
-  m.Dp = q.size(2);
+  m.H = heads;
+  m.Dp = kc.size(3);
+  m.q_rows = q.has_value() ? m.T : 0;
+  m.kv_rows = write_kv ? m.T : 0;
   m.G = kc.size(1);
   m.bs = kc.size(2);
   m.E = vc.size(2);
   m.D = dim;
-  TORCH_CHECK(m.Dp % 8 == 0 && dim > 0 && dim <= m.Dp && q.size(0) == m.T);
-  TORCH_CHECK(kc.size(3) == m.Dp && vc.size(0) == kc.size(0) &&
-              vc.size(1) == m.G && vc.size(3) == m.bs);
-  for (const auto& t : {q, kc, vc})
+  TORCH_CHECK(m.Dp % 8 == 0 && dim > 0 && dim <= m.Dp);
+  TORCH_CHECK(vc.size(0) == kc.size(0) && vc.size(1) == m.G &&
+              vc.size(3) == m.bs);
+  if (q.has_value())
+    TORCH_CHECK(q->dim() == 3 && q->size(0) == m.T && q->size(1) == m.H &&
+                q->size(2) == m.Dp && q->is_contiguous() &&
+                q->scalar_type() == z.scalar_type());
+  for (const auto& t : {kc, vc})
     TORCH_CHECK(t.is_contiguous() && t.scalar_type() == z.scalar_type());
-  TORCH_CHECK(z.stride(1) == 1 && q_at + m.H * dim <= z.size(1) &&
-              k_at + m.G * dim <= z.size(1) && v_at + m.G * m.E <= z.size(1));
+  TORCH_CHECK(z.stride(1) == 1);
+  if (q.has_value()) TORCH_CHECK(q_at + m.H * dim <= z.size(1));
+  if (write_kv)
+    TORCH_CHECK(k_at >= 0 && k_at + m.G * dim <= z.size(1) && v_at >= 0 &&
+                v_at + m.G * m.E <= z.size(1));
   TORCH_CHECK(slots.scalar_type() == torch::kInt64 && slots.numel() == m.T &&
               slots.is_contiguous());
   m.cs = table(cs, m.T, m.nk);
@@ -283,7 +318,7 @@ void attn_epilogue(torch::Tensor q, torch::Tensor kc, torch::Tensor vc,
   m.k_at = k_at;
   m.v_at = v_at;
   m.eps = (float)eps;
-  if (m.T == 0) return;
+  if (m.q_rows + m.kv_rows == 0) return;
   m.per = m.T > 1024 ? PER : 1;
   if (z.scalar_type() == torch::kBFloat16) launch<uint16_t>(q, kc, vc, z, m);
   else if (z.scalar_type() == torch::kFloat32) launch<float>(q, kc, vc, z, m);

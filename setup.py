@@ -38,7 +38,8 @@ def extension(name, folder):
 
 EXTENSIONS = {"_C": HIP_DIR, "_C_ext": os.path.join(HIP_DIR, "ext"),
               "_C_hybrid": os.path.join(HIP_DIR, "hybrid"),
-              "_C_gated": os.path.join(HIP_DIR, "gated")}
+              "_C_gated": os.path.join(HIP_DIR, "gated"),
+              "_C_routed": os.path.join(HIP_DIR, "routed")}
 only = [n for n in os.environ.get("HELIX_BUILD_ONLY", "").split(",") if n]
 
 setup(
