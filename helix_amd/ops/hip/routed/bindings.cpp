@@ -18,6 +18,7 @@ void route(T ids, T weights, T rank, T hist, T z, T correction,
 void place(T order, T slot, T tiles, T ids, T rank, T hist, int64_t per,
            int64_t height);
 bool experts_fit(T a, T w);
+int64_t expert_tile_rows();
 void expert_product(T out, T a, T w, T tiles, OptT order, int64_t choices,
                     int64_t height, bool relu2, bool plain);
 void conv_silu(T out, T z, int64_t x_at, T conv, T bias, T ring, T slots,
@@ -40,6 +41,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("route", &route, "Choice of experts per token");
   m.def("place", &place, "Experts' token lists and tiles");
   m.def("experts_fit", &experts_fit);
+  m.def("expert_tile_rows", &expert_tile_rows);
   m.def("expert_product", &expert_product, "All experts' matrix products");
   m.def("conv_silu", &conv_silu, "Short causal convolution and silu");
   m.def("scan_max_state", &scan_max_state);

@@ -57,6 +57,8 @@ DEFAULT_SPECS = {
     "nibezen-1b": ModelSpec("nibezen-1b", "llm", "nibezen-1b"),
     "motolix-8b": ModelSpec("motolix-8b", "llm", "motolix-8b"),
     "motolix-1b": ModelSpec("motolix-1b", "llm", "motolix-1b"),
+    "dibizen-28b": ModelSpec("dibizen-28b", "llm", "dibizen-28b"),
+    "dibizen-3b": ModelSpec("dibizen-3b", "llm", "dibizen-3b"),
     "bge-base": ModelSpec("bge-base", "embedding", "bge-base"),
     "siglip-base": ModelSpec("siglip-base", "vision", "siglip-base"),
     "tiny-vit": ModelSpec("tiny-vit", "vision", "tiny-vit"),
@@ -73,6 +75,8 @@ DEFAULT_SPECS = {
     "tiny-nibezen": ModelSpec("tiny-nibezen", "llm", "tiny-nibezen",
                               max_model_len=256, kv_cache_blocks=256),
     "tiny-motolix": ModelSpec("tiny-motolix", "llm", "tiny-motolix",
+                              max_model_len=256, kv_cache_blocks=256),
+    "tiny-dibizen": ModelSpec("tiny-dibizen", "llm", "tiny-dibizen",
                               max_model_len=256, kv_cache_blocks=256),
     "tiny-bert": ModelSpec("tiny-bert", "embedding", "tiny-bert"),
 }

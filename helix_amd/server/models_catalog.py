@@ -42,6 +42,12 @@ STATIC_MODEL_INFO: Dict[str, dict] = {
     "motolix-1b": {"context_length": 32768, "prompt_price_per_m": 0.02,
                    "completion_price_per_m": 0.04, "family": "motolix",
                    "runtime": "helix_amd", "kind": "chat"},
+    "dibizen-28b": {"context_length": 32768, "prompt_price_per_m": 0.08,
+                    "completion_price_per_m": 0.16, "family": "dibizen",
+                    "runtime": "helix_amd", "kind": "chat"},
+    "dibizen-3b": {"context_length": 32768, "prompt_price_per_m": 0.02,
+                   "completion_price_per_m": 0.04, "family": "dibizen",
+                   "runtime": "helix_amd", "kind": "chat"},
     "bge-base": {"context_length": 512, "prompt_price_per_m": 0.005,
                  "completion_price_per_m": 0.0, "family": "bge",
                  "runtime": "helix_amd", "kind": "embedding"},
