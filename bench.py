@@ -137,15 +137,15 @@ def run_coresident(args) -> None:
 
 
 def run_design(args) -> None:
-    """Prefill / decode throughput of Zederax, Nibezen or Motolix presets and
-    of equally large Llama models, and kernel by kernel distance from the
-    roofline."""
+    """Prefill / decode throughput of Zederax, Nibezen, Motolix or Dibizen
+    presets and of equally large Llama models, and kernel by kernel distance
+    from the roofline."""
     from helix_amd.engine import design_bench
     names = args.design.split(",")
     res = design_bench.run(names, "cuda:0", min(args.steps, 32),
                            args.design_part)
     first = next((v for k, v in res[names[0]].items()
-                  if k in ("zederax", "nibezen", "motolix")), None)
+                  if k in ("zederax", "nibezen", "motolix", "dibizen")), None)
     print(json.dumps({
         "metric": "tokens/sec (design)",
         "value": first[-1]["decode_tok_s"] if first else None,
@@ -180,8 +180,8 @@ def main():
     ap.add_argument("--top-p", type=float, default=1.0)
     ap.add_argument("--design", type=str, default="",
                     help="instead of the headline: comma-separated Zederax, "
-                         "Nibezen or Motolix presets, each beside a Llama of "
-                         "equal size")
+                         "Nibezen, Motolix or Dibizen presets, each beside a "
+                         "Llama of equal size")
     ap.add_argument("--design-part", type=str, default="all",
                     choices=["all", "throughput", "kernels"])
     args = ap.parse_args()

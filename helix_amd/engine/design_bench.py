@@ -226,11 +226,14 @@ def zederax_kernels(z: ZederaxConfig, device, decode_batch: int = 256,
 def _families():
     from helix_amd.engine import design_bench_gated as gated
     from helix_amd.engine import design_bench_hybrid as hybrid
+    from helix_amd.engine import design_bench_routed as routed
+    from helix_amd.models.dibizen import DibizenConfig
     from helix_amd.models.motolix import MotolixConfig
     from helix_amd.models.nibezen import NibezenConfig
     return {ZederaxConfig: ("zederax", zederax_twin, zederax_kernels),
             NibezenConfig: ("nibezen", hybrid.twin, hybrid.kernels),
-            MotolixConfig: ("motolix", gated.twin, gated.kernels)}
+            MotolixConfig: ("motolix", gated.twin, gated.kernels),
+            DibizenConfig: ("dibizen", routed.twin, routed.kernels)}
 
 
 def run(names: List[str], device: str, steps: int, what: str) -> dict:

@@ -75,11 +75,12 @@ class SelectiveScan(Float32Kept):
         s = self.spec = spec
         I, N = s.inner, s.state
         b_at = round_up(s.dt_rank, 8)
-        c_at = round_up(b_at + N, 8)
+        c_at = b_at + routed.state_columns(N)
         self.params = routed.ScanParams(
             I, N, s.conv, s.dt_rank, x_at=at["in"], z_at=at["in"] + I,
             b_at=b_at, c_at=c_at)
-        self.x_w = nn.Parameter(torch.zeros(round_up(c_at + N, 32), I))
+        self.x_w = nn.Parameter(torch.zeros(
+            round_up(self.params.columns, 32), I))
         self.dt_w = nn.Parameter(torch.zeros(I, s.dt_rank))
         self.dt_b = nn.Parameter(torch.zeros(I))
         self.conv_w = nn.Parameter(torch.zeros(s.conv, I))

@@ -18,12 +18,12 @@ void route(T ids, T weights, T rank, T hist, T z, T correction,
 void place(T order, T slot, T tiles, T ids, T rank, T hist, int64_t per,
            int64_t height);
 bool experts_fit(T a, T w);
-int64_t expert_tile_rows();
 void expert_product(T out, T a, T w, T tiles, OptT order, int64_t choices,
-                    int64_t height, bool relu2, bool plain);
+                    int64_t height, const std::string& kind, bool relu2);
 void conv_silu(T out, T z, int64_t x_at, T conv, T bias, T ring, T slots,
                T pos, OptT cu, int64_t max_len);
 int64_t scan_max_state();
+int64_t scan_columns(int64_t N);
 void scan_step(T y, T x, T z, int64_t z_at, T dt, T bias, T bc, int64_t b_at,
                int64_t c_at, T A, T D, T state, T slots, T pos);
 void scan_prompt(T y, T x, T z, int64_t z_at, T dt, T bias, T bc,
@@ -41,10 +41,10 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("route", &route, "Choice of experts per token");
   m.def("place", &place, "Experts' token lists and tiles");
   m.def("experts_fit", &experts_fit);
-  m.def("expert_tile_rows", &expert_tile_rows);
   m.def("expert_product", &expert_product, "All experts' matrix products");
   m.def("conv_silu", &conv_silu, "Short causal convolution and silu");
   m.def("scan_max_state", &scan_max_state);
+  m.def("scan_columns", &scan_columns);
   m.def("scan_step", &scan_step, "Selective scan of single tokens");
   m.def("scan_prompt", &scan_prompt, "Selective scan of prompt portions");
 }

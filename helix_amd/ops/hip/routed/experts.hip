@@ -6,12 +6,11 @@
 // that of the list itself, or (gather) of the token a list entry belongs to.
 // act: none, or the square of relu.
 //
-// bf16 comes in two shapes. Few rows per expert (decoding): the weights are
-// the traffic, so a wave streams them straight into MFMA operands, the waves
-// of a workgroup share the inner dimension and meet in LDS at the end. Many
-// rows: tiles of 128 x 128 through LDS, filled by direct loads; 16-byte
-// pieces of a row are stored crosswise (piece ^ row % 8), so that operands
-// leave LDS without bank conflicts. fp32 and odd sizes run a plain kernel.
+// bf16 comes in two shapes. A row or two per expert: a wave streams weights
+// straight into MFMA operands, the waves of a workgroup share the inner
+// dimension and meet in LDS at the end. More: tiles through LDS, filled by
+// direct loads; 16-byte pieces of a row are stored crosswise (piece ^ row % 8),
+// so that operands leave LDS without bank conflicts. fp32 and odd sizes run a plain kernel.
 #include "../hybrid/tile.h"
 #include <torch/extension.h>
 #include <ATen/hip/HIPContext.h>
@@ -47,7 +46,7 @@ __device__ __forceinline__ int xcd_chunk(int orig, int nwg) {
   return (xcd < r ? xcd * (q + 1) : r * (q + 1) + (xcd - r) * q) + pos;
 }
 
-// --- few rows: 16 MI rows x 16 NI columns of a workgroup; a wave has every
+// --- streams: 16 MI rows x 16 NI columns of a workgroup; a wave has every
 // fourth stretch of 32 U of the inner dimension.
 template <int MI, int NI, int U>
 __global__ __launch_bounds__(NT) void expert_rows_kernel(
@@ -145,77 +144,96 @@ __global__ __launch_bounds__(NT) void expert_rows_kernel(
   }
 }
 
-// --- many rows: 128 x 128, inner dimension in steps of 64 (K % 64 == 0).
-constexpr int BT = 128, BK = 64;
+// --- tiles: BM x BN of a workgroup, WM x WN waves, inner dimension in
+// steps of 64 (K % 64 == 0). The next step's tiles are on their way to one
+// half of LDS while the other is worked on.
+constexpr int BK = 64;
 
-__global__ __launch_bounds__(NT) void expert_tiles_kernel(
+template <int BM, int BN, int WM, int WN>
+__global__ __launch_bounds__(WM* WN* WAVE) void expert_tiles_kernel(
     uint16_t* __restrict__ out, const uint16_t* __restrict__ a,
     const uint16_t* __restrict__ w, Mix m) {
-  __shared__ __attribute__((aligned(16))) uint16_t al[BT * BK];
-  __shared__ __attribute__((aligned(16))) uint16_t wl[BT * BK];
+  constexpr int TH = WM * WN * WAVE;
+  constexpr int MI = BM / WM / 16, NI = BN / WN / 16;
+  constexpr int AT = BM * BK / (TH * 8), WT = BN * BK / (TH * 8);
+  extern __shared__ __attribute__((aligned(16))) uint16_t lds[];
   const int lin = xcd_chunk(blockIdx.x, gridDim.x);
   const int4 tile = m.tiles[lin / m.n_tiles];
   if (tile.x < 0) return;
-  const int n0 = lin % m.n_tiles * BT;
+  const int n0 = lin % m.n_tiles * BN;
   const int tid = threadIdx.x, wid = tid / WAVE, lane = tid & (WAVE - 1);
   const int lo = lane & 15, hi = lane >> 4;
-  const int wr = wid >> 1, wc = wid & 1;      // 64 rows x 64 columns each
+  const int wr = wid / WN, wc = wid % WN;
 
-  // this thread's four 16-byte pieces of either tile
-  constexpr int ITS = BT * BK / (NT * 8);
-  const uint16_t *ap[ITS], *wp[ITS];
+  // this thread's 16-byte pieces of either tile
+  const uint16_t *ap[AT], *wp[WT];
+  const int row0 = tid / 8;
 #pragma unroll
-  for (int it = 0; it < ITS; ++it) {
-    const int row = it * (NT / 8) + tid / 8;
-    const int col = ((tid & 7) ^ (row & 7)) * 8;
-    ap[it] = a + source_row(m, tile.y + min(row, tile.z - 1)) * m.a_stride +
-             col;
-    wp[it] = w + ((int64_t)tile.x * m.N + min(n0 + row, m.N - 1)) * m.K + col;
+  for (int i = 0; i < AT; ++i) {
+    const int row = i * (TH / 8) + row0;
+    ap[i] = a + source_row(m, tile.y + min(row, tile.z - 1)) * m.a_stride +
+            ((tid & 7) ^ (row & 7)) * 8;
   }
-  floatx4 acc[4][4];
 #pragma unroll
-  for (int j = 0; j < 4; ++j)
+  for (int i = 0; i < WT; ++i) {
+    const int row = i * (TH / 8) + row0;
+    wp[i] = w + ((int64_t)tile.x * m.N + min(n0 + row, m.N - 1)) * m.K +
+            ((tid & 7) ^ (row & 7)) * 8;
+  }
+  auto load = [&](int k0, uint16_t* dst) {
 #pragma unroll
-    for (int i = 0; i < 4; ++i) acc[j][i] = floatx4{0, 0, 0, 0};
+    for (int i = 0; i < AT; ++i)
+      __builtin_amdgcn_global_load_lds(
+          (const __attribute__((address_space(1))) uint32_t*)(ap[i] + k0),
+          (__attribute__((address_space(3))) uint32_t*)(dst +
+                                                        (i * TH + tid) * 8),
+          16, 0, 0);
+#pragma unroll
+    for (int i = 0; i < WT; ++i)
+      __builtin_amdgcn_global_load_lds(
+          (const __attribute__((address_space(1))) uint32_t*)(wp[i] + k0),
+          (__attribute__((address_space(3))) uint32_t*)(
+              dst + BM * BK + (i * TH + tid) * 8),
+          16, 0, 0);
+  };
+  floatx4 acc[NI][MI];
+#pragma unroll
+  for (int j = 0; j < NI; ++j)
+#pragma unroll
+    for (int i = 0; i < MI; ++i) acc[j][i] = floatx4{0, 0, 0, 0};
 
-  for (int k0 = 0; k0 < m.K; k0 += BK) {
-    __syncthreads();
-#pragma unroll
-    for (int it = 0; it < ITS; ++it) {
-      const int e = (it * NT + tid) * 8;
-      __builtin_amdgcn_global_load_lds(
-          (const __attribute__((address_space(1))) uint32_t*)(ap[it] + k0),
-          (__attribute__((address_space(3))) uint32_t*)(al + e), 16, 0, 0);
-      __builtin_amdgcn_global_load_lds(
-          (const __attribute__((address_space(1))) uint32_t*)(wp[it] + k0),
-          (__attribute__((address_space(3))) uint32_t*)(wl + e), 16, 0, 0);
-    }
+  constexpr int HALF = (BM + BN) * BK;
+  load(0, lds);
+  for (int k0 = 0, cur = 0; k0 < m.K; k0 += BK, cur ^= 1) {
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     __syncthreads();
+    if (k0 + BK < m.K) load(k0 + BK, lds + (cur ^ 1) * HALF);
+    const uint16_t* al = lds + cur * HALF + (wr * MI * 16 + lo) * BK;
+    const uint16_t* wl = lds + cur * HALF + (BM + wc * NI * 16 + lo) * BK;
 #pragma unroll
     for (int kk = 0; kk < BK / 32; ++kk) {
       const int piece = ((kk * 4 + hi) ^ (lo & 7)) * 8;
-      u16x8 af[4], wf[4];
+      u16x8 af[MI], wf[NI];
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        af[i] = ld_u16x8(al + (wr * 64 + i * 16 + lo) * BK + piece);
-        wf[i] = ld_u16x8(wl + (wc * 64 + i * 16 + lo) * BK + piece);
-      }
+      for (int i = 0; i < MI; ++i) af[i] = ld_u16x8(al + i * 16 * BK + piece);
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
+      for (int j = 0; j < NI; ++j) wf[j] = ld_u16x8(wl + j * 16 * BK + piece);
 #pragma unroll
-        for (int i = 0; i < 4; ++i) acc[j][i] = mfma16(wf[j], af[i], acc[j][i]);
+      for (int j = 0; j < NI; ++j)
+#pragma unroll
+        for (int i = 0; i < MI; ++i)
+          acc[j][i] = mfma16(wf[j], af[i], acc[j][i]);
     }
   }
   // lane: columns 4 hi + r of row lo
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int r = wr * 64 + i * 16 + lo;
+  for (int i = 0; i < MI; ++i) {
+    const int r = (wr * MI + i) * 16 + lo;
     if (r >= tile.z) continue;
     uint16_t* o = out + (int64_t)(tile.y + r) * m.N;
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      const int c = n0 + wc * 64 + j * 16 + hi * 4;
+    for (int j = 0; j < NI; ++j) {
+      const int c = n0 + (wc * NI + j) * 16 + hi * 4;
       if (m.N % 4 == 0) {
         const float v[4] = {finish(m, acc[j][i][0]), finish(m, acc[j][i][1]),
                             finish(m, acc[j][i][2]), finish(m, acc[j][i][3])};
@@ -227,6 +245,23 @@ __global__ __launch_bounds__(NT) void expert_tiles_kernel(
       }
     }
   }
+}
+
+template <int BM, int BN, int WM, int WN>
+void launch_tiles(torch::Tensor out, torch::Tensor a, torch::Tensor w,
+                  Mix m) {
+  static const hipError_t big = hipFuncSetAttribute(
+      (const void*)expert_tiles_kernel<BM, BN, WM, WN>,
+      hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+  TORCH_CHECK(big == hipSuccess, "LDS size refused");
+  m.n_tiles = cdiv(m.N, BN);
+  hipLaunchKernelGGL((expert_tiles_kernel<BM, BN, WM, WN>),
+                     dim3(m.n_tiles * m.m_tiles), dim3(WM * WN * WAVE),
+                     2 * (BM + BN) * BK * 2,
+                     at::hip::getCurrentHIPStream(),
+                     (uint16_t*)out.data_ptr(),
+                     (const uint16_t*)a.data_ptr(),
+                     (const uint16_t*)w.data_ptr(), m);
 }
 
 // --- any size and type: 32 x 32, fp32 inside.
@@ -279,13 +314,11 @@ bool experts_fit(torch::Tensor a, torch::Tensor w) {
          a.stride(0) % 8 == 0 && (uintptr_t)a.data_ptr() % 16 == 0;
 }
 
-int64_t expert_tile_rows() { return BT; }
-
-// tiles [n, 4] of at most `height` rows: 16, 32 or 64 (few rows), 128 (many
-// rows; w.size(2) % 64 == 0), or 32 with plain.
+// tiles [n, 4] of at most `height` rows. kind: "stream" (height 32 or 64),
+// "tile" (32, 64, 128 or 256; w.size(2) % 64 == 0), "plain" (32).
 void expert_product(torch::Tensor out, torch::Tensor a, torch::Tensor w,
                     torch::Tensor tiles, OptT order, int64_t choices,
-                    int64_t height, bool relu2, bool plain) {
+                    int64_t height, const std::string& kind, bool relu2) {
   TORCH_CHECK(out.dim() == 2 && a.dim() == 2 && w.dim() == 3);
   Mix m{};
   m.N = w.size(1);
@@ -320,7 +353,7 @@ void expert_product(torch::Tensor out, torch::Tensor a, torch::Tensor w,
                        stream, (S*)out.data_ptr(), (const S*)a.data_ptr(),   \
                        (const S*)w.data_ptr(), m);                           \
   } while (0)
-  if (plain) {
+  if (kind == "plain") {
     TORCH_CHECK(height == PT);
     if (a.scalar_type() == torch::kBFloat16)
       HELIX_MIX((expert_plain_kernel<uint16_t>), uint16_t, PT);
@@ -332,16 +365,21 @@ void expert_product(torch::Tensor out, torch::Tensor a, torch::Tensor w,
   }
   TORCH_CHECK(experts_fit(a, w) && (uintptr_t)w.data_ptr() % 16 == 0 &&
               (uintptr_t)out.data_ptr() % 8 == 0);
-  if (height == BT) {
-    TORCH_CHECK(m.K % BK == 0);
-    HELIX_MIX(expert_tiles_kernel, uint16_t, BT);
-  } else if (height == 64) {
+  if (kind == "tile") {
+    TORCH_CHECK(m.K % BK == 0, "inner size ", m.K);
+    if (height == 256) launch_tiles<256, 256, 2, 4>(out, a, w, m);
+    else if (height == 128) launch_tiles<128, 128, 2, 2>(out, a, w, m);
+    else if (height == 64) launch_tiles<64, 128, 1, 4>(out, a, w, m);
+    else if (height == 32) launch_tiles<32, 128, 1, 4>(out, a, w, m);
+    else TORCH_CHECK(false, "tiles of ", height, " rows");
+    return;
+  }
+  TORCH_CHECK(kind == "stream", kind);
+  if (height == 64) {
     HELIX_MIX((expert_rows_kernel<4, 2, 2>), uint16_t, 32);
-  } else if (height == 32) {
-    HELIX_MIX((expert_rows_kernel<2, 2, 2>), uint16_t, 32);
   } else {
-    TORCH_CHECK(height == 16, "tiles of ", height, " rows");
-    HELIX_MIX((expert_rows_kernel<1, 2, 4>), uint16_t, 32);
+    TORCH_CHECK(height == 32, "streams of ", height, " rows");
+    HELIX_MIX((expert_rows_kernel<2, 2, 2>), uint16_t, 32);
   }
 #undef HELIX_MIX
 }

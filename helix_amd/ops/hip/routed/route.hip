@@ -3,7 +3,8 @@
 // route: softmax over all router outputs (fp32). Choice scores have a
 // correction on top; only experts of the best groups can be chosen; the
 // weights are the uncorrected scores of the chosen, normalised. A wave has a
-// token. Each workgroup also counts its tokens per expert and numbers them.
+// token at a time. Each workgroup also counts its tokens per expert and
+// numbers them.
 //
 // place: a (token, choice) pair's row in the experts' common list, from the
 // counts of all workgroups; no global atomics, nothing to clear. The list is
@@ -19,6 +20,7 @@ namespace {
 constexpr int NT = 256, NW = NT / WAVE;
 constexpr int MAX_OUTPUTS = 1024;             // router outputs
 constexpr int PER = MAX_OUTPUTS / NT;
+constexpr int MANY = 1024;                    // threads, many tokens
 
 struct Route {
   int* ids;                    // [T, K]
@@ -30,27 +32,19 @@ struct Route {
   int T, n, E, K, groups, size, keep, per;
 };
 
-// best (value, index), the lower index among equals
-__device__ __forceinline__ void take_better(float& v, int& i, float w,
-                                            int j) {
-  if (w > v || (w == v && j < i)) {
-    v = w;
-    i = j;
-  }
-}
-
 // NJ: router outputs per lane
 template <int NJ>
-__global__ __launch_bounds__(NT) void route_kernel(Route m) {
+__global__ __launch_bounds__(MANY) void route_kernel(Route m) {
   extern __shared__ float sh[];
   const int wid = threadIdx.x / WAVE, lane = threadIdx.x & (WAVE - 1);
+  const int nw = blockDim.x / WAVE;
   float* choice = sh + wid * m.n;
-  float* score = sh + (NW + wid) * m.n;
-  float* best = sh + 2 * NW * m.n + wid * m.groups;
-  int* count = (int*)(sh + 2 * NW * m.n + NW * m.groups);
-  for (int e = threadIdx.x; e < m.E; e += NT) count[e] = 0;
+  float* score = sh + (nw + wid) * m.n;
+  float* best = sh + 2 * nw * m.n + wid * m.groups;
+  int* count = (int*)(sh + 2 * nw * m.n + nw * m.groups);
+  for (int e = threadIdx.x; e < m.E; e += blockDim.x) count[e] = 0;
   const int first = blockIdx.x * m.per;
-  for (int i = 0; i < m.per; i += NW) {
+  for (int i = 0; i < m.per; i += nw) {
     const int t = first + i + wid;
     const bool live = i + wid < m.per && t < m.T;
     const float* z = m.z + (int64_t)min(t, m.T - 1) * m.z_stride;
@@ -102,17 +96,16 @@ __global__ __launch_bounds__(NT) void route_kernel(Route m) {
     int mine = 0;
     float weight = 0.f, total = 0.f;
     for (int k = 0; k < m.K; ++k) {
-      float v = -INFINITY;
-      int at = 1 << 30;
+      float v = c[0];
 #pragma unroll
-      for (int j = 0; j < NJ; ++j) take_better(v, at, c[j], j * WAVE + lane);
+      for (int j = 1; j < NJ; ++j) v = fmaxf(v, c[j]);
+      v = wave_reduce_max(v);
+      int at = m.n - 1;                       // whatever the scores are
 #pragma unroll
-      for (int off = 32; off > 0; off >>= 1) {
-        const float w = __shfl_xor(v, off, WAVE);
-        const int o = __shfl_xor(at, off, WAVE);
-        take_better(v, at, w, o);
+      for (int j = NJ - 1; j >= 0; --j) {     // the lowest index that has it
+        const unsigned long long who = __ballot(c[j] == v);
+        if (who != 0) at = min(j * WAVE + __builtin_ctzll(who), m.n - 1);
       }
-      at = min(at, m.n - 1);                  // whatever the scores are
 #pragma unroll
       for (int j = 0; j < NJ; ++j)
         if (j * WAVE + lane == at) c[j] = -INFINITY;
@@ -131,7 +124,7 @@ __global__ __launch_bounds__(NT) void route_kernel(Route m) {
     }
   }
   __syncthreads();
-  for (int e = threadIdx.x; e < m.E; e += NT)
+  for (int e = threadIdx.x; e < m.E; e += blockDim.x)
     m.hist[(int64_t)blockIdx.x * m.E + e] = count[e];
 }
 
@@ -145,24 +138,28 @@ struct Place {
 
 __global__ __launch_bounds__(NT) void place_kernel(Place m) {
   __shared__ int at[MAX_OUTPUTS];             // this workgroup's first rows
+  __shared__ int rows_of[MAX_OUTPUTS];
   __shared__ int sums[2][NW];
   const int tid = threadIdx.x, wid = tid / WAVE, lane = tid & (WAVE - 1);
+  for (int e = tid; e < MAX_OUTPUTS; e += NT) at[e] = rows_of[e] = 0;
+  __syncthreads();
+  const int mine = blockIdx.x * m.E;
+#pragma unroll 8
+  for (int i = tid; i < m.blocks * m.E; i += NT) {
+    const int c = m.hist[i], e = i % m.E;
+    if (c != 0) {
+      atomicAdd(rows_of + e, c);
+      if (i < mine) atomicAdd(at + e, c);
+    }
+  }
+  __syncthreads();
   // thread t has experts t PER ..
   int total[PER], rows = 0, tiles = 0;
 #pragma unroll
   for (int i = 0; i < PER; ++i) {
-    const int e = tid * PER + i;
-    int all = 0, before = 0;
-    if (e < m.E)
-      for (int b = 0; b < m.blocks; ++b) {
-        const int c = m.hist[(int64_t)b * m.E + e];
-        all += c;
-        before += b < (int)blockIdx.x ? c : 0;
-      }
-    total[i] = all;
-    at[e] = before;
-    rows += all;
-    tiles += (all + m.height - 1) / m.height;
+    total[i] = rows_of[tid * PER + i];
+    rows += total[i];
+    tiles += (total[i] + m.height - 1) / m.height;
   }
   int r = rows, q = tiles;                    // running sums over threads
 #pragma unroll
@@ -260,10 +257,12 @@ void route(torch::Tensor ids, torch::Tensor weights, torch::Tensor rank,
   m.z_stride = z.stride(0);
   m.correction = correction.data_ptr<float>();
   if (m.T == 0) return;
-  const int lds = (2 * NW * m.n + NW * m.groups + m.E) * 4;
+  const int threads = per >= 16 && m.n <= 256 ? MANY : NT;
+  const int nw = threads / WAVE;
+  const int lds = (2 * nw * m.n + nw * m.groups + m.E) * 4;
   const int nj = cdiv(m.n, WAVE);
 #define HELIX_ROUTE(NJ)                                                      \
-  hipLaunchKernelGGL(route_kernel<NJ>, dim3(blocks), dim3(NT), lds,          \
+  hipLaunchKernelGGL(route_kernel<NJ>, dim3(blocks), dim3(threads), lds,     \
                      at::hip::getCurrentHIPStream(), m)
   if (nj <= 1) HELIX_ROUTE(1);
   else if (nj <= 2) HELIX_ROUTE(2);

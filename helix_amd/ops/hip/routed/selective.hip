@@ -9,8 +9,8 @@
 // own, since projections of its result come in between.
 //
 // State is [slots, N, C]: neighbouring lanes have neighbouring channels, B
-// and C of a token are the same for all of them. A is kept as [N, C] times
-// log2(e).
+// and C of a token are the same for all of them and come by scalar loads. A
+// is kept as [N, C] times log2(e).
 //
 // Prompts: one wave per 64 channels and sequence where that fills the chip.
 // Where it does not, sequences are cut into chunks: every chunk's scan from
@@ -207,18 +207,17 @@ __global__ __launch_bounds__(CT) void scan_step_kernel(
 
 constexpr int ST = 64;                        // channels of a workgroup
 constexpr int TT = 8;                         // tokens loaded at a time
-constexpr int BT = 32;                        // tokens whose B, C wait in LDS
+typedef const __attribute__((address_space(4))) float* uniform_f32;
 
 enum Pass { WHOLE, LOCAL, FINAL };
 
-// NS: states in registers (N <= NS). WHOLE: sequences from their slots'
+// NS: states in registers (N <= NS; B and C are zero from N to NS). WHOLE: sequences from their slots'
 // state and back. LOCAL: chunks from zero, only the state they end with.
 // FINAL: chunks from their entry state, only results.
 template <typename S, int NS, int PASS>
 __global__ __launch_bounds__(ST) void scan_kernel(
     S* __restrict__ y, const S* __restrict__ x, const S* __restrict__ z,
     Scan m) {
-  __shared__ __attribute__((aligned(16))) float bcs[BT][2 * NS];
   const int u = blockIdx.y, lane = threadIdx.x;
   const int c0 = blockIdx.x * ST, c = min(c0 + lane, m.C - 1);
   const bool mine = c0 + lane < m.C;
@@ -261,48 +260,59 @@ __global__ __launch_bounds__(ST) void scan_kernel(
       if constexpr (PASS != LOCAL) zr[i] = zp[r * m.z_stride];
     }
   };
-  load(0);
-  for (int t0 = 0; t0 < len; t0 += BT) {
-    __syncthreads();
-    for (int i = lane; i < BT * 2 * NS; i += ST) {
-      const int t = i / (2 * NS), k = i % (2 * NS), n = k % NS;
-      const float* r = m.bc + (int64_t)(row0 + min(t0 + t, len - 1)) *
-                                  m.bc_stride;
-      bcs[t][k] = n < m.N ? r[(k < NS ? m.b_at : m.c_at) + n] : 0.f;
+  // uniform: scalar registers
+  constexpr bool AHEAD = NS <= 16;
+  float b[NS], c_[NS], nb[NS], nc[NS];
+  auto fetch = [&](int t, float* bn, float* cn) {
+    const uniform_f32 r = (uniform_f32)(uintptr_t)(
+        m.bc + (int64_t)(row0 + min(t, len - 1)) * m.bc_stride);
+#pragma unroll
+    for (int n = 0; n < NS; ++n) {
+      bn[n] = r[m.b_at + n];
+      if constexpr (PASS != LOCAL) cn[n] = r[m.c_at + n];
     }
-    __syncthreads();
-    for (int t = t0; t < min(len, t0 + BT); t += TT) {
-      float xv[TT], dv[TT], zv[TT];
+  };
+  load(0);
+  if constexpr (AHEAD) fetch(0, b, c_);
+  for (int t = 0; t < len; t += TT) {
+    float xv[TT], dv[TT], zv[TT];
 #pragma unroll
-      for (int i = 0; i < TT; ++i) {
-        // past the end: a step of size zero changes nothing
-        dv[i] = t + i < len ? softplus_of<S>(dr[i] + bias) : 0.f;
-        xv[i] = ld1(&xr[i]);
-        if constexpr (PASS != LOCAL) zv[i] = ld1(&zr[i]);
+    for (int i = 0; i < TT; ++i) {
+      // past the end: a step of size zero changes nothing
+      dv[i] = t + i < len ? softplus_of<S>(dr[i] + bias) : 0.f;
+      xv[i] = ld1(&xr[i]);
+      if constexpr (PASS != LOCAL) zv[i] = ld1(&zr[i]);
+    }
+    if (t + TT < len) load(t + TT);
+#pragma unroll
+    for (int i = 0; i < TT; ++i) {
+      if constexpr (AHEAD) {
+        // a token's B and C are on their way while the one before it is
+        // worked on; nothing moves across the fences
+        fetch(t + i + 1, nb, nc);
+        __builtin_amdgcn_sched_barrier(0);
+      } else {
+        fetch(t + i, b, c_);
       }
-      if (t + TT < len) load(t + TT);
+      const float w = dv[i] * xv[i];
+      if constexpr (PASS == LOCAL) total += dv[i];
+      float acc[4] = {D * xv[i], 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int i = 0; i < TT; ++i) {
-        const float *B = bcs[t - t0 + i], *Cc = B + NS;
-        const float w = dv[i] * xv[i];
-        if constexpr (PASS == LOCAL) total += dv[i];
-        float acc[4] = {D * xv[i], 0.f, 0.f, 0.f};
+      for (int n = 0; n < NS; ++n) {
+        s[n] = exp2_(dv[i] * a[n]) * s[n] + w * b[n];
+        if constexpr (PASS != LOCAL) acc[n & 3] += s[n] * c_[n];
+      }
+      if constexpr (PASS != LOCAL) {
+        const float o = (acc[0] + acc[1]) + (acc[2] + acc[3]);
+        if (mine && t + i < len)
+          st1(yp + (int64_t)(t + i) * m.y_stride, o * silu_s<S>(zv[i]));
+      }
+      if constexpr (AHEAD) {
+        __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-        for (int n = 0; n < NS; n += 4) {
-          const f32x4 bv = *reinterpret_cast<const f32x4*>(B + n);
-          f32x4 cv;
-          if constexpr (PASS != LOCAL)
-            cv = *reinterpret_cast<const f32x4*>(Cc + n);
-#pragma unroll
-          for (int j = 0; j < 4; ++j) {
-            s[n + j] = exp2_(dv[i] * a[n + j]) * s[n + j] + w * bv[j];
-            if constexpr (PASS != LOCAL) acc[j] += s[n + j] * cv[j];
-          }
-        }
-        if constexpr (PASS != LOCAL) {
-          const float o = (acc[0] + acc[1]) + (acc[2] + acc[3]);
-          if (mine && t + i < len)
-            st1(yp + (int64_t)(t + i) * m.y_stride, o * silu_s<S>(zv[i]));
+        for (int n = 0; n < NS; ++n) {
+          b[n] = nb[n];
+          c_[n] = nc[n];
         }
       }
     }
@@ -393,6 +403,13 @@ Scan arguments(const torch::Tensor& y, const torch::Tensor& x,
   return m;
 }
 
+// Columns that B and C take in a row.
+int columns_of(int N) {
+  int n = 8;
+  while (n < N) n *= 2;
+  return n;
+}
+
 template <int PASS>
 void launch_scan(torch::Tensor y, torch::Tensor x, torch::Tensor z, Scan m,
                  int units) {
@@ -418,7 +435,10 @@ void launch_scan(torch::Tensor y, torch::Tensor x, torch::Tensor z, Scan m,
 
 }  // namespace
 
+// Most states per channel, and the columns that N take in B's and C's rows
+// (zero from N on).
 int64_t scan_max_state() { return 128; }
+int64_t scan_columns(int64_t N) { return columns_of(N); }
 
 // out [T, C] <- silu of the causal convolution of z's columns x_at ..; conv
 // [taps, C]. z rows: one token of sequence r each, or (with cu) the
@@ -516,6 +536,10 @@ void scan_prompt(torch::Tensor y, torch::Tensor x, torch::Tensor z,
   const int B = slots.numel();
   check_rows(slots, pos, B, x.size(0));
   TORCH_CHECK(m.N <= scan_max_state(), "state size ", m.N);
+  const int64_t cols = columns_of(m.N);
+  TORCH_CHECK(b_at + cols <= bc.size(1) && c_at + cols <= bc.size(1) &&
+                  std::abs(b_at - c_at) >= cols,
+              "B and C take ", cols, " columns each");
   TORCH_CHECK(x.scalar_type() == torch::kBFloat16 ||
               x.scalar_type() == torch::kFloat32);
   m.slots = slots.data_ptr<int>();

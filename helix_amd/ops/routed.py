@@ -144,29 +144,29 @@ class ExpertLists(NamedTuple):
     slot: torch.Tensor           # [T, top] int32 row, -1: identity
     tiles: torch.Tensor          # [n, 4] int32 expert, first row, rows
     height: int                  # rows of a tile at most
-    plain: bool                  # which kernel family
+    kind: str                    # kernel family: stream, tile or plain
 
 
-# Rows per expert from which tiles through LDS beat streamed weights.
-TILE_ROWS = 48
+# Height of a tile by the rows an expert has on average (the weights are the
+# traffic until there are hundreds).
+TILE_HEIGHTS = ((4, 32), (12, 128), (384, 256))
 
 
 def tile_height(rows: int, p: RouterParams, a: torch.Tensor,
                 ups: torch.Tensor, downs: torch.Tensor):
-    """(rows of a tile, plain kernel) for `rows` (token, choice) pairs."""
+    """(rows of a tile, kernel family) for `rows` (token, choice) pairs."""
     C = _native()
     if not (C.experts_fit(a, ups) and downs.shape[2] % 8 == 0):
-        return 32, True
+        return 32, "plain"
     each = rows / p.outputs
-    if each >= TILE_ROWS and ups.shape[2] % 64 == 0 and \
-            downs.shape[2] % 64 == 0:
-        return C.expert_tile_rows(), False
-    # the fullest expert has more than the mean
-    return (16 if each <= 8 else 32 if each <= 20 else 64), False
+    if each < TILE_HEIGHTS[0][0] or ups.shape[2] % 64 or \
+            downs.shape[2] % 64:
+        return 32 if each < 16 else 64, "stream"
+    return [h for n, h in TILE_HEIGHTS if each >= n][-1], "tile"
 
 
 def expert_lists(ids, rank, hist, p: RouterParams, height: int,
-                 plain: bool) -> ExpertLists:
+                 kind: str) -> ExpertLists:
     T, dev = ids.shape[0], ids.device
     P = T * p.top
     order = torch.empty(P, dtype=torch.int32, device=dev)
@@ -175,7 +175,7 @@ def expert_lists(ids, rank, hist, p: RouterParams, height: int,
                         dtype=torch.int32, device=dev)
     _native().place(order, slot, tiles, ids, rank, hist,
                     _tokens_per_group(T), height)
-    return ExpertLists(order, slot, tiles, height, plain)
+    return ExpertLists(order, slot, tiles, height, kind)
 
 
 def expert_products(h: torch.Tensor, ups: torch.Tensor, downs: torch.Tensor,
@@ -188,11 +188,11 @@ def expert_products(h: torch.Tensor, ups: torch.Tensor, downs: torch.Tensor,
 
     def up():
         C.expert_product(act, h, ups, lists.tiles, lists.order, top,
-                         lists.height, True, lists.plain)
+                         lists.height, lists.kind, True)
 
     def down():
         C.expert_product(rows, act, downs, lists.tiles, None, 1,
-                         lists.height, False, lists.plain)
+                         lists.height, lists.kind, False)
 
     return (up, down), rows
 
@@ -229,6 +229,16 @@ class ScanParams:
     b_at: int
     c_at: int
 
+    @property
+    def columns(self) -> int:
+        return self.c_at + state_columns(self.state)
+
+
+def state_columns(state: int) -> int:
+    """Columns that B and C take each: the registers of a scan (zero past
+    the state size)."""
+    return max(8, 1 << (state - 1).bit_length())
+
 
 class ScanWeights(NamedTuple):
     """conv [taps, inner], conv_b and D [inner], A [state, inner] (times
@@ -243,14 +253,15 @@ class ScanWeights(NamedTuple):
     D: torch.Tensor
 
 
-# Waves that should be under way before a scan's chunks get longer.
-SCAN_WAVES = 2048
+# Waves that carry whole sequences without a chip half empty, and waves of
+# chunks where there are fewer.
+SCAN_WHOLE, SCAN_WAVES = 2048, 8192
 
 
 def scan_chunk(inner: int, rows: int, seqs: int) -> int:
     """Tokens of a chunk, 0: sequences as a whole fill the chip."""
     waves = -(-inner // 64)
-    if waves * seqs >= SCAN_WAVES // 2 or rows < 128 * seqs:
+    if waves * seqs >= SCAN_WHOLE or rows < 128 * seqs:
         return 0
     return max(64, -(-rows * waves // SCAN_WAVES // 32) * 32)
 

@@ -196,10 +196,11 @@ def mixture_case(W, F, p, T, dtype, seed=0):
     (20, 28, ROUTERS[2], 9),
     (8, 8, ROUTERS[3], 3),
     (64, 64, ROUTERS[4], 1),
-    (192, 96, ROUTERS[0], 60),                 # 32 rows a tile
-    (128, 160, ROUTERS[2], 30),                # 64 rows a tile
-    (128, 192, ROUTERS[1], 420),               # tiles through LDS
-    (64, 320, ROUTERS[7], 200),
+    (192, 96, ROUTERS[0], 60),                 # streams of few rows, of many
+    (136, 160, ROUTERS[2], 70),
+    (64, 192, ROUTERS[0], 25),                 # tiles of 32, 128, 256 rows
+    (128, 192, ROUTERS[1], 420),
+    (64, 320, ROUTERS[7], 600),
     (320, 64, ROUTERS[3], 129),
     (64, 72, ROUTERS[6], 130),                 # most experts have few rows
 ])
@@ -233,7 +234,7 @@ def test_expert_lists(T, p, height):
     z = rnd(gen(T), T, p.outputs, std=2.0).float().cuda()
     corr = torch.zeros(p.outputs, device="cuda")
     ids, _, rank, hist = routed._route(z, corr, p)
-    l = routed.expert_lists(ids, rank, hist, p, height, False)
+    l = routed.expert_lists(ids, rank, hist, p, height, "tile")
     ids, slot = ids.cpu().flatten(), l.slot.cpu().flatten()
     order, tiles = l.order.cpu(), l.tiles.cpu().tolist()
     real = (ids < p.experts).nonzero().flatten()
@@ -609,9 +610,11 @@ def test_scan_in_chunks(dtype, inner, state):
         None, None, None, None, put(rnd(g, inner, std=2.0) - 4.0),
         put(-torch.exp(rnd(g, state, inner)) * math.log2(math.e)),
         put(rnd(g, inner)))
-    p = routed.ScanParams(inner, state, 4, 1, 0, 0, 8, 8 + state)
+    at = 8 + routed.state_columns(state)
+    p = routed.ScanParams(inner, state, 4, 1, 0, 0, 8, at)
     x, z = (put(rnd(g, T, inner), dtype) for _ in range(2))
-    dt, bc = put(rnd(g, T, inner, std=3.0)), put(rnd(g, T, 8 + 2 * state))
+    dt, bc = put(rnd(g, T, inner, std=3.0)), put(rnd(g, T, p.columns))
+    bc[:, 8 + state:at] = bc[:, at + state:] = 0
     cu = np.concatenate([[0], np.cumsum(lens)])
     meta = prompt_meta([(0, 413), (50, 51), (7, 293)],
                        np.zeros((3, 60), int), 8, "cuda", [2, 0, 1])
@@ -626,7 +629,7 @@ def test_scan_in_chunks(dtype, inner, state):
         for t, (xt, dd, q) in enumerate(zip(x[s].double().cpu(), d,
                                             bc[s].double().cpu())):
             S = torch.exp(dd * A) * S + (dd * xt) * q[8:8 + state, None]
-            want[int(cu[b]) + t] = (S * q[8 + state:, None]).sum(0) \
+            want[int(cu[b]) + t] = (S * q[at:at + state, None]).sum(0) \
                 + w.D.double().cpu() * xt
         states.append(S)
     want = want * do.silu(z.double().cpu())
