@@ -167,8 +167,7 @@ def kernels(z: DibizenConfig, device, decode_batch: int = 256,
         bc = rand(T, sw.x.shape[0], dtype=torch.float32)
         t = _time(lambda: routed.scan_prompt(y, x, zz, sp, sw, state, raw, bc,
                                              meta), reps=5)
-        # x, z, y and the step sizes; an exponential is a quarter-rate
-        # instruction, the rest of a state's update four full-rate ones
+        # x, z, y and the step sizes
         pair("scan" + tag, _row(t, T * I * 10.0), like)
         del zz, y, x, raw, bc
 
@@ -241,14 +240,12 @@ def kernels(z: DibizenConfig, device, decode_batch: int = 256,
         pair(f"experts_down_t{T}", _row(
             _time(steps[1], reps=10), wbytes + 2.0 * n * (W + F), flops), like)
         del a, b
-        gu = rand(T, 2 * twin_ff)
-        act = _row(_time(lambda: ops.silu_and_mul(gu)),
-                   2.0 * T * 3 * twin_ff)
-        del gu
+        # a dense model has nothing like these
         t = _time(lambda: routed._route(logits, moe.correction, r))
-        pair(f"route_t{T}", _row(t, 4.0 * T * (r.outputs + 3 * r.top)), act)
+        out[f"route_t{T}"] = {
+            "new": _row(t, 4.0 * T * (r.outputs + 3 * r.top))}
         t = _time(lambda: routed.expert_lists(ids, rank, hist, r, *height))
-        pair(f"place_t{T}", _row(t, 4.0 * T * r.top * 4), act)
+        out[f"place_t{T}"] = {"new": _row(t, 4.0 * T * r.top * 4)}
 
         # --- streams
         x, y = rand(T, S, W, dtype=torch.float32), rand(T, W)

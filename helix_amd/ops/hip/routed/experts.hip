@@ -148,6 +148,8 @@ __global__ __launch_bounds__(NT) void expert_rows_kernel(
 // steps of 64 (K % 64 == 0). The next step's tiles are on their way to one
 // half of LDS while the other is worked on.
 constexpr int BK = 64;
+// instruction classes of the scheduling hints
+constexpr int MFMA = 0x008, DS_READ = 0x100;
 
 template <int BM, int BN, int WM, int WN>
 __global__ __launch_bounds__(WM* WN* WAVE) void expert_tiles_kernel(
@@ -223,6 +225,16 @@ __global__ __launch_bounds__(WM* WN* WAVE) void expert_tiles_kernel(
 #pragma unroll
         for (int i = 0; i < MI; ++i)
           acc[j][i] = mfma16(wf[j], af[i], acc[j][i]);
+    }
+    if constexpr (MI * NI == 32) {
+      // the second half's operands leave LDS between the first products
+      __builtin_amdgcn_sched_group_barrier(DS_READ, MI + NI, 0);
+#pragma unroll
+      for (int i = 0; i < MI + NI; ++i) {
+        __builtin_amdgcn_sched_group_barrier(MFMA, 2, 0);
+        __builtin_amdgcn_sched_group_barrier(DS_READ, 1, 0);
+      }
+      __builtin_amdgcn_sched_group_barrier(MFMA, 64 - 2 * (MI + NI), 0);
     }
   }
   // lane: columns 4 hi + r of row lo

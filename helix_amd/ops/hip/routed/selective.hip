@@ -206,7 +206,7 @@ __global__ __launch_bounds__(CT) void scan_step_kernel(
 }
 
 constexpr int ST = 64;                        // channels of a workgroup
-constexpr int TT = 8;                         // tokens loaded at a time
+constexpr int TT = 4;                         // tokens loaded at a time
 typedef const __attribute__((address_space(4))) float* uniform_f32;
 
 enum Pass { WHOLE, LOCAL, FINAL };

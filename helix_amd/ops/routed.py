@@ -253,9 +253,9 @@ class ScanWeights(NamedTuple):
     D: torch.Tensor
 
 
-# Waves that carry whole sequences without a chip half empty, and waves of
-# chunks where there are fewer.
-SCAN_WHOLE, SCAN_WAVES = 2048, 8192
+# Waves from which whole sequences keep the chip busy; below, chunks of at
+# most SCAN_CHUNK tokens, for SCAN_WAVES waves.
+SCAN_WHOLE, SCAN_WAVES, SCAN_CHUNK = 2048, 4096, 256
 
 
 def scan_chunk(inner: int, rows: int, seqs: int) -> int:
@@ -263,7 +263,8 @@ def scan_chunk(inner: int, rows: int, seqs: int) -> int:
     waves = -(-inner // 64)
     if waves * seqs >= SCAN_WHOLE or rows < 128 * seqs:
         return 0
-    return max(64, -(-rows * waves // SCAN_WAVES // 32) * 32)
+    return min(SCAN_CHUNK,
+               max(64, -(-rows * waves // SCAN_WAVES // 32) * 32))
 
 
 def conv_silu(z: torch.Tensor, p: ScanParams, w: ScanWeights, ring, slots,
