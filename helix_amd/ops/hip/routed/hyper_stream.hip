@@ -90,11 +90,11 @@ __global__ __launch_bounds__(NT) void hyper_stream_kernel(
         const int at = m.slot[t * m.K + k];
         const float g = m.weight[t * m.K + k];
         float e[N];
+        // row 0 may never have been written: selected, not multiplied by 0
         get<S, N>(y + (int64_t)max(at, 0) * m.W + d, e);
-        const float f = at < 0 ? 0.f : g;
         self += at < 0 ? g : 0.f;
 #pragma unroll
-        for (int j = 0; j < N; ++j) r[j] += f * e[j];
+        for (int j = 0; j < N; ++j) r[j] += at < 0 ? 0.f : g * e[j];
       }
       if (self != 0.f) {
         float e[N];

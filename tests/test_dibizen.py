@@ -86,10 +86,11 @@ def test_streams(dev, dtype, T, S, W):
     close(xd, want, F32)
     close(tap, want.sum(1), F32)
     close(h, h_want, dtype)
-    # a mixture's rows: two experts, one identity
+    # a mixture's rows: two experts, one identity; row 0 is nobody's
     K = 3
-    rows, self = rnd(g, T * K, W, dtype=dtype), rnd(g, T, W, dtype=dtype)
-    slot = torch.randperm(T * K, generator=g).int().view(T, K)
+    rows, self = rnd(g, T * K + 1, W, dtype=dtype), rnd(g, T, W, dtype=dtype)
+    rows[0] = float("nan")
+    slot = 1 + torch.randperm(T * K, generator=g).int().view(T, K)
     slot[:, 1] = -1
     wt = rnd(g, T, K)
     y = sum(wt[:, k, None] * (self if k == 1 else rows[slot[:, k].long()])
@@ -223,6 +224,30 @@ def test_mixture(dev, dtype, W, F, p, T):
                                                torch.zeros(W, device=dev)))
     want = do.mixture(h, w, "", {"router": r})
     close_rows(streams[:, 0], want, dtype, float(want.pow(2).mean().sqrt()))
+
+
+@pytest.mark.parametrize("dev", DEVICES)
+@pytest.mark.parametrize("dtype", [F32, BF16])
+@pytest.mark.parametrize("T", [1, 9])
+def test_identity_experts_alone(dev, dtype, T):
+    """No expert with weights is chosen, so no row of theirs is written, and
+    what lies in that memory must not show."""
+    W, p = 48, RouterParams(4, 2, 4, 2, 1)
+    w, h = mixture_case(W, 16, p, T, dtype)
+    w["correction"][4:] = 3.0
+    mod = Mixture(MixtureSpec(16, p), W).to(dtype)
+    with torch.inference_mode():
+        for n, t in mod.targets("").items():
+            t.copy_(w[n].to(t.dtype))
+        mod = mod.to(dev)
+        out = mod(on(dev, h, dtype))
+        assert (out.slot == -1).all()
+        out.rows.fill_(float("nan"))
+        x, one = torch.zeros(T, 1, W, device=dev), torch.ones(1, device=dev)
+        routed.hyper_step(x, out, routed.Return(one.view(1, 1), one), one,
+                          routed.TanhNorm(one, torch.ones(W, device=dev),
+                                          torch.zeros(W, device=dev)))
+    close(x[:, 0], h, F32)
 
 
 @pytest.mark.gpu
